@@ -4,6 +4,7 @@
 // of c vectors that W_uv_h turns into the head's values afterwards.  The attention kernels are the
 // grouped-query ones with one KV head.
 //
+//  * yalm_latent_norm: the RMS norm of a latent vector that is a part of a wider product (the queries' one).
 //  * yalm_latent_pack: per token, the RMS norm of the down projection's first `rank` columns, and the
 //    head-shaped rows that the rotation kernel reads (query rotated parts scaled, key, value).
 //  * yalm_head_matmul: out[t, h, :] = scale * in[t, h, :] Wt[h] for every head, Wt [H, K, N]
@@ -92,24 +93,39 @@ __global__ __launch_bounds__(HM_THREADS) void head_matmul_kernel(const TI* __res
   }
 }
 
+// out[r, :n] = x[r, :n] / sqrt(mean over those n of x^2 + eps) * w, the rows of x `x_row` apart: the norm of a latent
+// vector that is a part of a wider product.  A wave a row.
+template <typename TW, typename TO>
+__global__ __launch_bounds__(4 * WAVE) void latent_norm_kernel(const float* __restrict__ x, long x_row, const TW* __restrict__ w,
+                                                               float eps, TO* __restrict__ out, int R, int n) {
+  const int r = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  if (r >= R) return;
+  const float* row = x + (size_t)r * x_row;
+  float ss = 0.f;
+  for (int i = lane; i < n; i += WAVE) ss = fmaf(row[i], row[i], ss);
+  const float s = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
+  for (int i = lane; i < n; i += WAVE) out[(size_t)r * n + i] = from_f32<TO>(row[i] * s * to_f32(w[i]));
+}
+
 // One wave a (token, job).  job < H: the rotated part of query head `job`, scaled, and zeros behind the
 // latent part; job == H (has_kv only): the key and value rows.
 template <typename TN>
-__global__ __launch_bounds__(WAVE) void latent_pack_kernel(const float* __restrict__ proj, long proj_row, int q_head,
-                                                           int q_rot_off, int kv_off, const TN* __restrict__ norm_w, float eps,
+__global__ __launch_bounds__(WAVE) void latent_pack_kernel(const float* __restrict__ queries, long q_row, int q_head,
+                                                           int q_rot_off, const float* __restrict__ kv, long kv_row, int kv_off,
+                                                           const TN* __restrict__ norm_w, float eps,
                                                            float q_scale, float* __restrict__ out, int H, int rot, int rank,
                                                            int Dk, int has_kv) {
   const int t = blockIdx.x, job = blockIdx.y, lane = threadIdx.x;
-  const float* row = proj + (size_t)t * proj_row;
   float* dst = out + (size_t)t * (H + 2) * Dk;
   if (job < H) {
+    const float* row = queries + (size_t)t * q_row;
     float* q = dst + (size_t)job * Dk;
     for (int i = lane; i < rot; i += WAVE) q[i] = row[(size_t)job * q_head + q_rot_off + i] * q_scale;
     for (int i = rot + rank + lane; i < Dk; i += WAVE) q[i] = 0.f;
     return;
   }
   if (!has_kv) return;
-  const float* d = row + kv_off;
+  const float* d = kv + (size_t)t * kv_row + kv_off;
   float ss = 0.f;
   for (int i = lane; i < rank; i += WAVE) ss += d[i] * d[i];
   ss = wave_sum(ss);
@@ -299,20 +315,36 @@ extern "C" int yalm_head_matmul_mfma(const void* in, int in_dtype, long in_row, 
   return launch_status();
 }
 
-extern "C" int yalm_latent_pack(const float* proj, long proj_row, int q_head, int q_rot_off, int kv_off,
-                                const void* norm_w, int norm_dtype, float eps, float q_scale, float* out, int T, int H,
+extern "C" int yalm_latent_norm(const float* x, long x_row, const void* w, int w_dtype, float eps, void* out, int out_dtype,
+                                int R, int n, hipStream_t stream) {
+  if (R <= 0) return YALM_OK;
+  if (n <= 0 || x_row < n) return YALM_ERR_ARG;
+  const int blocks = ceil_div(R, 4);
+#define LN(TW_, TO_) latent_norm_kernel<TW_, TO_><<<blocks, 4 * WAVE, 0, stream>>>(x, x_row, (const TW_*)w, eps, (TO_*)out, R, n)
+  if (w_dtype == YALM_F32 && out_dtype == YALM_F32) LN(float, float);
+  else if (w_dtype == YALM_F32 && out_dtype == YALM_BF16) LN(float, bf16);
+  else if (w_dtype == YALM_BF16 && out_dtype == YALM_F32) LN(bf16, float);
+  else if (w_dtype == YALM_BF16 && out_dtype == YALM_BF16) LN(bf16, bf16);
+  else return YALM_ERR_DTYPE;
+#undef LN
+  return launch_status();
+}
+
+extern "C" int yalm_latent_pack(const float* queries, long q_row, int q_head, int q_rot_off, const float* kv, long kv_row,
+                                int kv_off, const void* norm_w, int norm_dtype, float eps, float q_scale, float* out, int T, int H,
                                 int rot, int rank, int Dk, int has_kv, hipStream_t stream) {
   if (T <= 0) return YALM_OK;
   if (H <= 0 || rot < 0 || rank <= 0 || Dk < rot + rank || q_rot_off < 0 || q_rot_off + rot > q_head ||
-      (long)H * q_head > proj_row || (has_kv && (norm_w == nullptr || kv_off < 0 || (long)kv_off + rank + rot > proj_row)))
+      (long)H * q_head > q_row ||
+      (has_kv && (norm_w == nullptr || kv == nullptr || kv_off < 0 || (long)kv_off + rank + rot > kv_row)))
     return YALM_ERR_ARG;
   dim3 grid(T, H + 1);
   if (norm_dtype == YALM_BF16)
-    latent_pack_kernel<bf16><<<grid, WAVE, 0, stream>>>(proj, proj_row, q_head, q_rot_off, kv_off, (const bf16*)norm_w, eps,
-                                                        q_scale, out, H, rot, rank, Dk, has_kv);
+    latent_pack_kernel<bf16><<<grid, WAVE, 0, stream>>>(queries, q_row, q_head, q_rot_off, kv, kv_row, kv_off,
+                                                        (const bf16*)norm_w, eps, q_scale, out, H, rot, rank, Dk, has_kv);
   else if (norm_dtype == YALM_F32)
-    latent_pack_kernel<float><<<grid, WAVE, 0, stream>>>(proj, proj_row, q_head, q_rot_off, kv_off, (const float*)norm_w,
-                                                         eps, q_scale, out, H, rot, rank, Dk, has_kv);
+    latent_pack_kernel<float><<<grid, WAVE, 0, stream>>>(queries, q_row, q_head, q_rot_off, kv, kv_row, kv_off,
+                                                         (const float*)norm_w, eps, q_scale, out, H, rot, rank, Dk, has_kv);
   else
     return YALM_ERR_DTYPE;
   return launch_status();

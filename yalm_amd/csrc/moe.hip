@@ -2,12 +2,12 @@
 //
 //  * yalm_moe_route: per token, logits = W_router h in float32, scores = softmax over all experts, the
 //    `top` largest (the lowest index on ties), with their scores as weights (optionally renormalised
-//    to sum 1).  One wave a token.
+//    to sum 1).  One wave a token.  yalm_moe_select_groups: sigmoid scores, choice inside the best groups.
 //  * yalm_moe_pair_gate_up / yalm_moe_pair_down: every pair reads its expert's weights: a wave per output
 //    row, the lanes along K with 16-byte loads.  What a decode step needs (few pairs, each bound by
 //    the one pass over its expert), and correct for any number of tokens.
 //    Expert unit: g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit), mid = g sigmoid(alpha g) (u + 1)
-//    (limit <= 0: no clamping); out[t] (+)= sum over the token's choices, in order, of weight * W_down mid.
+//    (limit <= 0: no clamping); or without a gate matrix mid = relu(W_up h)^2; out[t] (+)= sum over the token's choices, in order, of weight * W_down mid.
 #include "common.h"
 #include "yalm_hip.h"
 
@@ -124,7 +124,85 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const T* __restrict__ h
     for (int k = lane; k < top; k += WAVE) wts[(size_t)t * top + k] /= total;
 }
 
-template <typename T>
+// Sigmoid scores and choice inside the best groups: s = sigmoid(logit), c = s + correction; experts e of neighbours form
+// n_groups equal groups, a group's score is the sum of its two largest c, the `keep` best groups stay (the others'
+// c counts as minus infinity), the `top` largest c are chosen, and their weights are s / (sum of the chosen s + 1e-20) *
+// scale.  One wave a token; ties go to the lower index.
+__global__ __launch_bounds__(WAVE) void moe_select_groups_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
+                                                                 int* __restrict__ ids, float* __restrict__ wts, int E, int top,
+                                                                 int n_groups, int keep, float scale) {
+  __shared__ float score[MOE_MAX_EXPERTS];        // s
+  __shared__ float choice[MOE_MAX_EXPERTS];       // c
+  __shared__ float group[MOE_MAX_EXPERTS];
+  const int t = blockIdx.x, lane = threadIdx.x, per = E / n_groups;
+  for (int e = lane; e < E; e += WAVE) {
+    const float s = 1.0f / (1.0f + expf(-logits[(size_t)t * E + e]));
+    score[e] = s;
+    choice[e] = s + (correction != nullptr ? correction[e] : 0.f);
+  }
+  __syncthreads();
+  // the largest of v[0 .. n) over the wave: every lane gets value and place
+  auto largest = [&](const float* v, int n, int& at) {
+    float best = -INFINITY;
+    at = 0x7fffffff;
+    for (int e = lane; e < n; e += WAVE) {
+      const float x = v[e];
+      if (x > best) { best = x; at = e; }
+    }
+    for (int o = WAVE / 2; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, WAVE);
+      const int oa = __shfl_xor(at, o, WAVE);
+      if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+    }
+    if (at == 0x7fffffff) at = 0;                 // nothing finite is left
+  };
+  if (keep < n_groups) {
+    for (int g = lane; g < n_groups; g += WAVE) {
+      float a = -INFINITY, b = -INFINITY;
+      for (int e = g * per; e < (g + 1) * per; ++e) {
+        const float x = choice[e];
+        if (x > a) { b = a; a = x; } else if (x > b) { b = x; }
+      }
+      group[g] = per > 1 ? a + b : a;
+    }
+    __syncthreads();
+    // the kept groups are marked by plus infinity one after another, the others' experts then drop out
+    for (int k = 0; k < keep; ++k) {
+      float best = -INFINITY;
+      int at = 0x7fffffff;
+      for (int g = lane; g < n_groups; g += WAVE) {
+        const float x = group[g];
+        if (x != INFINITY && x > best) { best = x; at = g; }
+      }
+      for (int o = WAVE / 2; o > 0; o >>= 1) {
+        const float ob = __shfl_xor(best, o, WAVE);
+        const int oa = __shfl_xor(at, o, WAVE);
+        if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+      }
+      if (lane == 0 && at < n_groups) group[at] = INFINITY;
+      __syncthreads();
+    }
+    for (int e = lane; e < E; e += WAVE)
+      if (group[e / per] != INFINITY) choice[e] = -INFINITY;
+    __syncthreads();
+  }
+  float total = 0.f;
+  for (int k = 0; k < top; ++k) {
+    int at;
+    largest(choice, E, at);
+    const float s = score[at];
+    if (lane == 0) {
+      ids[(size_t)t * top + k] = at;
+      wts[(size_t)t * top + k] = s;
+      choice[at] = -INFINITY;                     // taken
+    }
+    total += s;
+    __syncthreads();
+  }
+  for (int k = lane; k < top; k += WAVE) wts[(size_t)t * top + k] = wts[(size_t)t * top + k] / (total + 1e-20f) * scale;
+}
+
+template <typename T, bool GATED>
 __global__ __launch_bounds__(PAIR_WAVES * WAVE) void moe_pair_gate_up_kernel(const T* __restrict__ h, const T* __restrict__ w_gate,
                                                                              const T* __restrict__ w_up, const int* __restrict__ ids,
                                                                              float limit, float alpha, float up_shift, T* __restrict__ mid, int top,
@@ -137,8 +215,13 @@ __global__ __launch_bounds__(PAIR_WAVES * WAVE) void moe_pair_gate_up_kernel(con
   const int f0 = blockIdx.y * PAIR_ROWS;
   for (int f = f0 + wave; f < min(F, f0 + PAIR_ROWS); f += PAIR_WAVES) {
     const size_t r = ((size_t)e * F + f) * D;
-    float g = wave_sum(dot_row<T>(w_gate + r, x, D, lane));
     float u = wave_sum(dot_row<T>(w_up + r, x, D, lane));
+    if constexpr (!GATED) {
+      u = fmaxf(u, 0.f);
+      if (lane == 0) mid[(size_t)pair * F + f] = from_f32<T>(u * u);
+      continue;
+    }
+    float g = wave_sum(dot_row<T>(w_gate + r, x, D, lane));
     if (limit > 0.f) {
       g = fminf(g, limit);
       u = fminf(fmaxf(u, -limit), limit);
@@ -234,14 +317,17 @@ typedef __attribute__((ext_vector_type(16))) float gr_f32x16;
 // for eight matrix instructions (v_mfma_f32_32x32x16_bf16: operand rows = lane % 32, 8 k a lane at k offset
 // 8 * (lane / 32); C: column = lane % 32, rows 8 (r / 4) + 4 (lane / 32) + r % 4).  One LDS buffer, the next k tile
 // waits in registers.
-// GATED: A rows are gathered (row -> pair -> token); a wave's 128 weight rows are 64 gate rows and the 64 up rows of
-// the same hidden columns, and the epilogue writes mid[row, f] = act(g, u).  Else: A = mid rows as they lie, the
-// weight rows are 256 rows of the expert's down matrix, and the epilogue stores float32 out[row, n].
-template <bool GATED>
+// GR_GATED: A rows are gathered (row -> pair -> token); a wave's 128 weight rows are 64 gate rows and the 64 up rows of
+// the same hidden columns, and the epilogue writes mid[row, f] = act(g, u).  GR_RELU2: A rows gathered as well, the weight
+// rows are 256 up rows, the epilogue writes mid[row, f] = relu(u)^2.  GR_DOWN: A = mid rows as they lie, the weight rows
+// are 256 rows of the expert's down matrix, and the epilogue stores float32 out[row, n].
+constexpr int GR_DOWN = 0, GR_GATED = 1, GR_RELU2 = 2;
+template <int MODE>
 __global__ __launch_bounds__(GR_THREADS, 2) void moe_grouped_kernel(const bf16* __restrict__ A, const bf16* __restrict__ W0,
                                                                     const bf16* __restrict__ W1, const int* __restrict__ tile_expert,
                                                                     const int* __restrict__ pair_of_row, int top, void* __restrict__ Cv,
                                                                     int N, int K, float limit, float alpha, float up_shift) {
+  constexpr bool GATED = MODE == GR_GATED, GATHER = MODE != GR_DOWN;
   const int e = tile_expert[blockIdx.y];
   if (e < 0) return;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
@@ -263,7 +349,7 @@ __global__ __launch_bounds__(GR_THREADS, 2) void moe_grouped_kernel(const bf16* 
     const int row = m0 + lrow + RPP * p;
     const int pair = pair_of_row[row];
     aok[p] = pair >= 0;
-    ap[p] = A + (size_t)(GATED ? (aok[p] ? pair / top : 0) : row) * K + lk;
+    ap[p] = A + (size_t)(GATHER ? (aok[p] ? pair / top : 0) : row) * K + lk;
   }
 #pragma unroll
   for (int p = 0; p < LB; ++p) {
@@ -350,7 +436,13 @@ __global__ __launch_bounds__(GR_THREADS, 2) void moe_grouped_kernel(const bf16* 
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
           const int n = n0 + wn * 128 + b * 32 + li;
-          if (n < N) ((float*)Cv)[(size_t)row * N + n] = acc[a][b][r];
+          if (n >= N) continue;
+          if (MODE == GR_RELU2) {
+            const float u = fmaxf(acc[a][b][r], 0.f);
+            ((bf16*)Cv)[(size_t)row * N + n] = static_cast<bf16>(u * u);
+          } else {
+            ((float*)Cv)[(size_t)row * N + n] = acc[a][b][r];
+          }
         }
       }
     }
@@ -396,21 +488,35 @@ extern "C" int yalm_moe_select(const float* logits, const float* bias, int* ids,
   return launch_status();
 }
 
+extern "C" int yalm_moe_select_groups(const float* logits, const float* correction, int* ids, float* wts, int T, int E, int top,
+                                      int n_groups, int keep, float scale, hipStream_t stream) {
+  if (T <= 0) return YALM_OK;
+  if (E <= 0 || E > MOE_MAX_EXPERTS || n_groups <= 0 || E % n_groups || keep <= 0 || keep > n_groups || top <= 0 ||
+      top > keep * (E / n_groups))
+    return YALM_ERR_ARG;
+  moe_select_groups_kernel<<<T, WAVE, 0, stream>>>(logits, correction, ids, wts, E, top, n_groups, keep, scale);
+  return launch_status();
+}
+
 extern "C" int yalm_moe_pair_gate_up(const void* h, const void* w_gate, const void* w_up, const int* ids, float limit,
                                      float alpha, float up_shift, void* mid, int T, int top, int D, int F, int E, int dtype,
                                      hipStream_t stream) {
   if (T <= 0) return YALM_OK;
   if (D <= 0 || F <= 0 || E <= 0 || top <= 0) return YALM_ERR_ARG;
   dim3 grid(T * top, ceil_div(F, PAIR_ROWS));
-  if (dtype == YALM_BF16)
-    moe_pair_gate_up_kernel<bf16><<<grid, PAIR_WAVES * WAVE, 0, stream>>>((const bf16*)h, (const bf16*)w_gate, (const bf16*)w_up,
-                                                                          ids, limit, alpha, up_shift, (bf16*)mid, top, D, F, E);
-  else if (dtype == YALM_F32)
-    moe_pair_gate_up_kernel<float><<<grid, PAIR_WAVES * WAVE, 0, stream>>>((const float*)h, (const float*)w_gate,
-                                                                           (const float*)w_up, ids, limit, alpha, up_shift, (float*)mid,
-                                                                           top, D, F, E);
-  else
+#define PAIR_UP(T_, G_)                                                                                                      \
+  moe_pair_gate_up_kernel<T_, G_><<<grid, PAIR_WAVES * WAVE, 0, stream>>>((const T_*)h, (const T_*)w_gate, (const T_*)w_up, ids, \
+                                                                          limit, alpha, up_shift, (T_*)mid, top, D, F, E)
+  if (dtype == YALM_BF16) {
+    if (w_gate != nullptr) PAIR_UP(bf16, true);
+    else PAIR_UP(bf16, false);
+  } else if (dtype == YALM_F32) {
+    if (w_gate != nullptr) PAIR_UP(float, true);
+    else PAIR_UP(float, false);
+  } else {
     return YALM_ERR_DTYPE;
+  }
+#undef PAIR_UP
   return launch_status();
 }
 
@@ -449,9 +555,13 @@ extern "C" int yalm_moe_grouped(const void* h, const void* w_gate, const void* w
   if (max_tiles > 65535) return YALM_ERR_ARG;
   moe_group_kernel<<<1, GROUP_THREADS, 0, stream>>>(ids, (int)n_pairs, E, max_tiles, pair_of_row, row_of_pair, tile_expert);
   const size_t lds = (size_t)(GR_TM + GR_TN) * GR_ROW * sizeof(bf16);
-  moe_grouped_kernel<true><<<dim3(ceil_div(F, GR_TN / 2), max_tiles), GR_THREADS, lds, stream>>>(
-      (const bf16*)h, (const bf16*)w_gate, (const bf16*)w_up, tile_expert, pair_of_row, top, mid, F, D, limit, alpha, up_shift);
-  moe_grouped_kernel<false><<<dim3(ceil_div(D, GR_TN), max_tiles), GR_THREADS, lds, stream>>>(
+  if (w_gate != nullptr)
+    moe_grouped_kernel<GR_GATED><<<dim3(ceil_div(F, GR_TN / 2), max_tiles), GR_THREADS, lds, stream>>>(
+        (const bf16*)h, (const bf16*)w_gate, (const bf16*)w_up, tile_expert, pair_of_row, top, mid, F, D, limit, alpha, up_shift);
+  else
+    moe_grouped_kernel<GR_RELU2><<<dim3(ceil_div(F, GR_TN), max_tiles), GR_THREADS, lds, stream>>>(
+        (const bf16*)h, (const bf16*)w_up, nullptr, tile_expert, pair_of_row, top, mid, F, D, 0.f, 0.f, 0.f);
+  moe_grouped_kernel<GR_DOWN><<<dim3(ceil_div(D, GR_TN), max_tiles), GR_THREADS, lds, stream>>>(
       (const bf16*)mid, (const bf16*)w_down, nullptr, tile_expert, pair_of_row, top, y, D, F, 0.f, 0.f, 0.f);
   moe_combine_kernel<<<T, 256, 0, stream>>>(y, row_of_pair, wts, out, top, D, accumulate);
   return launch_status();

@@ -1,4 +1,5 @@
-// Small per-row kernels: an embedding with a learned position vector, an activation between the two products of an
+// Small per-row kernels: an embedding with a learned position vector, an embedding that adds a row of a table hashed by
+// the previous and the present token, an activation between the two products of an
 // ungated feed-forward (or of a gated one whose products carry biases), the add of a sublayer's result under a gate
 // of one number a token, a short causal convolution over time on every channel with its carried inputs, a sigmoid
 // gate on an attention's heads, and the way into a walk of looped layers.
@@ -21,6 +22,39 @@ __global__ void embed_learned_kernel(const T* __restrict__ table, const T* __res
   }
   const T* row = table + (size_t)tok * D;
   const T* pr = pos_table + (size_t)min(max(positions[t], 0), P - 1) * D;
+  for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = fmaf(to_f32(row[i]), scale, to_f32(pr[i]));
+}
+
+// x[t, :] = table[tokens[t], :] * scale + pair_table[row, :], row = (previous * mul_prev + token * mul_cur) mod buckets,
+// or `buckets` (the table's last row) for a sequence's first token (position 0).  The previous token is the step's
+// own, or for a sequence's first token of the step the one that last[slot] holds; the workgroup of that first token
+// reads it and then leaves the sequence's last token of the step there, so that nobody reads what another writes.
+template <typename T>
+__global__ void embed_pairs_kernel(const T* __restrict__ table, const T* __restrict__ pair_table, const int* __restrict__ tokens,
+                                   const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
+                                   const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slot, int* __restrict__ last,
+                                   long mul_prev, long mul_cur, long buckets, float scale, float* __restrict__ out, int D, int V) {
+  const int t = blockIdx.x;
+  const int tok = tokens[t], b = tok_seq[t];
+  const int slot = b >= 0 ? seq_slot[b] : -1;
+  float* o = out + (size_t)t * D;
+  if (tok < 0 || tok >= V || slot < 0) {
+    for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = 0.f;
+    return;
+  }
+  const bool opens = t == cu_seqlens[b];
+  long r = buckets;
+  if (tok_pos[t] > 0) {
+    const long prev = opens ? last[slot] : tokens[t - 1];
+    r = (prev * mul_prev + (long)tok * mul_cur) % buckets;
+    if (r < 0) r += buckets;
+  }
+  if (opens) {
+    __syncthreads();                              // every thread has read last[slot]
+    if (threadIdx.x == 0) last[slot] = tokens[cu_seqlens[b + 1] - 1];
+  }
+  const T* row = table + (size_t)tok * D;
+  const T* pr = pair_table + (size_t)r * D;
   for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = fmaf(to_f32(row[i]), scale, to_f32(pr[i]));
 }
 
@@ -225,6 +259,23 @@ __global__ void loop_pack_kernel(float* __restrict__ x, const float* __restrict_
 }
 
 }  // namespace
+
+extern "C" int yalm_embed_pairs(const void* table, const void* pair_table, int dtype, const int* tokens, const int* tok_seq,
+                                const int* tok_pos, const int* cu_seqlens, const int* seq_slot, int* last, long mul_prev,
+                                long mul_cur, long buckets, float scale, float* out, int T, int D, int V, hipStream_t stream) {
+  if (T <= 0) return YALM_OK;
+  if (D <= 0 || V <= 0 || buckets <= 0) return YALM_ERR_ARG;
+  const int threads = D >= 1024 ? 1024 : (D >= 256 ? 256 : 64);
+  if (dtype == YALM_F32)
+    embed_pairs_kernel<float><<<T, threads, 0, stream>>>((const float*)table, (const float*)pair_table, tokens, tok_seq, tok_pos,
+                                                         cu_seqlens, seq_slot, last, mul_prev, mul_cur, buckets, scale, out, D, V);
+  else if (dtype == YALM_BF16)
+    embed_pairs_kernel<bf16><<<T, threads, 0, stream>>>((const bf16*)table, (const bf16*)pair_table, tokens, tok_seq, tok_pos,
+                                                        cu_seqlens, seq_slot, last, mul_prev, mul_cur, buckets, scale, out, D, V);
+  else
+    return YALM_ERR_DTYPE;
+  return launch_status();
+}
 
 extern "C" int yalm_embed_learned(const void* table, const void* pos_table, int dtype, const int* tokens,
                                   const int* positions, float scale, float* out, int T, int D, int V, int P,

@@ -1,5 +1,5 @@
 // Kernels of layers that norm a sublayer's OUTPUT before it joins the residual stream
-// (x <- x + rms(y) * w), and of the PolyNorm activation.  Everything is float32 arithmetic on a row
+// (x <- x + rms(y) * w) or the SUM of both (x <- LN(alpha x + y)), and of the PolyNorm activation.  Everything is float32 arithmetic on a row
 // per workgroup; inputs from GEMMs are float32, outputs go to the compute dtype.
 #include "common.h"
 #include "yalm_hip.h"
@@ -75,6 +75,77 @@ __global__ __launch_bounds__(NT) void norm_add_kernel(const float* __restrict__ 
   } else {
     for (int i = threadIdx.x; i < D; i += NT) h[row + i] = from_f32<T>(x[row + i] * scale2 * next_w[i]);   // its own stores
   }
+}
+
+// The layer norm of a weighted sum: n[r] = LN(alpha * x[row(r)] + y[r]) (y may be null), LN(v) = (v - mean) / sqrt(mean of
+// the squared deviations + eps) * w + b.  STORE_X: x[r] = n[r] (the stream after a layer that norms the sum).  h, if given:
+// h[r] = T(n[r]), or with next_w the layer norm that reads the stream next, h[r] = T(LN(n[r]; next_w, next_b, next_eps)).
+// PER > 0: the row fits PER values a thread and stays in registers from the sum to the last result; PER = 0: any
+// width (STORE_X then keeps the row in x, else it is formed again for every pass).
+template <typename T, int NT, int PER, bool STORE_X>
+__global__ __launch_bounds__(NT) void layer_norm_kernel(float* __restrict__ x, const float* __restrict__ y, float alpha,
+                                                        const int* __restrict__ row_index, const float* __restrict__ w,
+                                                        const float* __restrict__ b, float eps, T* __restrict__ h,
+                                                        const float* __restrict__ next_w, const float* __restrict__ next_b,
+                                                        float next_eps, int D) {
+  __shared__ float red[NT / WAVE];
+  const size_t row = (size_t)blockIdx.x * D;
+  float* xr = x + (size_t)(row_index != nullptr ? row_index[blockIdx.x] : (int)blockIdx.x) * D;
+  const float inv_d = 1.0f / (float)D;
+  float keep[PER > 0 ? PER : 1];
+  auto each = [&](auto f) {                        // f(element, place in keep)
+    if constexpr (PER > 0) {
+#pragma unroll
+      for (int j = 0; j < PER; ++j) {
+        const int i = threadIdx.x + j * NT;
+        if (i < D) f(i, j);
+      }
+    } else {
+      for (int i = threadIdx.x; i < D; i += NT) f(i, 0);
+    }
+  };
+  auto input = [&](int i) { return fmaf(alpha, xr[i], y != nullptr ? y[row + i] : 0.f); };
+  // v(i, j): the row's element at the present stage
+  auto at = [&](int i, int j) {
+    if constexpr (PER > 0) return keep[j];
+    else return STORE_X ? xr[i] : input(i);
+  };
+  float sum = 0.f;
+  each([&](int i, int j) {
+    const float v = input(i);
+    if constexpr (PER > 0) keep[j] = v;
+    else if (STORE_X) xr[i] = v;                   // a thread reads back its own stores only
+    sum += v;
+  });
+  const float mean = block_sum<NT / WAVE>(sum, red) * inv_d;
+  float ss = 0.f;
+  each([&](int i, int j) {
+    const float dv = at(i, j) - mean;
+    ss = fmaf(dv, dv, ss);
+  });
+  const float r = 1.0f / sqrtf(block_sum<NT / WAVE>(ss, red) * inv_d + eps);
+  const bool second = h != nullptr && next_w != nullptr;
+  float sum2 = 0.f;
+  each([&](int i, int j) {
+    const float n = fmaf((at(i, j) - mean) * r, w[i], b[i]);
+    if constexpr (PER > 0) keep[j] = n;
+    if (STORE_X) xr[i] = n;
+    if (h != nullptr && !second) h[row + i] = from_f32<T>(n);
+    sum2 += n;
+  });
+  if (!second) return;
+  auto normed = [&](int i, int j) {
+    if constexpr (PER > 0) return keep[j];
+    else return STORE_X ? xr[i] : fmaf((input(i) - mean) * r, w[i], b[i]);
+  };
+  const float mean2 = block_sum<NT / WAVE>(sum2, red) * inv_d;
+  float ss2 = 0.f;
+  each([&](int i, int j) {
+    const float dv = normed(i, j) - mean2;
+    ss2 = fmaf(dv, dv, ss2);
+  });
+  const float r2 = 1.0f / sqrtf(block_sum<NT / WAVE>(ss2, red) * inv_d + next_eps);
+  each([&](int i, int j) { h[row + i] = from_f32<T>(fmaf((normed(i, j) - mean2) * r2, next_w[i], next_b[i])); });
 }
 
 // out = a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + eps) over the row.  PER > 0: the row fits PER
@@ -176,6 +247,36 @@ extern "C" int yalm_norm_add(const float* y, const void* w, int w_dtype, float e
               : norm_add_launch<float, float>(y, w, eps, x, h_out, next_w, next_eps, R, D, stream);
   return hb ? norm_add_launch<bf16, bf16>(y, w, eps, x, h_out, next_w, next_eps, R, D, stream)
             : norm_add_launch<bf16, float>(y, w, eps, x, h_out, next_w, next_eps, R, D, stream);
+}
+
+template <typename T, bool STORE_X>
+static int layer_norm_launch(float* x, const float* y, float alpha, const int* row_index, const float* w, const float* b,
+                             float eps, void* h, const float* next_w, const float* next_b, float next_eps, int R, int D,
+                             hipStream_t stream) {
+#define LN(NT_, PER_)                                                                                                    \
+  layer_norm_kernel<T, NT_, PER_, STORE_X><<<R, NT_, 0, stream>>>(x, y, alpha, row_index, w, b, eps, (T*)h, next_w, next_b, \
+                                                                  next_eps, D)
+  if (D <= 1024) LN(256, 4);
+  else if (D <= 4096) LN(1024, 4);
+  else if (D <= 16384) LN(1024, 16);
+  else LN(1024, 0);
+#undef LN
+  return launch_status();
+}
+
+extern "C" int yalm_layer_norm(float* x, const float* y, float alpha, const int* row_index, const float* w, const float* b,
+                               float eps, int store_x, void* h, int h_dtype, const float* next_w, const float* next_b,
+                               float next_eps, int R, int D, hipStream_t stream) {
+  if (R <= 0) return YALM_OK;
+  if (D <= 0 || w == nullptr || b == nullptr || (store_x && row_index != nullptr) || (!store_x && h == nullptr) ||
+      (next_w != nullptr && (next_b == nullptr || h == nullptr)))
+    return YALM_ERR_ARG;
+  if (h != nullptr && h_dtype != YALM_F32 && h_dtype != YALM_BF16) return YALM_ERR_DTYPE;
+#define LN(T_, S_) layer_norm_launch<T_, S_>(x, y, alpha, row_index, w, b, eps, h, next_w, next_b, next_eps, R, D, stream)
+  const bool hb = h != nullptr && h_dtype == YALM_BF16;
+  if (store_x) return hb ? LN(bf16, true) : LN(float, true);
+  return hb ? LN(bf16, false) : LN(float, false);
+#undef LN
 }
 
 extern "C" int yalm_polynorm(const float* z, const float* coef, float eps, void* out, int out_dtype, int R, int F,

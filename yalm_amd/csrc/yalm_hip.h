@@ -255,6 +255,12 @@ int yalm_token_prob(const float* logits, const int* index, float* prob, int R, i
 int yalm_cast(const float* x, void* out, long n, int out_dtype, hipStream_t stream);
 int yalm_norm_add(const float* y, const void* w, int w_dtype, float eps, float* x, void* h_out, int h_dtype,
                   const float* next_w, float next_eps, int R, int D, hipStream_t stream);
+// yalm_layer_norm: n[r] = LN(alpha * x[row(r)] + y[r]), LN(v) = (v - mean) / sqrt(mean of the squared deviations + eps) * w + b,
+// row(r) = row_index ? row_index[r] : r; y may be null.  store_x (no row_index then): x[r] = n[r].  h (optional with
+// store_x): dtype(n[r]), or with next_w, next_b the layer norm with those of n[r].  All weights float32 [D].
+int yalm_layer_norm(float* x, const float* y, float alpha, const int* row_index, const float* w, const float* b, float eps,
+                    int store_x, void* h, int h_dtype, const float* next_w, const float* next_b, float next_eps, int R, int D,
+                    hipStream_t stream);
 int yalm_polynorm(const float* z, const float* coef, float eps, void* out, int out_dtype, int R, int F,
                   hipStream_t stream);
 
@@ -263,10 +269,13 @@ int yalm_polynorm(const float* z, const float* coef, float eps, void* out, int o
 // (n < N, k < K <= 512), times sigmoid(gate[t * gate_row + h * N + n]) if gate (float32) is given.  Types (in, wt,
 // out): all float32; float32, bfloat16, float32; all bfloat16.
 // yalm_latent_pack fills out float32 [T, (H + 2) * Dk], the head-shaped rows that yalm_rope_kv_write reads with
-// H query heads and one KV head of size Dk = [rot | rank | zeros]: query head h gets q_scale * proj[t, h * q_head +
+// H query heads and one KV head of size Dk = [rot | rank | zeros]: query head h gets q_scale * queries[t, h * q_head +
 // q_rot_off + i] in its first rot places and zeros behind rot + rank (the places between are the caller's, see
-// yalm_head_matmul); with has_kv the key row is [proj[t, kv_off + rank + i] | c | 0] and the value row [0 | c | 0], c =
-// proj[t, kv_off + i] * rsqrt(mean over the rank columns of their squares + eps) * norm_w[i].
+// yalm_head_matmul); with has_kv the key row is [kv[t, kv_off + rank + i] | c | 0] and the value row [0 | c | 0], c =
+// kv[t, kv_off + i] * rsqrt(mean over the rank columns of their squares + eps) * norm_w[i].
+// yalm_latent_norm: out[r, i] (`out_dtype` [R, n]) = x[r * x_row + i] * rsqrt(mean over those n of their squares + eps) * w[i].
+int yalm_latent_norm(const float* x, long x_row, const void* w, int w_dtype, float eps, void* out, int out_dtype, int R, int n,
+                     hipStream_t stream);
 int yalm_head_matmul(const void* in, int in_dtype, long in_row, int in_head, int in_off, const void* wt, int w_dtype,
                      void* out, int out_dtype, long out_row, int out_head, int out_off, float scale, const float* gate,
                      long gate_row, int T, int H, int K, int N, hipStream_t stream);
@@ -276,8 +285,8 @@ int yalm_head_matmul(const void* in, int in_dtype, long in_row, int in_head, int
 int yalm_head_matmul_mfma(const void* in, int in_dtype, long in_row, int in_head, int in_off, const void* wn, void* out,
                           int out_dtype, long out_row, int out_head, int out_off, float scale, const float* gate,
                           long gate_row, int T, int H, int K, int N, hipStream_t stream);
-int yalm_latent_pack(const float* proj, long proj_row, int q_head, int q_rot_off, int kv_off, const void* norm_w,
-                     int norm_dtype, float eps, float q_scale, float* out, int T, int H, int rot, int rank, int Dk,
+int yalm_latent_pack(const float* queries, long q_row, int q_head, int q_rot_off, const float* kv, long kv_row, int kv_off,
+                     const void* norm_w, int norm_dtype, float eps, float q_scale, float* out, int T, int H, int rot, int rank, int Dk,
                      int has_kv, hipStream_t stream);
 
 // Mixture of experts (moe.hip).  yalm_moe_route: ids, wts [T, top] = the `top` experts with the largest
@@ -292,6 +301,12 @@ int yalm_moe_route(const void* h, const void* w_router, int dtype, int* ids, flo
 // weighted by the softmax over the chosen logits alone.
 int yalm_moe_select(const float* logits, const float* bias, int* ids, float* wts, int T, int E, int top, int renorm,
                     hipStream_t stream);
+// Sigmoid scores and choice inside the best groups: s = sigmoid(logit), c = s + correction (float32 [E], may be null);
+// neighbours form n_groups equal groups, a group's score is the sum of its two largest c, experts outside the `keep` best
+// groups are out, the `top` (<= keep * E / n_groups) largest c are chosen and weigh s / (sum of the chosen s + 1e-20) * scale.
+int yalm_moe_select_groups(const float* logits, const float* correction, int* ids, float* wts, int T, int E, int top,
+                           int n_groups, int keep, float scale, hipStream_t stream);
+// w_gate null (here and in yalm_moe_grouped): experts of two matrices, mid = relu(w_up h)^2.
 // up_shift: the number added to the clamped up value (mid = g sigmoid(alpha g) (u + up_shift); the text above has 1;
 // alpha 1, limit 0 and up_shift 0 give silu(gate) * up).
 int yalm_moe_pair_gate_up(const void* h, const void* w_gate, const void* w_up, const int* ids, float limit, float alpha,
@@ -380,6 +395,13 @@ int yalm_gated_delta(const float* proj, const float* low, const float* conv_w, c
 // outside the vocabulary gives a row of zeros.
 int yalm_embed_learned(const void* table, const void* pos_table, int dtype, const int* tokens, const int* positions,
                        float scale, float* out, int T, int D, int V, int P, hipStream_t stream);
+// x[t, :] = table[tokens[t], :] * scale + pair_table[row, :] (both of `dtype`, [V, D] and [buckets + 1, D]), row = (previous
+// token * mul_prev + token * mul_cur) mod buckets, or `buckets` for a sequence's first token (tok_pos 0).  last int32
+// [slots] holds every sequence's last token: read for a sequence's first token of the step, then set to its last one.  A
+// token outside the vocabulary or of a padding row (slot -1) gives zeros and leaves `last` alone.
+int yalm_embed_pairs(const void* table, const void* pair_table, int dtype, const int* tokens, const int* tok_seq,
+                     const int* tok_pos, const int* cu_seqlens, const int* seq_slot, int* last, long mul_prev, long mul_cur,
+                     long buckets, float scale, float* out, int T, int D, int V, hipStream_t stream);
 // out[i] = act(z[i]), out of `out_dtype`; kind 0: z/2 (1 + erf(z / sqrt 2)), 1: the tanh form of the same, 2: silu.
 int yalm_activate(const float* z, void* out, long n, int kind, int out_dtype, hipStream_t stream);
 // x[t, :] (+)= sigmoid(h[t, :] . w) * y[t, :]; h [T, D] and w [D] of `dtype`, x and y float32; accumulate 0: x is written.
@@ -409,6 +431,15 @@ int yalm_loop_pack(float* x, const float* x0, const float* start, void* both, in
 int yalm_hgrn2(const float* proj, const float* f_bias, const float* lower, const float* w_norm, float* state, float* raw,
                const int* cu_seqlens, const int* seq_slot, void* out, int T, int B, int n_heads, int d, int dv, float eps,
                int out_dtype, hipStream_t stream);
+
+// Gated linear attention (gla.hip): proj float32 [T, 2 H d + 2 H dv + rank] = q | k | v | g | low of every token; a decay per
+// head and key channel f = sigmoid(w2 low + bias)^inv_tau (w2 float32 [H d, rank rounded up to a multiple of 4], zeros behind
+// the rank; bias float32 [H d]); per head S <- diag(f) S + k v^T, o = S^T (q_scale q); out (`out_dtype` [T, H dv]) = o over
+// its root mean square a head, times w_norm (float32 [dv]) and silu(g).  State, raw, sequences and padding rows as for
+// yalm_hgrn2.  d <= 256, rank <= 256.
+int yalm_gla(const float* proj, const float* w2, const float* bias, const float* w_norm, float* state, float* raw,
+             const int* cu_seqlens, const int* seq_slot, void* out, int T, int B, int n_heads, int d, int dv, int rank,
+             float q_scale, float inv_tau, float eps, int out_dtype, hipStream_t stream);
 
 // Yardsticks for the measurement (probes.hip): a kernel that only reads `bytes` bytes once with `workgroups`
 // workgroups (out: 1,024 words of scratch), and a loop of matrix-core instructions on registers (shape 32:

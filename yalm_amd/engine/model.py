@@ -120,8 +120,12 @@ class Model:
 
     # ------------------------------------------------------------------ the cache's needs
     def cache_requests(self):
-        """{cache line: what its mixer asks of the cache}, for the lines that are written."""
+        """{cache line: what its mixer asks of the cache}, for the lines that are written, and the embedding's line."""
         out = {}
+        if hasattr(self.embedding, "cache_request"):                     # an embedding may keep something of a sequence too
+            req = self.embedding.cache_request()
+            if req is not None:
+                out[self.embedding.CACHE_LINE] = req
         for e in self.schedule:
             if e.writes_cache:
                 block = self.blocks[e.layer]

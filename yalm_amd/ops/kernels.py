@@ -792,6 +792,39 @@ def norm_add(y, weight, eps, x, h_out=None, next_norm=None):
     return x
 
 
+def layer_norm(x, weight, bias, eps, out, row_index=None):
+    """out[r] = LN(x[row(r)]) * weight + bias, LN(v) = (v - mean) / sqrt(mean of the squared deviations + eps); x, weight and
+    bias float32, out [R, D] in the compute dtype, row(r) = row_index[r] (int32) or r."""
+    D = x.shape[1]
+    R = x.shape[0] if row_index is None else row_index.shape[0]
+    library.check(library.lib().yalm_layer_norm(
+        _need(x, "x", torch.float32, (None, D)), None, 1.0, _opt(row_index, "row_index", torch.int32, (R,)),
+        _need(weight, "weight", torch.float32, (D,)), _need(bias, "bias", torch.float32, (D,)), float(eps), 0,
+        _need(out, "out", None, (R, D)), dtype_code(out.dtype), None, None, 0.0, R, D, _stream()), "layer_norm")
+    return out
+
+
+def layer_norm_sum(y, weight, bias, eps, alpha, x, h_out=None, next_norm=None):
+    """x = LN(alpha x + y) * weight + bias, row by row (x, y float32 [R, D]); h_out (optional, the compute dtype) receives
+    the new x, or with next_norm = (float32 weight, bias, eps) the layer norm with those of the new x."""
+    R, D = y.shape
+    p_h, h_code = None, 0
+    if h_out is not None:
+        p_h, h_code = _need(h_out, "h_out", None, (R, D)), dtype_code(h_out.dtype)
+    p_w = p_b = None
+    n_eps = 0.0
+    if next_norm is not None:
+        if h_out is None:
+            raise ValueError("layer_norm_sum: the next norm's output needs h_out")
+        p_w, p_b = (_need(t, "next norm", torch.float32, (D,)) for t in next_norm[:2])
+        n_eps = float(next_norm[2])
+    library.check(library.lib().yalm_layer_norm(
+        _need(x, "x", torch.float32, (R, D)), _need(y, "y", torch.float32, (R, D)), float(alpha), None,
+        _need(weight, "weight", torch.float32, (D,)), _need(bias, "bias", torch.float32, (D,)), float(eps), 1, p_h, h_code,
+        p_w, p_b, n_eps, R, D, _stream()), "layer_norm_sum")
+    return x
+
+
 def polynorm(z, coef, eps, out):
     """out[r] = a N(z[r]) + b N(z[r]^2) + c N(z[r]^3) + e, powers element by element, N(v) = v / sqrt(mean(v^2) + eps);
     z float32 [R, F], coef float32 [4] = (a, b, c, e) on the device, out [R, F] in the compute dtype."""
@@ -846,18 +879,32 @@ def head_matmul(src, src_head, src_off, wt, out, out_head, out_off, scale=1.0, g
     return out
 
 
-def latent_pack(proj, q_head, q_rot_off, kv_off, norm_w, eps, q_scale, out, n_heads, rot, rank, padded, has_kv):
+def latent_norm(x, n, w, eps, out):
+    """out[r] = x[r, :n] over their root mean square, times w [n]; x float32 [R, >= n], out [R, n] in the compute dtype."""
+    R = x.shape[0]
+    if x.shape[1] < n:
+        raise ValueError("latent_norm: %d of %d columns" % (n, x.shape[1]))
+    library.check(library.lib().yalm_latent_norm(
+        _need(x, "x", torch.float32, (R, None)), x.shape[1], _need(w, "w", None, (n,)), dtype_code(w.dtype), float(eps),
+        _need(out, "out", None, (R, n)), dtype_code(out.dtype), R, n, _stream()), "latent_norm")
+    return out
+
+
+def latent_pack(queries, q_head, q_rot_off, kv_off, norm_w, eps, q_scale, out, n_heads, rot, rank, padded, has_kv, kv=None):
     """Fills out float32 [T, (n_heads + 2) * padded], the rows that rope_kv_write reads as n_heads query heads and
-    one KV head of size `padded`, each [rot | rank | zeros]: the rotated parts of the queries from proj (float32
+    one KV head of size `padded`, each [rot | rank | zeros]: the rotated parts of the queries (float32
     [T, *]; head h at column h * q_head + q_rot_off) times q_scale, zeros in the padding, and with has_kv the key
-    [proj[kv_off + rank:][:rot] | c | 0] and the value [0 | c | 0], c the RMS norm (weights norm_w, eps) of
-    proj[kv_off:][:rank].  The queries' rank places are left for head_matmul."""
-    T = proj.shape[0]
+    [kv[kv_off + rank:][:rot] | c | 0] and the value [0 | c | 0], c the RMS norm (weights norm_w, eps) of
+    kv[kv_off:][:rank] (kv float32 [T, *]; None: the queries' rows hold it).  The queries' rank places are left for
+    head_matmul."""
+    T = queries.shape[0]
     p_n, n_code = None, 0
     if has_kv:
         p_n, n_code = _need(norm_w, "norm_w", None, (rank,)), dtype_code(norm_w.dtype)
+    kv = queries if kv is None else kv
     library.check(library.lib().yalm_latent_pack(
-        _need(proj, "proj", torch.float32, (T, None)), proj.shape[1], q_head, q_rot_off, kv_off if has_kv else 0, p_n,
+        _need(queries, "queries", torch.float32, (T, None)), queries.shape[1], q_head, q_rot_off,
+        _need(kv, "kv", torch.float32, (T, None)), kv.shape[1], kv_off if has_kv else 0, p_n,
         n_code, float(eps), float(q_scale), _need(out, "out", torch.float32, (T, (n_heads + 2) * padded)), T, n_heads,
         rot, rank, padded, 1 if has_kv else 0, _stream()), "latent_pack")
     return out
@@ -1064,6 +1111,23 @@ def embed_learned(table, pos_table, tokens, positions, scale, out):
     return out
 
 
+def embed_pairs(table, pair_table, tokens, tok_seq, tok_pos, cu_seqlens, seq_slot, last, mul_prev, mul_cur, scale, out):
+    """out[t] = table[tokens[t]] * scale + pair_table[row], row = (previous token * mul_prev + tokens[t] * mul_cur) mod (rows of
+    pair_table - 1), the last row for a sequence's first token.  last int32 [slots] is every sequence's last token: read for
+    its first token of the step and set to its last one (slot -1: rows of zeros, nothing set)."""
+    V, D = table.shape
+    T, B = tokens.shape[0], seq_slot.shape[0]
+    if pair_table.shape[0] < 2:
+        raise ValueError("embed_pairs: a pair table has two rows or more")
+    library.check(library.lib().yalm_embed_pairs(
+        _need(table, "table", None, (V, D)), _need(pair_table, "pair_table", table.dtype, (None, D)), dtype_code(table.dtype),
+        _need(tokens, "tokens", torch.int32, (T,)), _need(tok_seq, "tok_seq", torch.int32, (T,)),
+        _need(tok_pos, "tok_pos", torch.int32, (T,)), _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)),
+        _need(seq_slot, "seq_slot", torch.int32, (B,)), _need(last, "last", torch.int32), int(mul_prev), int(mul_cur),
+        pair_table.shape[0] - 1, float(scale), _need(out, "out", torch.float32, (T, D)), T, D, V, _stream()), "embed_pairs")
+    return out
+
+
 ACTIVATIONS = {"gelu_erf": 0, "gelu_tanh": 1, "silu": 2}
 
 
@@ -1181,6 +1245,42 @@ def hgrn2(proj, f_bias, lower, w_norm, state, raw, cu_seqlens, seq_slot, out, n_
 
 
 # ---------------------------------------------------------------------------------------------------------------
+# gated linear attention
+GLA_MAX_KEY_DIM = 256             # rows of a state column over a workgroup's lanes
+GLA_MAX_RANK = 256                # of the decays' low-rank product
+
+
+def gla_state_elements(n_heads, d, dv):
+    return n_heads * d * dv
+
+
+def gla_padded_rank(rank):
+    return (rank + 3) // 4 * 4
+
+
+def gla(proj, w2, bias, w_norm, state, raw, cu_seqlens, seq_slot, out, n_heads, d, dv, rank, q_scale, tau, eps):
+    """Gated linear attention over a step's tokens.  proj float32 [T, 2 H d + 2 H dv + rank] = q | k | v | g | low; f =
+    sigmoid(w2 low + bias)^(1 / tau) per head and key channel (w2 float32 [H d, gla_padded_rank(rank)]); per head S <- diag(f)
+    S + k v^T, o = S^T (q_scale q); out [T, H dv] = o over its root mean square a head, times w_norm [dv] and silu(g).
+    state float32 [slots, H dv d] (a head's S column by column) is read and left advanced; raw float32 [T, H dv] is
+    scratch.  Sequence b's tokens are cu_seqlens[b] .. cu_seqlens[b + 1] - 1."""
+    T = proj.shape[0]
+    B = seq_slot.shape[0]
+    N = 2 * n_heads * d + 2 * n_heads * dv + rank
+    if not 0 < d <= GLA_MAX_KEY_DIM or not 0 < rank <= GLA_MAX_RANK:
+        raise ValueError("gla: key heads of %d (at most %d) with decays of rank %d (at most %d)"
+                         % (d, GLA_MAX_KEY_DIM, rank, GLA_MAX_RANK))
+    library.check(library.lib().yalm_gla(
+        _need(proj, "proj", torch.float32, (T, N)), _need(w2, "w2", torch.float32, (n_heads * d, gla_padded_rank(rank))),
+        _need(bias, "bias", torch.float32, (n_heads * d,)), _need(w_norm, "w_norm", torch.float32, (dv,)),
+        _need(state, "state", torch.float32, (None, n_heads * d * dv)), _need(raw, "raw", torch.float32, (T, n_heads * dv)),
+        _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)), _need(seq_slot, "seq_slot", torch.int32, (B,)),
+        _need(out, "out", None, (T, n_heads * dv)), T, B, n_heads, d, dv, rank, float(q_scale), 1.0 / float(tau), float(eps),
+        dtype_code(out.dtype), _stream()), "gla")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------------------------
 # mixture of experts
 MOE_MAX_EXPERTS = 1024
 
@@ -1214,15 +1314,31 @@ def moe_select(logits, ids, wts, renormalize=False, bias=None):
         "moe_select")
 
 
+def moe_select_groups(logits, correction, ids, wts, n_groups=1, keep=1, scale=1.0):
+    """ids, wts [T, top] from float32 logits [T, E]: scores s = sigmoid(logit), choice scores c = s + correction (float32 [E]
+    or None); E experts form n_groups equal groups of neighbours, a group's score is the sum of its two largest c; among
+    the experts of the `keep` best groups the top largest c are chosen (the lower index on ties) and weigh s / (sum of the
+    chosen s + 1e-20) * scale."""
+    T, E = logits.shape
+    top = ids.shape[1]
+    if E > MOE_MAX_EXPERTS or n_groups <= 0 or E % n_groups or not 0 < keep <= n_groups or not 0 < top <= keep * (E // n_groups):
+        raise ValueError("moe_select_groups: %d of %d experts from %d of %d groups is not offered (at most %d experts)"
+                         % (top, E, keep, n_groups, MOE_MAX_EXPERTS))
+    library.check(library.lib().yalm_moe_select_groups(
+        _need(logits, "logits", torch.float32, (T, E)), _opt(correction, "correction", torch.float32, (E,)),
+        _need(ids, "ids", torch.int32, (T, top)), _need(wts, "wts", torch.float32, (T, top)), T, E, top, n_groups, keep,
+        float(scale), _stream()), "moe_select_groups")
+
+
 def moe_pair_gate_up(h, w_gate, w_up, ids, limit, alpha, mid, up_shift=1.0):
-    """mid[t * top + k] = g sigmoid(alpha g) (u + up_shift), g = min(w_gate[e] h[t], limit), u = clamp(w_up[e] h[t], +-limit)
+    """w_gate None: mid[t * top + k] = relu(w_up[e] h[t])^2.  Else mid[t * top + k] = g sigmoid(alpha g) (u + up_shift), g = min(w_gate[e] h[t], limit), u = clamp(w_up[e] h[t], +-limit)
     for e = ids[t, k] (limit <= 0: unclamped; alpha 1, up_shift 0: silu(gate) * up); w_gate, w_up [E, F, D]."""
     T, D = h.shape
-    E, F, _ = w_gate.shape
+    E, F, _ = w_up.shape
     top = ids.shape[1]
     dt = h.dtype
     library.check(library.lib().yalm_moe_pair_gate_up(
-        _need(h, "h", dt, (T, D)), _need(w_gate, "w_gate", dt, (E, F, D)), _need(w_up, "w_up", dt, (E, F, D)),
+        _need(h, "h", dt, (T, D)), _opt(w_gate, "w_gate", dt, (E, F, D)), _need(w_up, "w_up", dt, (E, F, D)),
         _need(ids, "ids", torch.int32, (T, top)), float(limit), float(alpha), float(up_shift),
         _need(mid, "mid", dt, (T * top, F)), T, top, D, F, E, dtype_code(dt), _stream()), "moe_pair_gate_up")
     return mid
@@ -1260,7 +1376,7 @@ def moe_grouped(h, w_gate, w_up, w_down, ids, wts, limit, alpha, scratch, out, a
     the device and every product is one launch over all experts' tiles on the matrix cores.  scratch(name, shape,
     dtype) hands out the buffers (pair_of_row, row_of_pair, tile_expert, mid, y)."""
     T, D = h.shape
-    E, F, _ = w_gate.shape
+    E, F, _ = w_up.shape
     top = ids.shape[1]
     dt = torch.bfloat16
     tiles = moe_grouped_tiles(T * top, E)
@@ -1271,7 +1387,7 @@ def moe_grouped(h, w_gate, w_up, w_down, ids, wts, limit, alpha, scratch, out, a
     mid = scratch("moe.hidden", (rows, F), dt)
     y = scratch("moe.y", (rows, D), torch.float32)
     library.check(library.lib().yalm_moe_grouped(
-        _need(h, "h", dt, (T, D)), _need(w_gate, "w_gate", dt, (E, F, D)), _need(w_up, "w_up", dt, (E, F, D)),
+        _need(h, "h", dt, (T, D)), _opt(w_gate, "w_gate", dt, (E, F, D)), _need(w_up, "w_up", dt, (E, F, D)),
         _need(w_down, "w_down", dt, (E, D, F)), _need(ids, "ids", torch.int32, (T, top)),
         _need(wts, "wts", torch.float32, (T, top)), float(limit), float(alpha), float(up_shift),
         _need(pair_of_row, "pair_of_row", torch.int32, (rows,)), _need(row_of_pair, "row_of_pair", torch.int32, (T * top,)),

@@ -55,7 +55,12 @@ _SIGNATURES = {
                               _I, _I, _I, _I, _P]),
     "yalm_head_matmul_mfma": (_I, [_P, _I, ctypes.c_long, _I, _I, _P, _P, _I, ctypes.c_long, _I, _I, _F, _P, ctypes.c_long,
                                    _I, _I, _I, _I, _P]),
-    "yalm_latent_pack": (_I, [_P, ctypes.c_long, _I, _I, _I, _P, _I, _F, _F, _P, _I, _I, _I, _I, _I, _I, _P]),
+    "yalm_latent_pack": (_I, [_P, ctypes.c_long, _I, _I, _P, ctypes.c_long, _I, _P, _I, _F, _F, _P, _I, _I, _I, _I, _I, _I, _P]),
+    "yalm_latent_norm": (_I, [_P, ctypes.c_long, _P, _I, _F, _P, _I, _I, _I, _P]),
+    "yalm_layer_norm": (_I, [_P, _P, _F, _P, _P, _P, _F, _I, _P, _I, _P, _P, _F, _I, _I, _P]),
+    "yalm_embed_pairs": (_I, [_P, _P, _I, _P, _P, _P, _P, _P, _P, ctypes.c_long, ctypes.c_long, ctypes.c_long, _F, _P, _I, _I, _I, _P]),
+    "yalm_moe_select_groups": (_I, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P]),
+    "yalm_gla": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]),
     "yalm_moe_route": (_I, [_P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P]),
     "yalm_moe_select": (_I, [_P, _P, _P, _P, _I, _I, _I, _I, _P]),
     "yalm_moe_pair_gate_up": (_I, [_P, _P, _P, _P, _F, _F, _F, _P, _I, _I, _I, _I, _I, _I, _P]),
@@ -82,7 +87,7 @@ _SIGNATURES = {
     "yalm_probe_mfma": (_I, [_I, _I, _I, _P, _P, _P]),
 }
 
-ABI_VERSION = 35
+ABI_VERSION = 36
 
 
 class KernelError(RuntimeError):

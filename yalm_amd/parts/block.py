@@ -128,10 +128,11 @@ class StreamInput:
 @part("block", "postnorm_residual")
 class PostNormResidualBlock(Part):
     """x += norm(mixer(x)); x += norm(feed_forward(x)): the sublayers read the residual stream itself and
-    the norms act on their OUTPUTS.  Members: mixer, mixer_norm, and optionally feed_forward with
+    the norms act on their OUTPUTS, or, with norms whose `join` works on the sum (LayerNorm), x = norm(a x + mixer(x));
+    x = norm(a x + feed_forward(x)).  Members: mixer, mixer_norm, and optionally feed_forward with
     feed_forward_norm (a layer may have no feed-forward).  The sublayers offer forward_to(h, y, ...),
-    which writes their result to y instead of adding it to the stream; the norm's add_normed(y, x, h_out)
-    adds it normed and hands the new stream on in the compute dtype.  With float32 as the compute dtype the
+    which writes their result to y instead of adding it to the stream; the norm's join(y, x, h_out)
+    brings it into the stream and hands the new stream on in the compute dtype.  With float32 as the compute dtype the
     sublayers read the stream's own memory."""
 
     def __init__(self, layer_spec, dim, prefix=""):
@@ -165,18 +166,19 @@ class PostNormResidualBlock(Part):
             h = kernels.cast(x, ctx.ws.get("block.h", (T, self.dim), ctx.act_dtype))
         hand_on = None if same or not isinstance(next_norm, StreamInput) else ctx.ws.get("block.h", (T, self.dim), ctx.act_dtype)
         # the last layer of a decode step leaves the final norm's output for the head
-        final = next_norm if ctx.mode == "decode" and hasattr(next_norm, "fused") else None
+        last_norm = self.mixer_norm if self.feed_forward is None else self.feed_forward_norm
+        final = next_norm if ctx.mode == "decode" and last_norm.can_hand_to(next_norm) else None
         if final is not None:
             hand_on = ctx.ws.get("block.normed", (T, self.dim), ctx.act_dtype)
         y = ctx.ws.get("block.y", (T, self.dim), torch.float32)
         self.mixer.forward_to(h, y, ctx, line, writes_cache)
         if self.feed_forward is None:
-            self.mixer_norm.add_normed(y, x, ctx, h_out=hand_on, next_norm=final)
+            self.mixer_norm.join(y, x, ctx, h_out=hand_on, next_norm=final)
         else:
             h = x if same else ctx.ws.get("block.h", (T, self.dim), ctx.act_dtype)
-            self.mixer_norm.add_normed(y, x, ctx, h_out=None if same else h)
+            self.mixer_norm.join(y, x, ctx, h_out=None if same else h)
             self.feed_forward.forward_to(h, y, ctx)
-            self.feed_forward_norm.add_normed(y, x, ctx, h_out=hand_on, next_norm=final)
+            self.feed_forward_norm.join(y, x, ctx, h_out=hand_on, next_norm=final)
         if hand_on is not None:
             ctx.normed[id(next_norm)] = (hand_on, None, None)
 

@@ -1,5 +1,8 @@
 """Token embedding (optionally scaled, optionally with a sinusoidal position vector) and the LM head.  The head is the embedding table itself
 when tied (src/model.cpp:389-398); one copy on the device either way."""
+import torch
+
+from ..cache.manager import StateRequest
 from ..ops import kernels
 from ..weights.loader import ParamSpec, place
 from .base import Part, build_part, part
@@ -11,7 +14,9 @@ class TokenEmbedding(Part):
     a position vector whose entry 2i is sin(p b^(-2i / width)) and whose entry 2i + 1 is the cosine of the same angle
     (the frequencies are made in float64 and the angle is exact at every position), or, with `position_tensor` (a
     tensor's name) and `n_positions`, plus the row of that learned table [n_positions, width] at the token's position.
-    With `norm` (a norm's PartSpec) the result passes that norm at once, in float32; with `keep_output` a copy of what the
+    With `pairs` {tensor, buckets, mul_prev, mul_cur}: plus row (previous token * mul_prev + token * mul_cur) mod buckets of a
+    second table [buckets + 1, width], its last row for a sequence's first token; every sequence's last token is kept in
+    the cache's fixed-size state, under the line CACHE_LINE.  With `norm` (a norm's PartSpec) the result passes that norm at once, in float32; with `keep_output` a copy of what the
     part leaves stays in the step's buffer "embed.kept" for layers that read it again (the way into looped layers)."""
 
     def __init__(self, spec, dim, prefix):
@@ -24,9 +29,15 @@ class TokenEmbedding(Part):
         self.n_positions = int(spec.params.get("n_positions", 0) or 0)
         if self.position_tensor and (self.sinusoid_base or self.n_positions <= 0):
             raise ValueError("a learned position table needs n_positions, and goes without the sinusoid")
+        self.pairs = spec.params.get("pairs")
+        if self.pairs:
+            self.pairs = {"tensor": str(self.pairs.get("tensor", "pairs")), **{k: int(self.pairs[k]) for k in ("buckets", "mul_prev", "mul_cur")}}
+            if self.sinusoid_base or self.position_tensor or spec.params.get("keep_output"):
+                raise ValueError("an embedding of token pairs goes without position vectors and keeps no copy")
         self.table = None
         self.freq = None
         self.positions = None
+        self.pair_table = None
         self.norm = build_part("norm", spec.params["norm"], dim, prefix) if spec.params.get("norm") else None
         self.keep_output = bool(spec.params.get("keep_output", False))
 
@@ -37,23 +48,30 @@ class TokenEmbedding(Part):
         out = [ParamSpec(self.tensor, (self.vocab_size, self.dim), init="embedding")]
         if self.position_tensor:
             out.append(ParamSpec(self.prefix + str(self.position_tensor), (self.n_positions, self.dim), init="embedding"))
+        if self.pairs:
+            out.append(ParamSpec(self.prefix + self.pairs["tensor"], (self.pairs["buckets"] + 1, self.dim), init="embedding"))
         return out
+
+    CACHE_LINE = "embedding"          # what the embedding keeps of a sequence lies under this line of the cache
+
+    def cache_request(self):
+        return StateRequest((1,), torch.int32) if self.pairs else None
 
     def load(self, get, compute_dtype, device):
         self.table = place(get(self.tensor), compute_dtype, device)
+        if self.pairs:
+            self.pair_table = place(get(self.prefix + self.pairs["tensor"]), compute_dtype, device)
         if self.position_tensor:
             self.positions = place(get(self.prefix + str(self.position_tensor)), compute_dtype, device)
         if self.sinusoid_base:
-            import torch
             i = torch.arange((self.dim + 1) // 2, dtype=torch.float64)
             base = torch.tensor(float(self.sinusoid_base), dtype=torch.float64)
             self.freq = torch.pow(base, -2.0 * i / self.dim).to(device)
 
     def weight_bytes(self):
-        return (2 if self.positions is not None else 1) * self.dim * self.table.element_size()     # one row per token
+        return (2 if self.positions is not None or self.pair_table is not None else 1) * self.dim * self.table.element_size()     # one row per token
 
     def forward(self, tokens, x, ctx):
-        import torch
         kept = ctx.ws.get("embed.kept", tuple(x.shape), torch.float32) if self.keep_output else None
         if self.norm is None:
             self._rows(tokens, x, ctx)
@@ -72,6 +90,10 @@ class TokenEmbedding(Part):
             if ctx.max_position >= self.n_positions:
                 raise ValueError("position %d is beyond the %d rows of the position table" % (ctx.max_position, self.n_positions))
             return kernels.embed_learned(self.table, self.positions, tokens, ctx.tok_pos, self.scale, x)
+        if self.pair_table is not None:
+            last = ctx.cache.group_of(self.CACHE_LINE).line_state(self.CACHE_LINE)
+            return kernels.embed_pairs(self.table, self.pair_table, tokens, ctx.tok_seq, ctx.tok_pos, ctx.cu_seqlens, ctx.seq_slot,
+                                       last, self.pairs["mul_prev"], self.pairs["mul_cur"], self.scale, x)
         if self.freq is None and self.scale == 1.0:
             return kernels.embed(self.table, tokens, x)
         return kernels.embed_sinusoid(self.table, tokens, ctx.tok_pos, self.freq, self.scale, x)
@@ -103,10 +125,12 @@ class LMHead(Part):
         return self.weight.numel() * self.weight.element_size()
 
     def fuses_norm(self, norm, x, ctx):
-        if not hasattr(norm, "fused") or ctx.mode != "decode":
+        if ctx.mode != "decode":
             return False
         if id(norm) in ctx.normed:
             return True                                   # whoever prepared it checked the shape
+        if not hasattr(norm, "fused"):
+            return False
         return kernels.can_fuse_norm(x.shape[0], self.dim, self.weight.dtype)
 
     def forward_prenorm(self, x, norm, logits, ctx):

@@ -7,6 +7,7 @@ and latent size R:
     k_h^plain = W_uk,h c,  v_h = W_uv,h c
     score_h(i, j) = (q_h^plain(i) . k_h^plain(j) + rotate(q_h^rot(i)) . k^rot(j)) * scale
     out = W_o [softmax(score_h) v_h]_h,  optionally the heads' results times sigmoid(W_g h) before W_o.
+With `q_rank` the queries pass a latent vector of their own: q = W_q rms(W_dq h) w_cq, W_dq h being one product with W_dkv h.
 Only c and k^rot are kept.  Because k_h^plain and v_h are linear in c, attention runs in the latent space:
 q_h^plain . (W_uk,h c) = (W_uk,h^T q_h^plain) . c, and sum_j p_j W_uv,h c_j = W_uv,h sum_j p_j c_j.  So the cache
 line is ONE key/value head of size P = rot + R (rounded up to a multiple of 16, zeros behind) holding
@@ -34,7 +35,7 @@ from .attention import ROPE_TILES_MIN_TOKENS, decode_splits, kv_tiles
 from .base import Part, build_part, part
 from .rope import interleave_rows
 
-_NAMES = {"q": "q_proj.weight", "down_kv": "kv_down_proj.weight", "kv_norm": "kv_norm.weight",
+_NAMES = {"q": "q_proj.weight", "down_q": "q_down_proj.weight", "q_norm": "q_norm.weight", "down_kv": "kv_down_proj.weight", "kv_norm": "kv_norm.weight",
           "up_k": "k_up_proj.weight", "up_v": "v_up_proj.weight", "out": "o_proj.weight", "gate": "gate_proj.weight"}
 
 
@@ -50,6 +51,7 @@ class LatentAttention(Part):
         self.rot_dim = int(p["rot_dim"])
         self.v_dim = int(p["v_dim"])
         self.rank = int(p["kv_rank"])
+        self.q_rank = int(p.get("q_rank", 0) or 0)    # of the queries' latent vector (0: they are made from h itself)
         self.scale = float(p["scale"])
         self.window = int(p.get("window", 0) or 0)
         self.gated = bool(p.get("gated", False))
@@ -68,6 +70,8 @@ class LatentAttention(Part):
         self.q_cols = self.n_heads * (self.head_dim + self.rot_dim)
         self.kv_cols = self.rank + self.rot_dim if self.own_keys else 0
         self.gate_cols = self.n_heads * self.v_dim if self.gated else 0
+        self.in_q_cols = self.q_rank or self.q_cols   # what the first product makes for the queries
+        self.w_uq = self.q_norm = None
         self.w_in = self.w_uk = self.w_uv = self.w_o = self.kv_norm = self.w_uk_nk = self.w_uv_nk = None
 
     def children(self):
@@ -78,7 +82,9 @@ class LatentAttention(Part):
 
     def param_specs(self):
         D, H = self.dim, self.n_heads
-        out = [ParamSpec(self._name("q"), (self.q_cols, D), fan_in=D)]
+        out = [ParamSpec(self._name("q"), (self.q_cols, self.q_rank or D), fan_in=self.q_rank or D)]
+        if self.q_rank:
+            out += [ParamSpec(self._name("down_q"), (self.q_rank, D), fan_in=D), ParamSpec(self._name("q_norm"), (self.q_rank,), init="norm")]
         if self.own_keys:
             out += [ParamSpec(self._name("down_kv"), (self.rank + self.rot_dim, D), fan_in=D),
                     ParamSpec(self._name("kv_norm"), (self.rank,), init="norm")]
@@ -97,9 +103,13 @@ class LatentAttention(Part):
         def pairs(w, heads):          # rotated rows of `heads` heads of r rows each, pairs made adjacent
             return interleave_rows(w, heads, r, dims) if half_split and r else w
 
-        wq = get(self._name("q")).reshape(H, d + r, self.dim)
-        wq = torch.cat([wq[:, :d], pairs(wq[:, d:].reshape(H * r, self.dim), H).reshape(H, r, self.dim)], dim=1)
-        blocks = [wq.reshape(H * (d + r), self.dim)]
+        wq = get(self._name("q")).reshape(H, d + r, -1)
+        wq = torch.cat([wq[:, :d], pairs(wq[:, d:].reshape(H * r, wq.shape[-1]), H).reshape(H, r, -1)], dim=1)
+        wq = wq.reshape(H * (d + r), -1)
+        if self.q_rank:
+            self.w_uq = place(wq, compute_dtype, device)
+            self.q_norm = place(get(self._name("q_norm")), compute_dtype, device)
+        blocks = [get(self._name("down_q")) if self.q_rank else wq]
         if self.own_keys:
             wd = get(self._name("down_kv"))
             blocks.append(torch.cat([wd[:R], pairs(wd[R:], 1)], dim=0))
@@ -117,13 +127,13 @@ class LatentAttention(Part):
         self.w_o = place(get(self._name("out")), compute_dtype, device)
 
     def weight_bytes(self):
-        return sum(w.numel() * w.element_size() for w in (self.w_in, self.w_uk, self.w_uv, self.w_o))
+        return sum(w.numel() * w.element_size() for w in (self.w_in, self.w_uq, self.w_uk, self.w_uv, self.w_o) if w is not None)
 
     def cache_request(self):
         return KVRequest(1, self.padded, self.window, 0) if self.own_keys else None
 
     def row_elements(self):
-        return max(self.q_cols + self.kv_cols + self.gate_cols, (self.n_heads + 2) * self.padded)
+        return max(self.in_q_cols + self.kv_cols + self.gate_cols, (self.n_heads + 2) * self.padded)
 
     def describe(self, compute_dtype):
         what = "latent attention, %d heads on one latent head of %d (%d rotated + %d)%s" % (
@@ -156,14 +166,22 @@ class LatentAttention(Part):
                              % (ctx.max_position, pos.n_positions))
         prefill = ctx.mode == "prefill"
         # 1. one product for the queries, the down projection and the gate
-        n_in = self.q_cols + self.kv_cols + self.gate_cols
+        n_in = self.in_q_cols + self.kv_cols + self.gate_cols
+        kv_at = self.in_q_cols
         proj = ws.get("latent.proj", (T, n_in), torch.float32)
         self._gemm(ctx, h, self.w_in, proj, kernels.EPI_STORE_F32)
+        queries = proj
+        if self.q_rank:
+            c_q = ws.get("latent.cq", (T, self.q_rank), act)
+            kernels.latent_norm(proj, self.q_rank, self.q_norm, self.eps, c_q)
+            queries = ws.get("latent.queries", (T, self.q_cols), torch.float32)
+            self._gemm(ctx, c_q, self.w_uq, queries, kernels.EPI_STORE_F32)
         # 2. head-shaped rows [rot | rank | 0]: H query heads, then the key and the value
         heads = ws.get("latent.heads", (T, (H + 2) * P), torch.float32)
         q_scale = self.scale * math.sqrt(P)
-        kernels.latent_pack(proj, d + r, d, self.q_cols, self.kv_norm, self.eps, q_scale, heads, H, r, R, P, self.own_keys)
-        kernels.head_matmul(proj, d + r, 0, self.w_uk, heads, P, r, scale=q_scale, wt_nk=self.w_uk_nk)
+        kernels.latent_pack(queries, d + r, d, kv_at, self.kv_norm, self.eps, q_scale, heads, H, r, R, P, self.own_keys,
+                            kv=proj)
+        kernels.head_matmul(queries, d + r, 0, self.w_uk, heads, P, r, scale=q_scale, wt_nk=self.w_uk_nk)
         # 3. rotation, cache write, attention over the latent head
         q = ws.get("attn.q", (T, H * P), act)
         group = ctx.cache.group_of(line)
@@ -198,7 +216,7 @@ class LatentAttention(Part):
                                 H, 1, P, self.window, n_splits, step_max_len=ctx.step_max_len, seq_order=ctx.seq_order)
         # 4. the heads' values from their latent results, the gate, the output projection
         values = ws.get("latent.values", (T, H * self.v_dim), act)
-        gate = proj[:, self.q_cols + self.kv_cols:] if self.gated else None
+        gate = proj[:, kv_at + self.kv_cols:] if self.gated else None
         kernels.head_matmul(o, P, r, self.w_uv, values, self.v_dim, 0, gate=gate, wt_nk=self.w_uv_nk)
         self._gemm(ctx, values, self.w_o, out, epilogue)
         return out

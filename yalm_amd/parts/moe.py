@@ -1,4 +1,4 @@
-"""Mixture of experts: `n_experts` small gated feed-forwards, of which a token uses the `top` whose router
+"""Mixture of experts: `n_experts` small feed-forwards, of which a token uses the `top` whose router
 scores are largest.
 
 Router: s = softmax(W_router h (+ a bias, the tensor `router_bias`)) over all experts, in float32; the chosen experts'
@@ -6,7 +6,11 @@ weights are their scores (`renormalize`: divided by their sum; "chosen": the exp
 by the softmax over the chosen logits alone).  Expert: g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit),
 out = W_down (g sigmoid(alpha g) (u + up_shift)) (limit 0: no clamping; up_shift defaults to 1; alpha 1 and up_shift 0
 make silu(gate) * up).  The part's result is the weighted sum over
-a token's chosen experts, in the order of their scores.  With `shared` = {hidden, prefix, gate} one more expert of the
+a token's chosen experts, in the order of their scores.  `unit` "relu2": experts of two matrices, out = W_down
+relu(W_up h)^2.  `scores` "sigmoid": s = sigmoid(W_router h); experts are chosen by s plus a correction (the tensor
+`correction`, one number an expert), among the `keep_groups` best of `groups` equal groups of neighbouring experts (a
+group's score is the sum of its two largest corrected scores), and weigh s over the sum of the chosen s, times
+`weight_scale`.  With `shared` = {hidden, prefix, gate} one more expert of the
 same form (its tensors behind `prefix`, its own hidden size) runs for every token and is added, times sigmoid(w . h), one
 number a token (w: the tensor `gate` behind the prefix, [1, width]; no `gate`: added as it is).
 
@@ -43,12 +47,28 @@ class MixtureOfExperts(Part):
         self.renormalize = p.get("renormalize", False)
         self.renormalize = "chosen" if self.renormalize == "chosen" else bool(self.renormalize)
         self.expert_prefix = str(p.get("expert_prefix", "experts.%d."))
+        self.gated = p.get("unit", "gated") == "gated"
+        self.sigmoid = p.get("scores", "softmax") == "sigmoid"
+        if p.get("unit", "gated") not in ("gated", "relu2") or p.get("scores", "softmax") not in ("softmax", "sigmoid"):
+            raise ValueError("mixture of experts: unit %r with scores %r is not offered" % (p.get("unit"), p.get("scores")))
+        self.groups, self.keep_groups = int(p.get("groups", 1)), int(p.get("keep_groups", 1))
+        self.weight_scale = float(p.get("weight_scale", 1.0))
         self.names = {"router": "router", "gate": "gate", "up": "up", "down": "down"}
         self.names.update(p.get("tensors") or {})
         self.router_bias = self.names.get("router_bias")           # a tensor's name, or no bias
         if not 0 < self.top <= self.n_experts or self.n_experts > kernels.MOE_MAX_EXPERTS:
             raise ValueError("mixture of experts: %d of %d experts is not offered (at most %d experts)"
                              % (self.top, self.n_experts, kernels.MOE_MAX_EXPERTS))
+        if self.groups <= 0 or self.n_experts % self.groups or not 0 < self.keep_groups <= self.groups \
+                or self.top > self.keep_groups * (self.n_experts // self.groups):
+            raise ValueError("mixture of experts: %d of %d experts from %d of %d groups is not offered"
+                             % (self.top, self.n_experts, self.keep_groups, self.groups))
+        self.correction_name = self.names.get("correction")        # a tensor's name, or no correction
+        if not self.sigmoid and (self.groups > 1 or self.weight_scale != 1.0 or self.correction_name):
+            raise ValueError("groups, a correction and weight_scale go with sigmoid scores")
+        if self.sigmoid and (self.renormalize or self.router_bias):
+            raise ValueError("sigmoid scores are always brought to one sum and take no router bias")
+        self.correction = None
         self.w_router = self.w_gate = self.w_up = self.w_down = self.b_router = None
         self.shared = None
         if p.get("shared"):
@@ -66,9 +86,12 @@ class MixtureOfExperts(Part):
         out = [ParamSpec(self.prefix + self.names["router"], (self.n_experts, D), fan_in=D)]
         if self.router_bias:
             out.append(ParamSpec(self.prefix + self.router_bias, (self.n_experts,), init="bias"))
+        if self.correction_name:
+            out.append(ParamSpec(self.prefix + self.correction_name, (self.n_experts,), init="bias"))
         for e in range(self.n_experts):
-            out += [ParamSpec(self._expert(e, "gate"), (F, D), fan_in=D), ParamSpec(self._expert(e, "up"), (F, D), fan_in=D),
-                    ParamSpec(self._expert(e, "down"), (D, F), fan_in=F)]
+            if self.gated:
+                out.append(ParamSpec(self._expert(e, "gate"), (F, D), fan_in=D))
+            out += [ParamSpec(self._expert(e, "up"), (F, D), fan_in=D), ParamSpec(self._expert(e, "down"), (D, F), fan_in=F)]
         if self.shared:
             Fs = self.shared["hidden"]
             out += [ParamSpec(self._shared("gate"), (Fs, D), fan_in=D), ParamSpec(self._shared("up"), (Fs, D), fan_in=D),
@@ -85,7 +108,10 @@ class MixtureOfExperts(Part):
         self.w_router = place(get(self.prefix + self.names["router"]), compute_dtype, device)
         if self.router_bias:
             self.b_router = get(self.prefix + self.router_bias).to(torch.float32).to(device).contiguous()
-        self.w_gate = place(torch.stack([get(self._expert(e, "gate")) for e in range(E)]), compute_dtype, device)
+        if self.correction_name:
+            self.correction = get(self.prefix + self.correction_name).to(torch.float32).to(device).contiguous()
+        if self.gated:
+            self.w_gate = place(torch.stack([get(self._expert(e, "gate")) for e in range(E)]), compute_dtype, device)
         self.w_up = place(torch.stack([get(self._expert(e, "up")) for e in range(E)]), compute_dtype, device)
         self.w_down = place(torch.stack([get(self._expert(e, "down")) for e in range(E)]), compute_dtype, device)
         if self.shared:
@@ -99,7 +125,11 @@ class MixtureOfExperts(Part):
         """What a token's step reads: the router, `top` experts and the shared expert."""
         item = self.w_down.element_size()
         shared = (3 * self.shared["hidden"] + 1) * self.dim if self.shared else 0
-        return (self.n_experts * self.dim + self.top * 3 * self.hidden * self.dim + shared) * item
+        return (self.n_experts * self.dim + self.top * self.matrices() * self.hidden * self.dim + shared) * item
+
+    def matrices(self):
+        """Matrices an expert has."""
+        return 3 if self.gated else 2
 
     def row_elements(self):
         return max(self.top * self.hidden, self.shared["hidden"] if self.shared else 0)
@@ -125,7 +155,10 @@ class MixtureOfExperts(Part):
         wts = ws.get("moe.weights", (T, self.top), torch.float32)
         logits = ws.get("moe.logits", (T, self.n_experts), torch.float32)        # products exact, sums in float32
         self._gemm(ctx, h, self.w_router, logits, kernels.EPI_STORE_F32)
-        kernels.moe_select(logits, ids, wts, self.renormalize, bias=self.b_router)
+        if self.sigmoid:
+            kernels.moe_select_groups(logits, self.correction, ids, wts, self.groups, self.keep_groups, self.weight_scale)
+        else:
+            kernels.moe_select(logits, ids, wts, self.renormalize, bias=self.b_router)
         if T >= GROUPED_MIN_ROWS and kernels.can_moe_grouped(self.dim, self.hidden, h.dtype, T * self.top, self.n_experts):
             return kernels.moe_grouped(h, self.w_gate, self.w_up, self.w_down, ids, wts, self.limit, self.alpha, ws.get,
                                        out, accumulate, up_shift=self.up_shift)

@@ -1,8 +1,12 @@
 """RMSNorm: out = x * rsqrt(mean(x^2) + eps) * weight, sums in float32
 (src/infer.cpp:136-146, src/infer.cu:525-539).  The parameter `tensor` names the weight behind the
 part's prefix (default "weight"); with `offset` c the stored tensor is the weight's distance from c (weight = c +
-stored, formed in float32 and kept so, whatever the compute dtype: the sum has no bfloat16 of its own).  `add_normed` is the norm of a layer that norms a sublayer's OUTPUT:
-x += norm(y)."""
+stored, formed in float32 and kept so, whatever the compute dtype: the sum has no bfloat16 of its own).  `join` is
+the norm of a layer that norms a sublayer's OUTPUT: x += norm(y).
+
+LayerNorm: out = (x - mean) / sqrt(mean of the squared deviations + eps) * weight + bias, everything in float32; the bias is
+the tensor of the weight's name with `bias_suffix` (default ".b") behind it.  Its `join` norms the SUM of the stream,
+times `stream_scale` (default 1), and the sublayer's result: x = norm(stream_scale x + y)."""
 import torch
 
 from ..ops import kernels
@@ -39,7 +43,48 @@ class RMSNorm(Part):
     def forward(self, x, out, ctx, row_index=None):
         return kernels.rmsnorm(x, self.weight, out, self.eps, row_index)
 
-    def add_normed(self, y, x, ctx, h_out=None, next_norm=None):
+    def can_hand_to(self, next_norm):
+        """True if `join` can apply next_norm to the stream it leaves."""
+        return hasattr(next_norm, "fused")
+
+    def join(self, y, x, ctx, h_out=None, next_norm=None):
         """x += norm(y) (both float32 [T, dim]); h_out, if given, receives the new x in the compute dtype, or with
         next_norm (a norm that offers fused()) that norm's output for the new x."""
         return kernels.norm_add(y, self.weight, self.eps, x, h_out, None if next_norm is None else next_norm.fused())
+
+
+@part("norm", "layernorm")
+class LayerNorm(Part):
+    def __init__(self, spec, dim, prefix):
+        super().__init__(spec, dim, prefix)
+        self.eps = float(spec.params["eps"])
+        self.tensor = self.prefix + str(spec.params.get("tensor", "weight"))
+        self.bias_tensor = self.tensor + str(spec.params.get("bias_suffix", ".b"))
+        self.stream_scale = float(spec.params.get("stream_scale", 1.0))
+        self.weight = self.bias = None
+
+    def param_specs(self):
+        return [ParamSpec(self.tensor, (self.dim,), init="norm"), ParamSpec(self.bias_tensor, (self.dim,), init="bias")]
+
+    def load(self, get, compute_dtype, device):
+        self.weight, self.bias = (get(n).to(torch.float32).to(device).contiguous() for n in (self.tensor, self.bias_tensor))
+
+    def weight_bytes(self):
+        return 2 * self.dim * 4
+
+    def joined(self):
+        """(weight, bias, eps) for a norm whose `join` applies this one to the stream it leaves."""
+        return self.weight, self.bias, self.eps
+
+    def forward(self, x, out, ctx, row_index=None):
+        return kernels.layer_norm(x, self.weight, self.bias, self.eps, out, row_index)
+
+    def join(self, y, x, ctx, h_out=None, next_norm=None):
+        """x = norm(stream_scale x + y) (both float32 [T, dim]); h_out, if given, receives the new x in the compute dtype,
+        or with next_norm (a LayerNorm) that norm's output for the new x."""
+        return kernels.layer_norm_sum(y, self.weight, self.bias, self.eps, self.stream_scale, x, h_out,
+                                      None if next_norm is None else next_norm.joined())
+
+    def can_hand_to(self, next_norm):
+        """True if `join` can apply next_norm to the stream it leaves."""
+        return hasattr(next_norm, "joined")
