@@ -8,7 +8,7 @@ shape with its window of 4,096 positions and prompts of 6,000 tokens).
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers N] [--dtype bf16|fp32] [--shape NAME]
                     [--prompt-len N] [--prefill-len N] [--batch B] [--points B,B] [--no-prefill]
                     [--kernels] [--ragged] [--sweep]
-    python bench.py --design situlorn|gedunex|bovozen|rekirax [--sizes 2048,4096] [--kernels] [--steps K] [--warmup W]
+    python bench.py --design situlorn|gedunex|bovozen|rekirax|gemepel [--sizes 2048,4096] [--kernels] [--steps K] [--warmup W]
 
 --kernels adds the time of every kernel of a decode step and of a prompt step, each taken alone at the
 shape's sizes (src/test.cpp:340-405 times single kernels so), with its rate against the peak;
@@ -22,7 +22,9 @@ prompt of --prefill-len tokens and decode steps at --batch; with --kernels every
 gedunex does the same for four layers of the Gedunex design (three shaped attentions under a window and one mLSTM,
 dense and mixture-of-experts feed-forwards) beside the Situlorn and the Llama layers, --design rekirax for four layers
 of the Rekirax design (three side-by-side mixers of a chunked rotary attention and HGRN2, one window attention, gated
-feed-forwards with biases, a way into looped layers) beside the Bovozen and the Llama layers, --design bovozen for four layers
+feed-forwards with biases, a way into looped layers) beside the Bovozen and the Llama layers, --design gemepel for four
+layers of the Gemepel design (two latent attentions with latent queries, one on the other's keys, two gated linear
+attentions, mixtures of two-matrix experts) beside the Situlorn, the Rekirax and the Llama layers, --design bovozen for four layers
 of the Bovozen design (two gated delta rules, two attentions inside blocks of positions, a two-matrix feed-forward and
 mixtures of experts beside a shared expert) beside the Gedunex and the Llama layers.  The default workload and its
 line stay as they are.
@@ -118,8 +120,9 @@ KERNEL_FACES = ("embed", "rmsnorm", "gemm", "gemm_norm", "gemm_norm_qkv_rope", "
                 "attn_decode", "sink_store", "attn_sink_mix", "argmax", "cast", "norm_add", "polynorm", "head_matmul",
                 "latent_pack", "moe_route", "moe_select", "moe_pair_gate_up", "moe_pair_down", "moe_grouped", "embed_sinusoid",
                 "qkv_pack", "v_tiles", "mlstm_scan", "mlstm_chunks", "gated_delta", "embed_learned", "activate", "gated_add",
-                "time_conv", "gated_bias_act", "sigmoid_gate", "loop_pack", "hgrn2")
-FP32_FACES = ("mlstm_scan", "mlstm_chunks", "gated_delta", "hgrn2")     # kernels of float32 multiply-adds whatever the model's dtype: priced against that peak
+                "time_conv", "gated_bias_act", "sigmoid_gate", "loop_pack", "hgrn2", "layer_norm", "layer_norm_sum", "embed_pairs",
+                "latent_norm", "moe_select_groups", "gla")
+FP32_FACES = ("mlstm_scan", "mlstm_chunks", "gated_delta", "hgrn2", "gla")     # kernels of float32 multiply-adds whatever the model's dtype: priced against that peak
 
 
 def record_kernel_calls(run):
@@ -194,14 +197,22 @@ def kernel_cost(name, a, kw, kv_tokens, torch):
         return "latent_pack %d tokens" % a[0].shape[0], nbytes(a[7]), 0.0
     if name == "norm_add":
         return "norm_add %dx%d" % tuple(a[0].shape), 3 * nbytes(a[0]), 0.0
+    if name == "layer_norm_sum":
+        return "layer_norm_sum %dx%d" % tuple(a[0].shape), 3 * nbytes(a[0]) + (nbytes(a[6]) if len(a) > 6 and a[6] is not None else 0), 0.0
+    if name == "layer_norm":
+        return "layer_norm %dx%d" % tuple(a[4].shape), 3 * nbytes(a[4]), 0.0
+    if name == "latent_norm":
+        return "latent_norm %dx%d" % (a[0].shape[0], a[1]), 4 * a[0].shape[0] * a[1] + nbytes(a[4]), 0.0
+    if name == "embed_pairs":
+        return "embed_pairs %d" % a[2].shape[0], 2 * nbytes(a[10]), 0.0
     if name == "polynorm":
         return "polynorm %dx%d" % tuple(a[0].shape), nbytes(a[0], a[3]), 0.0
     if name == "cast":
         return "cast %d" % a[0].numel(), nbytes(a[0], a[1]), 0.0
     if name == "embed_sinusoid":
         return "embed_sinusoid %d" % a[1].shape[0], 2 * nbytes(a[5]), 0.0
-    if name == "moe_select":
-        return "moe_select %d tokens" % a[0].shape[0], nbytes(a[0], a[1], a[2]), 0.0
+    if name in ("moe_select", "moe_select_groups"):
+        return "%s %d tokens" % (name, a[0].shape[0]), nbytes(a[0], a[1] if name == "moe_select" else a[3], a[2]), 0.0
     if name == "qkv_pack":
         qkv, q_out = a[0], a[10]
         T = qkv.shape[0]
@@ -236,6 +247,12 @@ def kernel_cost(name, a, kw, kv_tokens, torch):
         # per token and head: the gate's blend and the read-out, each over the d x dv state; the read-outs pass through
         # memory twice (recurrence -> heads' norm), the state once each way
         return "hgrn2 %d tokens" % T, nbytes(proj, out) + 2 * nbytes(raw) + 2 * B * H * d * dv * 4, 4.0 * T * H * d * dv
+    if name == "gla":
+        proj, raw, seq_slot, out = a[0], a[5], a[7], a[8]
+        H, d, dv = a[9], a[10], a[11]
+        T, B = proj.shape[0], seq_slot.shape[0]
+        # per token and head: the decay, the rank-one write and the read-out, each over the d x dv state; the rest as for hgrn2
+        return "gla %d tokens" % T, nbytes(proj, out) + 2 * nbytes(raw) + 2 * B * H * d * dv * 4, 5.0 * T * H * d * dv
     if name == "time_conv":
         return "time_conv %dx%d" % tuple(a[0].shape), nbytes(a[0], a[3]), 0.0
     if name == "gated_bias_act":
@@ -253,12 +270,13 @@ def kernel_cost(name, a, kw, kv_tokens, torch):
     if name == "moe_route":
         return "moe_route %d tokens" % a[0].shape[0], nbytes(a[0], a[1]), 2.0 * a[0].shape[0] * a[1].numel()
     if name in ("moe_pair_gate_up", "moe_pair_down", "moe_grouped"):
-        h, w = a[0], a[1]
+        h, w = a[0], a[2] if name == "moe_pair_gate_up" else (a[3] if name == "moe_grouped" else a[1])
+        ungated = name != "moe_pair_down" and a[1] is None           # experts of two matrices
         ids = a[4] if name == "moe_grouped" else (a[3] if name == "moe_pair_gate_up" else a[2])
         pairs = ids.numel()
         E = w.shape[0]
         per_expert = w[0].numel() * w.element_size()
-        mats = {"moe_pair_gate_up": 2, "moe_pair_down": 1, "moe_grouped": 3}[name]
+        mats = {"moe_pair_gate_up": 2, "moe_pair_down": 1, "moe_grouped": 3}[name] - (1 if ungated else 0)
         # every expert that some pair chose is read once (at most all of them)
         return "%s %d pairs" % (name, pairs), min(pairs, E) * mats * per_expert + nbytes(h), 2.0 * pairs * mats * w[0].numel()
     return name, nbytes(*a), 0.0
@@ -391,6 +409,23 @@ def rekirax_config(width, n_layers=4):
             "loop": {"start": 1, "stop": min(3, n_layers), "times": 1}, "layers": [pattern[i % 4] for i in range(n_layers)]}
 
 
+def gemepel_config(width, n_layers=4):
+    """Layers of the Gemepel design at a real model's sizes: the latent head of situlorn_config with queries through a latent
+    vector of a quarter of the width, recurrent heads of 128 x 128 with decays of rank 16, and experts of two matrices with
+    as many weights together as situlorn_config's of three, chosen inside four of eight groups."""
+    heads = width // 128
+    attn = {"heads": heads, "dim": 96, "rot_dim": 32, "vdim": 128, "q_rank": width // 4, "kv_rank": 96, "scale": 128 ** -0.5,
+            "rot": {"base": 10000.0, "dims": 32}}
+    rec = {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0, "decay_rank": 16}
+    moe = {"kind": "moe", "expert": {"ff": width * 3 // 4},
+           "router": {"experts": 32, "top": 4, "scale": 2.5, "groups": {"count": 8, "keep": 4}}}
+    pattern = [{"type": "latent_attention", "mixer": attn, "mlp": moe}, {"type": "gla", "mixer": rec, "mlp": moe},
+               {"type": "gla", "mixer": rec, "mlp": moe}, {"type": "latent_attention", "mixer": dict(attn, kv_from=0), "mlp": moe}]
+    return {"architecture": "Gemepel", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "postln_alpha": 2.0,
+            "embedding": {"scale": 1.0, "bigram": {"buckets": 65521, "mul_prev": 8191, "mul_cur": 131}},
+            "layers": [pattern[i % 4] for i in range(n_layers)]}
+
+
 def llama_config(width, n_layers=4):
     return {"architectures": ["LlamaForCausalLM"], "hidden_size": width, "intermediate_size": width * 7 // 2,
             "num_hidden_layers": n_layers, "num_attention_heads": width // 128, "num_key_value_heads": width // 512,
@@ -409,10 +444,12 @@ def bench_design(args):
     sampler = Sampler(0)
     out = {}
     for width in [int(w) for w in args.sizes.split(",") if w]:
-        own = {"gedunex": gedunex_config, "situlorn": situlorn_config, "bovozen": bovozen_config, "rekirax": rekirax_config}[args.design]
+        own = {"gedunex": gedunex_config, "situlorn": situlorn_config, "bovozen": bovozen_config, "rekirax": rekirax_config,
+               "gemepel": gemepel_config}[args.design]
         own = (args.design, own(width))
         beside = {"gedunex": (("situlorn", situlorn_config(width)),), "bovozen": (("gedunex", gedunex_config(width)),),
-                  "rekirax": (("bovozen", bovozen_config(width)),)}.get(args.design, ())
+                  "rekirax": (("bovozen", bovozen_config(width)),),
+                  "gemepel": (("situlorn", situlorn_config(width)), ("rekirax", rekirax_config(width)))}.get(args.design, ())
         for design, cfg in (own,) + beside + (("llama", llama_config(width)),):
             model = Model.random(cfg, seed=0, dtype=dtype, device="cuda:0")
             V = model.vocab_size
@@ -453,7 +490,7 @@ def bench_design(args):
             step_bytes = model.weight_bytes() + kv
             for part in model.all_parts():              # a batch reads up to batch x top experts, not one token's top
                 if hasattr(part, "n_experts"):
-                    step_bytes += (min(part.n_experts, B * part.top) - part.top) * 3 * part.hidden * part.dim * part.w_down.element_size()
+                    step_bytes += (min(part.n_experts, B * part.top) - part.top) * part.matrices() * part.hidden * part.dim * part.w_down.element_size()
             r = {"prefill_tokens": T, "prefill_ms": round(prefill_s * 1e3, 3), "prefill_tok_s": round(T / prefill_s, 1),
                  "decode_batch": B, "decode_context": int(ctx_len), "decode_ms_per_step": round(step_s * 1e3, 4),
                  "decode_tok_s": round(B / step_s, 1), "decode_step_MB": round(step_bytes / 1e6, 1),
@@ -516,7 +553,7 @@ def main():
     ap.add_argument("--context", type=int, default=0,
                     help="the reference's -T: past this many positions two attention sinks and the last "
                          "<context> - 2 positions are attended to (0: the shape's own window, if any)")
-    ap.add_argument("--design", default="", choices=["", "situlorn", "gedunex", "bovozen", "rekirax"],
+    ap.add_argument("--design", default="", choices=["", "situlorn", "gedunex", "bovozen", "rekirax", "gemepel"],
                     help="measure layers of this design beside Llama layers of equal width instead of the default workload")
     ap.add_argument("--sizes", default="2048,4096", help="widths for --design")
     args = ap.parse_args()

@@ -120,7 +120,7 @@ def gla_scan(q, k, v, a, state):
     return torch.stack(out), state
 
 
-def gla(h, m, w, p, eps, memory):
+def gla(h, m, w, p, eps, memory, faint_out=None):
     H, d, dv = int(m["heads"]), int(m["dim"]), int(m["vdim"])
     T = h.shape[0]
     q = (h @ W(w, p + "q").T).reshape(T, H, d) * d ** -0.5
@@ -131,6 +131,9 @@ def gla(h, m, w, p, eps, memory):
     state = torch.zeros((H, d, dv), dtype=F64) if state is None else state
     outs, states = zip(*[gla_scan(q[:, i], k[:, i], v[:, i], a[:, i], state[i]) for i in range(H)])
     memory["state"] = torch.stack(states)
+    if faint_out is not None:                      # a head's read-out beside the layer's median: its norm divides by it
+        size = torch.stack(outs, dim=1).pow(2).mean(dim=-1).sqrt()
+        faint_out.append((size / size.median().clamp_min(1e-30)).min(dim=-1).values)
     o = rms_norm(torch.stack(outs, dim=1), W(w, p + "norm"), eps).reshape(T, H * dv)
     return (o * silu(h @ W(w, p + "g").T)) @ W(w, p + "o").T
 
@@ -195,10 +198,10 @@ def moe(h, mlp, w, p):
 
 
 # ------------------------------------------------------------------------------------------ the model
-def mixer(i, layer, x, positions, w, eps, memory):
+def mixer(i, layer, x, positions, w, eps, memory, faint_out=None):
     m, p = layer["mixer"], "l%d.mix." % i
     if layer["type"] == "gla":
-        return gla(x, m, w, p, eps, memory.setdefault(i, {}))
+        return gla(x, m, w, p, eps, memory.setdefault(i, {}), faint_out)
     src = m.get("kv_from")
     if src is None:
         made = latent_keys(x, positions, m, w, p, eps)
@@ -207,10 +210,11 @@ def mixer(i, layer, x, positions, w, eps, memory):
     return latent_attention(x, positions, m, w, p, eps, memory[i if src is None else int(src)]["kept"])
 
 
-def forward(config, w, tokens, memory=None, start=0, layers_out=None, margins_out=None):
+def forward(config, w, tokens, memory=None, start=0, layers_out=None, margins_out=None, faint_out=None):
     """Logits [T, vocab] of one sequence's tokens at positions start.. .  memory: {} at the sequence's start, handed
     in again to go on.  layers_out: a list that receives the residual stream after every layer; margins_out: one that
-    receives route_margin [T] of every feed-forward."""
+    receives route_margin [T] of every feed-forward; faint_out: one that receives, for every recurrence, how small the
+    smallest head's read-out is beside the layer's median [T]."""
     eps, alpha = float(config["norm"]["eps"]), float(config["postln_alpha"])
     memory = {} if memory is None else memory
     tokens = [int(t) for t in tokens]
@@ -218,7 +222,7 @@ def forward(config, w, tokens, memory=None, start=0, layers_out=None, margins_ou
     x = embed(tokens, config["embedding"], w, memory)
     for i, layer in enumerate(config["layers"]):
         p = "l%d." % i
-        x = norm(alpha * x + mixer(i, layer, x, positions, w, eps, memory), w, p + "norm1", eps)
+        x = norm(alpha * x + mixer(i, layer, x, positions, w, eps, memory, faint_out), w, p + "norm1", eps)
         if layer.get("mlp"):
             if margins_out is not None:
                 margins_out.append(route_margin(x, layer["mlp"]["router"], w, p + "mlp."))

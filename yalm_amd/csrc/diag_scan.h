@@ -37,7 +37,7 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
   constexpr int EL = TOK * DP / DS_THREADS;       // elements a thread forms for a group of tokens
   constexpr int VL = (TOK * COLS + DS_THREADS - 1) / DS_THREADS;     // values it fetches (threads behind TOK * COLS: none)
   constexpr int PROW = LANES + 4;                 // shares of a column: rows apart by 16 bytes more than their length
-  static_assert(NR % 4 == 0 && DS_THREADS % DP == 0 && EL >= 1, "");
+  static_assert(NR % 4 == 0 && (LANES == 8 || LANES == 16 || LANES == 32) && DS_THREADS % DP == 0 && EL >= 1, "");
   __shared__ __attribute__((aligned(16))) float s_q[TOK][DP];
   __shared__ __attribute__((aligned(16))) float s_f[TOK][DP];
   __shared__ __attribute__((aligned(16))) float s_k[Op::KEYS ? TOK : 1][Op::KEYS ? DP : 4];
@@ -169,13 +169,17 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
     for (int k = 0; k < VL; ++k) {
       const int tt = vt + k * (DS_THREADS / COLS);
       if (tt < n && col_ok) {
-        float sum[4] = {0.f, 0.f, 0.f, 0.f};
+        float sum[LANES / 4];                     // in pairs, pairs of pairs, ...
 #pragma unroll
-        for (int i = 0; i < LANES; i += 4) {
-          const float4 a = *reinterpret_cast<const float4*>(&s_part[tt][vc][i]);
-          sum[0] += a.x, sum[1] += a.y, sum[2] += a.z, sum[3] += a.w;
+        for (int i = 0; i < LANES / 4; ++i) {
+          const float4 a = *reinterpret_cast<const float4*>(&s_part[tt][vc][4 * i]);
+          sum[i] = (a.x + a.y) + (a.z + a.w);
         }
-        raw[(size_t)(tc + tt) * HV + h * dv + c0 + vc] = (sum[0] + sum[1]) + (sum[2] + sum[3]);
+#pragma unroll
+        for (int w = LANES / 8; w > 0; w /= 2)
+#pragma unroll
+          for (int i = 0; i < w; ++i) sum[i] = sum[2 * i] + sum[2 * i + 1];
+        raw[(size_t)(tc + tt) * HV + h * dv + c0 + vc] = sum[0];
       }
     }
   }

@@ -103,9 +103,10 @@ class LatentAttention(Part):
         def pairs(w, heads):          # rotated rows of `heads` heads of r rows each, pairs made adjacent
             return interleave_rows(w, heads, r, dims) if half_split and r else w
 
-        wq = get(self._name("q")).reshape(H, d + r, -1)
-        wq = torch.cat([wq[:, :d], pairs(wq[:, d:].reshape(H * r, wq.shape[-1]), H).reshape(H, r, -1)], dim=1)
-        wq = wq.reshape(H * (d + r), -1)
+        K = self.q_rank or self.dim
+        wq = get(self._name("q")).reshape(H, d + r, K)
+        wq = torch.cat([wq[:, :d], pairs(wq[:, d:].reshape(H * r, K), H).reshape(H, r, K)], dim=1)
+        wq = wq.reshape(H * (d + r), K)
         if self.q_rank:
             self.w_uq = place(wq, compute_dtype, device)
             self.q_norm = place(get(self._name("q_norm")), compute_dtype, device)
