@@ -121,8 +121,8 @@ KERNEL_FACES = ("embed", "rmsnorm", "gemm", "gemm_norm", "gemm_norm_qkv_rope", "
                 "latent_pack", "moe_route", "moe_select", "moe_pair_gate_up", "moe_pair_down", "moe_grouped", "embed_sinusoid",
                 "qkv_pack", "v_tiles", "mlstm_scan", "mlstm_chunks", "gated_delta", "embed_learned", "activate", "gated_add",
                 "time_conv", "gated_bias_act", "sigmoid_gate", "loop_pack", "hgrn2", "layer_norm", "layer_norm_sum", "embed_pairs",
-                "latent_norm", "moe_select_groups", "gla")
-FP32_FACES = ("mlstm_scan", "mlstm_chunks", "gated_delta", "hgrn2", "gla")     # kernels of float32 multiply-adds whatever the model's dtype: priced against that peak
+                "latent_norm", "moe_select_groups", "gla", "gla_tiles")
+FP32_FACES = ("mlstm_scan", "mlstm_chunks", "gated_delta", "hgrn2", "gla", "gla_tiles")     # kernels of float32 multiply-adds whatever the model's dtype: priced against that peak
 
 
 def record_kernel_calls(run):
@@ -247,6 +247,14 @@ def kernel_cost(name, a, kw, kv_tokens, torch):
         # per token and head: the gate's blend and the read-out, each over the d x dv state; the read-outs pass through
         # memory twice (recurrence -> heads' norm), the state once each way
         return "hgrn2 %d tokens" % T, nbytes(proj, out) + 2 * nbytes(raw) + 2 * B * H * d * dv * 4, 4.0 * T * H * d * dv
+    if name == "gla_tiles":
+        proj, raw, seq_slot, n_tiles, out = a[0], a[5], a[7], a[9], a[10]
+        H, d, dv = a[11], a[12], a[13]
+        T, B = proj.shape[0], seq_slot.shape[0]
+        # per token and head: the scores against half a tile and their mix, the query on the state, the state's update; the
+        # scaled queries and keys pass through memory once each way, the read-outs three times
+        return "gla_tiles %d tokens" % T, nbytes(proj, out) + 4 * n_tiles * 64 * H * d * 4 + 4 * nbytes(raw) + 2 * B * H * d * dv * 4, \
+            T * H * (64.0 * (d + dv) + 4.0 * d * dv)
     if name == "gla":
         proj, raw, seq_slot, out = a[0], a[5], a[7], a[8]
         H, d, dv = a[9], a[10], a[11]

@@ -246,6 +246,49 @@ def test_gla_kernel(H, d, dv, rank, tau, dtype, n_first):
     assert bool(torch.isnan(state[1]).all()) and float(state[3].abs().sum()) == 0.0
 
 
+@pytest.mark.parametrize("tau,shift", [(16.0, 0.0), (1.0, 1.0), (16.0, 6.0), (0.5, -4.0)])
+@pytest.mark.parametrize("H,d,dv,rank", [(1, 4, 4, 1), (3, 5, 9, 3), (4, 32, 64, 16), (2, 33, 17, 20), (2, 64, 40, 16), (1, 128, 128, 16), (3, 100, 200, 7),
+                                         (2, 128, 70, 96)])
+def test_gla_prompts_tile_by_tile(H, d, dv, rank, tau, shift):
+    """Prompts of unequal lengths (one token to several tiles, one that ends a tile and one just behind it), from states that
+    are not zero: read-outs and states as the recurrence gives them.  Decays from nearly none to e^-15 a token, so that
+    their products over a tile run far below float32's range."""
+    from yalm_amd.ops import kernels
+    lens = [1, 64, 65, 200, 17]
+    g = gen(H * 100 + d)
+    rn = lambda *s, sc=1.0: (torch.randn(*s, generator=g, dtype=F64) * sc).float().to(F64)
+    Hd, Hv = H * d, H * dv
+    w2, bias, w_norm = rn(Hd, rank, sc=2.0 * rank ** -0.5), rn(Hd) + shift, 1 + rn(dv, sc=0.2)
+    projs = [rn(n, 2 * Hd + 2 * Hv + rank, sc=1.5) for n in lens]
+    slots = [2, 0, 5, 3, 1]
+    S0 = rn(6, H, d, dv, sc=0.3)
+    w2p = torch.zeros(Hd, kernels.gla_padded_rank(rank), dtype=F64)
+    w2p[:, :rank] = w2
+    state = f32(S0.transpose(2, 3).reshape(6, -1))
+    cu, tile0 = np.concatenate([[0], np.cumsum(lens)]), np.concatenate([[0], np.cumsum([(n + 63) // 64 for n in lens])])
+    T = int(cu[-1])
+    raw = torch.full((T, Hv), float("nan"), dtype=torch.float32, device=DEV)
+    out = torch.full((T, Hv), float("nan"), dtype=torch.float32, device=DEV)
+    scratch = lambda name, shape, dt: torch.full(shape, float("nan"), dtype=dt, device=DEV)
+    kernels.gla_tiles(f32(torch.cat(projs)), f32(w2p), f32(bias), f32(w_norm), state, raw, i32(cu), i32(slots), i32(tile0), int(tile0[-1]),
+                      out, H, d, dv, rank, d ** -0.5, tau, 1e-5, scratch)
+    for b, pr in enumerate(projs):
+        n = pr.shape[0]
+        q, k = (pr[:, i * Hd:(i + 1) * Hd].reshape(n, H, d) for i in (0, 1))
+        v, gate = pr[:, 2 * Hd:2 * Hd + Hv].reshape(n, H, dv), pr[:, 2 * Hd + Hv:2 * Hd + 2 * Hv]
+        a = P.decays(pr[:, 2 * Hd + 2 * Hv:], {"heads": H, "dim": d, "tau": tau}, {"a1": torch.eye(rank), "a2": w2, "a2.b": bias}, "")
+        outs, states = zip(*[P.gla_scan(q[:, i] * d ** -0.5, k[:, i], v[:, i], a[:, i], S0[slots[b], i]) for i in range(H)])
+        o = torch.stack(outs, dim=1)
+        got = raw[cu[b]:cu[b + 1]].cpu().to(F64).reshape(n, H, dv)
+        assert float((got - o).abs().max()) <= 3e-5 * max(1.0, float(o.abs().max())), (b, float((got - o).abs().max()))
+        S = state[slots[b]].cpu().to(F64).reshape(H, dv, d).transpose(1, 2)
+        assert float((S - torch.stack(states)).abs().max()) <= 2e-5 * max(1.0, float(S.abs().max()))
+        want = P.rms_norm(o, w_norm, 1e-5).reshape(n, Hv) * P.silu(gate)
+        err = (out[cu[b]:cu[b + 1]].cpu().to(F64) - want).abs()
+        assert float(err.max()) <= 2e-3 and float(err.mean()) <= 1e-5
+    assert torch.equal(state[4].cpu(), S0[4].transpose(1, 2).reshape(-1).float())
+
+
 @pytest.mark.parametrize("n", [300, 2048])
 def test_gla_state_is_carried_in_32_bits(n):
     """Decays close to one (0.999 and above) and far from it (a channel whose z is -60, one whose z is 60), in steps of 1 to

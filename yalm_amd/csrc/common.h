@@ -103,6 +103,15 @@ __device__ __forceinline__ float block_max(float v, float* red) {
   return s;
 }
 
+// A barrier that waits for the wave's LDS traffic only.  __syncthreads() carries a fence that also waits for every global
+// load in flight, and operands asked for ahead are meant to stay in flight across the barriers of the work before them.
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("" ::: "memory");
+  __builtin_amdgcn_s_waitcnt(0x3F | (0x7 << 4) | (0x0 << 8) | (0x3 << 14));      // lgkmcnt(0), nothing else
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
 // More than 64 KB of dynamic LDS has to be allowed for a kernel before its first launch, on every device it is
 // launched on.  One LdsAllowance (a static of the launcher) per kernel: a bit per device, set under a lock.
 struct LdsAllowance {

@@ -8,9 +8,9 @@
 // consecutive rows of NC columns in registers, so that what a lane reads of q, f and k serves NC columns (the state is
 // kept column by column, [slot][head][column][row]).  The operands of TOK tokens at a time are formed once by the whole
 // workgroup (from projections that were asked for a group ahead and waited in registers) and wait in LDS, where the
-// lanes read them four at a time; a lane leaves its share of a column's read-out in LDS and goes on to the next token,
-// and the shares of a group's tokens are summed afterwards by all threads at once, so that no token waits for an
-// exchange between lanes.
+// lanes read them four at a time; a lane (a quad of lanes, where a column has more than eight) leaves its share of a
+// column's read-out in LDS and goes on to the next token, and the shares of a group's tokens are summed afterwards by
+// all threads at once, so that no token waits for LDS to exchange between lanes.
 //
 // heads_norm_kernel: out[t, h, :] = o[t, h, :] / sqrt(mean(o[t, h, :]^2) + eps) * w, optionally times silu of a gate;
 // a wave a (token, head).
@@ -19,7 +19,7 @@
 //   KEYS                        whether k is a number of its own
 //   LOW                         whether form() reads a short vector a token (`low`, low_size() floats padded to a multiple of 4)
 //   Row begin(h, r, ok)         what a thread that forms row r of head h keeps in registers
-//   fetch(t, h, r, z)           two floats of token t's projections (plain loads; ok rows only)
+//   fetch(t, h, r, z)           two floats of token t's projections (plain loads)
 //   form(row, z, low, q, f, k)  the operands from them
 //   value(t, h, j)              v_t[j];  low(t, i) the short vector's elements
 #pragma once
@@ -27,6 +27,12 @@
 
 namespace {
 constexpr int DS_THREADS = 256;
+
+// the value of another lane of the same quad (a DPP quad_perm control)
+template <int CTRL>
+__device__ __forceinline__ float quad_swap(float v) {
+  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), CTRL, 0xF, 0xF, true));
+}
 
 template <class Op, int NR, int LANES, int NC, int TOK>
 __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __restrict__ state, float* __restrict__ raw,
@@ -36,13 +42,13 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
   constexpr int GROUPS = DS_THREADS / LANES, COLS = GROUPS * NC;
   constexpr int EL = TOK * DP / DS_THREADS;       // elements a thread forms for a group of tokens
   constexpr int VL = (TOK * COLS + DS_THREADS - 1) / DS_THREADS;     // values it fetches (threads behind TOK * COLS: none)
-  constexpr int PROW = LANES + 4;                 // shares of a column: rows apart by 16 bytes more than their length
+  constexpr int SHARES = LANES > 8 ? LANES / 4 : LANES;         // shares of a column's read-out that go through LDS
   static_assert(NR % 4 == 0 && (LANES == 8 || LANES == 16 || LANES == 32) && DS_THREADS % DP == 0 && EL >= 1, "");
   __shared__ __attribute__((aligned(16))) float s_q[TOK][DP];
   __shared__ __attribute__((aligned(16))) float s_f[TOK][DP];
   __shared__ __attribute__((aligned(16))) float s_k[Op::KEYS ? TOK : 1][Op::KEYS ? DP : 4];
   __shared__ __attribute__((aligned(16))) float s_v[TOK][COLS];
-  __shared__ __attribute__((aligned(16))) float s_part[TOK][COLS][PROW];
+  __shared__ __attribute__((aligned(16))) float s_part[TOK][COLS][SHARES];
   extern __shared__ __attribute__((aligned(16))) float s_low[];              // Op::LOW: [2][TOK][padded size]
   const int b = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * COLS, tid = threadIdx.x;
   const int group = tid / LANES, rl = tid % LANES, j0 = c0 + group * NC, r0 = rl * NR;
@@ -81,21 +87,18 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
   auto fetch = [&](int tc) {                      // a group's operands into registers: asked for a group ahead
 #pragma unroll
     for (int k = 0; k < EL; ++k) {
-      const int t = tc + gt + k * (DS_THREADS / DP);
-      z[k][0] = z[k][1] = 0.f;
-      if (row_ok && t < t1) op.fetch(t, h, gr, z[k]);
+      op.fetch(min(tc + gt + k * (DS_THREADS / DP), t1 - 1), h, min(gr, d - 1), z[k]);      // no branch: what lies behind is not used
     }
 #pragma unroll
     for (int k = 0; k < VL; ++k) {
-      const int t = tc + vt + k * (DS_THREADS / COLS);
-      zv[k] = col_ok && t < t1 ? op.value(t, h, c0 + vc) : 0.f;
+      zv[k] = op.value(min(tc + vt + k * (DS_THREADS / COLS), t1 - 1), h, min(c0 + vc, dv - 1));
     }
   };
   auto low_at = [&](int tc, int i) {              // element i of the group's short vectors, tokens one behind the other
     const int t = tc + i / rp, e = i % rp;
     return t < t1 && e < op.low_size() ? op.low(t, e) : 0.f;
   };
-  fetch(t0);
+  if (t1 > t0) fetch(t0);
   if constexpr (Op::LOW) {                        // the short vectors are a group further ahead: LDS holds the group's, a register the next one's
     for (int i = tid; i < TOK * rp; i += DS_THREADS) s_low[i] = low_at(t0, i);
     if (tid < TOK * rp) zl = low_at(t0 + TOK, tid);
@@ -103,17 +106,22 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
   int turn = 0;
   for (int tc = t0; tc < t1; tc += TOK, turn ^= 1) {
     const int n = min(TOK, t1 - tc);
-    __syncthreads();                              // the group before is read
-#pragma unroll
-    for (int k = 0; k < EL; ++k) {
+    lds_barrier();                              // the group before is read
+    auto form = [&](int k) {
       const int tt = gt + k * (DS_THREADS / DP);
-      if (tt < n) {
-        float q, f, kk = 0.f;
-        op.form(mine, z[k], s_low + (turn * TOK + tt) * rp, q, f, kk);
-        s_q[tt][gr] = row_ok ? q : 0.f;
-        s_f[tt][gr] = row_ok ? f : 0.f;
-        if constexpr (Op::KEYS) s_k[tt][gr] = row_ok ? kk : 0.f;
-      }
+      float q, f, kk = 0.f;
+      op.form(mine, z[k], s_low + (turn * TOK + tt) * rp, q, f, kk);
+      s_q[tt][gr] = row_ok ? q : 0.f;
+      s_f[tt][gr] = row_ok ? f : 0.f;
+      if constexpr (Op::KEYS) s_k[tt][gr] = row_ok ? kk : 0.f;
+    };
+    if (n == TOK) {                               // a whole group: no branch between a thread's elements
+#pragma unroll
+      for (int k = 0; k < EL; ++k) form(k);
+    } else {
+#pragma unroll
+      for (int k = 0; k < EL; ++k)
+        if (gt + k * (DS_THREADS / DP) < n) form(k);
     }
 #pragma unroll
     for (int k = 0; k < VL; ++k)
@@ -126,7 +134,7 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
         if (tid < TOK * rp && tc + 2 * TOK < t1) zl = low_at(tc + 2 * TOK, tid);
       }
     }
-    __syncthreads();
+    lds_barrier();
     auto token = [&](int tt) {
       float v[NC], acc[NC][2];
 #pragma unroll
@@ -155,7 +163,16 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
           }
       }
 #pragma unroll
-      for (int c = 0; c < NC; ++c) s_part[tt][group * NC + c][rl] = acc[c][0] + acc[c][1];
+      for (int c = 0; c < NC; ++c) {
+        float sum = acc[c][0] + acc[c][1];
+        if constexpr (LANES > 8) {                // the four lanes of a quad first
+          sum += quad_swap<0xB1>(sum);            // lane ^ 1
+          sum += quad_swap<0x4E>(sum);            // lane ^ 2
+          if ((rl & 3) == 0) s_part[tt][group * NC + c][rl >> 2] = sum;
+        } else {
+          s_part[tt][group * NC + c][rl] = sum;
+        }
+      }
     };
     if (n == TOK) {                               // a whole group: its tokens unrolled, so that a token's reads of LDS stand under the token before
 #pragma unroll
@@ -163,20 +180,20 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
     } else {
       for (int tt = 0; tt < n; ++tt) token(tt);
     }
-    __syncthreads();
+    lds_barrier();
     // a column's read-out is the sum over its lanes: VL (token, column) pairs a thread
 #pragma unroll
     for (int k = 0; k < VL; ++k) {
       const int tt = vt + k * (DS_THREADS / COLS);
       if (tt < n && col_ok) {
-        float sum[LANES / 4];                     // in pairs, pairs of pairs, ...
+        float sum[SHARES / 4];                    // in pairs, pairs of pairs, ...
 #pragma unroll
-        for (int i = 0; i < LANES / 4; ++i) {
+        for (int i = 0; i < SHARES / 4; ++i) {
           const float4 a = *reinterpret_cast<const float4*>(&s_part[tt][vc][4 * i]);
           sum[i] = (a.x + a.y) + (a.z + a.w);
         }
 #pragma unroll
-        for (int w = LANES / 8; w > 0; w /= 2)
+        for (int w = SHARES / 8; w > 0; w /= 2)
 #pragma unroll
           for (int i = 0; i < w; ++i) sum[i] = sum[2 * i] + sum[2 * i + 1];
         raw[(size_t)(tc + tt) * HV + h * dv + c0 + vc] = sum[0];

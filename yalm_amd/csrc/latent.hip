@@ -94,17 +94,47 @@ __global__ __launch_bounds__(HM_THREADS) void head_matmul_kernel(const TI* __res
 }
 
 // out[r, :n] = x[r, :n] / sqrt(mean over those n of x^2 + eps) * w, the rows of x `x_row` apart: the norm of a latent
-// vector that is a part of a wider product.  A wave a row.
-template <typename TW, typename TO>
-__global__ __launch_bounds__(4 * WAVE) void latent_norm_kernel(const float* __restrict__ x, long x_row, const TW* __restrict__ w,
-                                                               float eps, TO* __restrict__ out, int R, int n) {
-  const int r = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-  if (r >= R) return;
-  const float* row = x + (size_t)r * x_row;
+// vector that is a part of a wider product.  A workgroup of NT threads a row; PER > 0: the row fits PER values a thread,
+// asked for together with their weights and kept in registers; PER = 0: any length.
+template <typename TW, typename TO, int NT, int PER>
+__global__ __launch_bounds__(NT) void latent_norm_kernel(const float* __restrict__ x, long x_row, const TW* __restrict__ w,
+                                                         float eps, TO* __restrict__ out, int n) {
+  __shared__ float red[NT / WAVE];
+  const float* row = x + (size_t)blockIdx.x * x_row;
+  TO* o = out + (size_t)blockIdx.x * n;
   float ss = 0.f;
-  for (int i = lane; i < n; i += WAVE) ss = fmaf(row[i], row[i], ss);
-  const float s = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
-  for (int i = lane; i < n; i += WAVE) out[(size_t)r * n + i] = from_f32<TO>(row[i] * s * to_f32(w[i]));
+  if constexpr (PER > 0) {
+    float v[PER], g[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int i = threadIdx.x + j * NT;
+      v[j] = i < n ? row[i] : 0.f;
+      g[j] = i < n ? to_f32(w[i]) : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < PER; ++j) ss = fmaf(v[j], v[j], ss);
+    const float s = 1.0f / sqrtf(block_sum<NT / WAVE>(ss, red) / (float)n + eps);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int i = threadIdx.x + j * NT;
+      if (i < n) o[i] = from_f32<TO>(v[j] * s * g[j]);
+    }
+  } else {
+    for (int i = threadIdx.x; i < n; i += NT) ss = fmaf(row[i], row[i], ss);
+    const float s = 1.0f / sqrtf(block_sum<NT / WAVE>(ss, red) / (float)n + eps);
+    for (int i = threadIdx.x; i < n; i += NT) o[i] = from_f32<TO>(row[i] * s * to_f32(w[i]));
+  }
+}
+
+template <typename TW, typename TO>
+int latent_norm_launch(const float* x, long x_row, const void* w, float eps, void* out, int R, int n, hipStream_t stream) {
+#define LN(NT_, PER_) latent_norm_kernel<TW, TO, NT_, PER_><<<R, NT_, 0, stream>>>(x, x_row, (const TW*)w, eps, (TO*)out, n)
+  if (n <= 128) LN(64, 2);
+  else if (n <= 1024) LN(256, 4);
+  else if (n <= 2048) LN(256, 8);
+  else LN(256, 0);
+#undef LN
+  return launch_status();
 }
 
 // One wave a (token, job).  job < H: the rotated part of query head `job`, scaled, and zeros behind the
@@ -319,15 +349,13 @@ extern "C" int yalm_latent_norm(const float* x, long x_row, const void* w, int w
                                 int R, int n, hipStream_t stream) {
   if (R <= 0) return YALM_OK;
   if (n <= 0 || x_row < n) return YALM_ERR_ARG;
-  const int blocks = ceil_div(R, 4);
-#define LN(TW_, TO_) latent_norm_kernel<TW_, TO_><<<blocks, 4 * WAVE, 0, stream>>>(x, x_row, (const TW_*)w, eps, (TO_*)out, R, n)
+#define LN(TW_, TO_) return latent_norm_launch<TW_, TO_>(x, x_row, w, eps, out, R, n, stream)
   if (w_dtype == YALM_F32 && out_dtype == YALM_F32) LN(float, float);
-  else if (w_dtype == YALM_F32 && out_dtype == YALM_BF16) LN(float, bf16);
-  else if (w_dtype == YALM_BF16 && out_dtype == YALM_F32) LN(bf16, float);
-  else if (w_dtype == YALM_BF16 && out_dtype == YALM_BF16) LN(bf16, bf16);
-  else return YALM_ERR_DTYPE;
+  if (w_dtype == YALM_F32 && out_dtype == YALM_BF16) LN(float, bf16);
+  if (w_dtype == YALM_BF16 && out_dtype == YALM_F32) LN(bf16, float);
+  if (w_dtype == YALM_BF16 && out_dtype == YALM_BF16) LN(bf16, bf16);
 #undef LN
-  return launch_status();
+  return YALM_ERR_DTYPE;
 }
 
 extern "C" int yalm_latent_pack(const float* queries, long q_row, int q_head, int q_rot_off, const float* kv, long kv_row,

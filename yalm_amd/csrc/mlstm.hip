@@ -133,15 +133,6 @@ constexpr int DVS = 64;                           // columns of S a workgroup ow
 constexpr int VROW = DVS + 16;                    // LDS row strides (floats)
 constexpr float NEVER = -3.0e38f;
 
-// A barrier that waits for the wave's LDS traffic only.  __syncthreads() carries a fence that also waits for every global
-// load in flight, and the next chunk's operands are meant to stay in flight across the barriers of this chunk's work.
-__device__ __forceinline__ void lds_barrier() {
-  asm volatile("" ::: "memory");
-  __builtin_amdgcn_s_waitcnt(0x3F | (0x7 << 4) | (0x0 << 8) | (0x3 << 14));      // lgkmcnt(0), nothing else
-  __builtin_amdgcn_s_barrier();
-  asm volatile("" ::: "memory");
-}
-
 template <int L>
 __host__ __device__ constexpr size_t chunk_lds_floats(int d16) {
   return (size_t)d16 * VROW + 2 * (size_t)L * (d16 + 4) + (size_t)L * VROW + (size_t)L * (L + 4) + d16 + 8 * L;

@@ -156,6 +156,13 @@ __global__ __launch_bounds__(WAVE) void moe_select_groups_kernel(const float* __
     }
     if (at == 0x7fffffff) at = 0;                 // nothing finite is left
   };
+  // the place of v[at] among v[0 .. n) by falling value, the lower index first among equals
+  auto place = [&](const float* v, int n, int at) {
+    const float mine = v[at];
+    int before = 0;
+    for (int i = 0; i < n; ++i) before += v[i] > mine || (v[i] == mine && i < at);
+    return before;
+  };
   if (keep < n_groups) {
     for (int g = lane; g < n_groups; g += WAVE) {
       float a = -INFINITY, b = -INFINITY;
@@ -166,27 +173,27 @@ __global__ __launch_bounds__(WAVE) void moe_select_groups_kernel(const float* __
       group[g] = per > 1 ? a + b : a;
     }
     __syncthreads();
-    // the kept groups are marked by plus infinity one after another, the others' experts then drop out
-    for (int k = 0; k < keep; ++k) {
-      float best = -INFINITY;
-      int at = 0x7fffffff;
-      for (int g = lane; g < n_groups; g += WAVE) {
-        const float x = group[g];
-        if (x != INFINITY && x > best) { best = x; at = g; }
-      }
-      for (int o = WAVE / 2; o > 0; o >>= 1) {
-        const float ob = __shfl_xor(best, o, WAVE);
-        const int oa = __shfl_xor(at, o, WAVE);
-        if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
-      }
-      if (lane == 0 && at < n_groups) group[at] = INFINITY;
-      __syncthreads();
-    }
     for (int e = lane; e < E; e += WAVE)
-      if (group[e / per] != INFINITY) choice[e] = -INFINITY;
+      if (place(group, n_groups, e / per) >= keep) choice[e] = -INFINITY;
     __syncthreads();
   }
   float total = 0.f;
+  if (E <= 2 * WAVE) {                            // few experts: everyone counts its own place
+    float mine = 0.f;
+    for (int e = lane; e < E; e += WAVE) {
+      const int k = place(choice, E, e);
+      if (k < top) {
+        ids[(size_t)t * top + k] = e;
+        mine += score[e];
+      }
+    }
+    total = wave_sum(mine) + 1e-20f;
+    for (int e = lane; e < E; e += WAVE) {
+      const int k = place(choice, E, e);
+      if (k < top) wts[(size_t)t * top + k] = score[e] / total * scale;
+    }
+    return;
+  }
   for (int k = 0; k < top; ++k) {
     int at;
     largest(choice, E, at);

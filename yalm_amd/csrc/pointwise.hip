@@ -55,7 +55,21 @@ __global__ void embed_pairs_kernel(const T* __restrict__ table, const T* __restr
   }
   const T* row = table + (size_t)tok * D;
   const T* pr = pair_table + (size_t)r * D;
-  for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = fmaf(to_f32(row[i]), scale, to_f32(pr[i]));
+  constexpr int PER = 16 / sizeof(T);             // elements of a 16-byte load
+  if (D % PER == 0 && ((((uintptr_t)table) | ((uintptr_t)pair_table) | ((uintptr_t)out)) & 15) == 0) {
+    for (int i = threadIdx.x * PER; i < D; i += blockDim.x * PER) {
+      const uint4 a4 = *reinterpret_cast<const uint4*>(row + i), b4 = *reinterpret_cast<const uint4*>(pr + i);
+      const T* a = reinterpret_cast<const T*>(&a4);
+      const T* b = reinterpret_cast<const T*>(&b4);
+#pragma unroll
+      for (int u = 0; u < PER; u += 4)
+        *reinterpret_cast<float4*>(o + i + u) =
+            make_float4(fmaf(to_f32(a[u]), scale, to_f32(b[u])), fmaf(to_f32(a[u + 1]), scale, to_f32(b[u + 1])),
+                        fmaf(to_f32(a[u + 2]), scale, to_f32(b[u + 2])), fmaf(to_f32(a[u + 3]), scale, to_f32(b[u + 3])));
+    }
+  } else {
+    for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = fmaf(to_f32(row[i]), scale, to_f32(pr[i]));
+  }
 }
 
 // activation codes: 0 the gelu with the error function, z/2 (1 + erf(z / sqrt(2))); 1 its tanh form; 2 silu
@@ -265,7 +279,7 @@ extern "C" int yalm_embed_pairs(const void* table, const void* pair_table, int d
                                 long mul_cur, long buckets, float scale, float* out, int T, int D, int V, hipStream_t stream) {
   if (T <= 0) return YALM_OK;
   if (D <= 0 || V <= 0 || buckets <= 0) return YALM_ERR_ARG;
-  const int threads = D >= 1024 ? 1024 : (D >= 256 ? 256 : 64);
+  const int threads = D >= 2048 ? 512 : (D >= 256 ? 256 : 64);
   if (dtype == YALM_F32)
     embed_pairs_kernel<float><<<T, threads, 0, stream>>>((const float*)table, (const float*)pair_table, tokens, tok_seq, tok_pos,
                                                          cu_seqlens, seq_slot, last, mul_prev, mul_cur, buckets, scale, out, D, V);

@@ -441,6 +441,15 @@ int yalm_gla(const float* proj, const float* w2, const float* bias, const float*
              const int* cu_seqlens, const int* seq_slot, void* out, int T, int B, int n_heads, int d, int dv, int rank,
              float q_scale, float inv_tau, float eps, int out_dtype, hipStream_t stream);
 
+// The same for steps of prompts, a tile of 64 tokens at a time on the matrix cores (float32): seq_tile0 int32 [B + 1] the
+// first tile of every sequence (ceil(tokens / 64) tiles each, n_tiles in all), DP = yalm_gla_tiles_fit(d, rank) the padded
+// key size (0: these sizes are not taken), scratch qd, kd float32 [n_tiles, H, 64, DP] and gd float32 [n_tiles, H, DP].
+int yalm_gla_tiles_fit(int d, int rank);
+int yalm_gla_tiles(const float* proj, const float* w2, const float* bias, const float* w_norm, float* state, float* raw, float* qd,
+                   float* kd, float* gd, const int* cu_seqlens, const int* seq_slot, const int* seq_tile0, int n_tiles, void* out,
+                   int T, int B, int n_heads, int d, int dv, int rank, float q_scale, float inv_tau, float eps, int out_dtype,
+                   hipStream_t stream);
+
 // Yardsticks for the measurement (probes.hip): a kernel that only reads `bytes` bytes once with `workgroups`
 // workgroups (out: 1,024 words of scratch), and a loop of matrix-core instructions on registers (shape 32:
 // v_mfma_f32_32x32x16_bf16, 16: v_mfma_f32_16x16x32_bf16; *flops, host memory, receives the launch's operations).

@@ -1280,6 +1280,37 @@ def gla(proj, w2, bias, w_norm, state, raw, cu_seqlens, seq_slot, out, n_heads, 
     return out
 
 
+GLA_TILES_MIN_TOKENS = 32         # tokens a sequence (on average) from which a step of prompts goes tile by tile
+
+
+def gla_tiles_fit(d, rank):
+    """The padded key size with which gla_tiles takes key heads of d and decays of this rank, or 0: it does not."""
+    return library.lib().yalm_gla_tiles_fit(int(d), int(rank))
+
+
+def gla_tiles(proj, w2, bias, w_norm, state, raw, cu_seqlens, seq_slot, seq_tile0, n_tiles, out, n_heads, d, dv, rank, q_scale,
+              tau, eps, scratch):
+    """gla for a step of prompts, a tile of 64 tokens at a time on the matrix cores in float32; seq_tile0 int32 [B + 1], the
+    first tile of every sequence (n_tiles in all).  scratch(name, shape, dtype) hands out the buffers."""
+    T, B = proj.shape[0], seq_slot.shape[0]
+    N = 2 * n_heads * d + 2 * n_heads * dv + rank
+    dp = gla_tiles_fit(d, rank)
+    if not dp:
+        raise ValueError("gla_tiles: key heads of %d with decays of rank %d are not taken" % (d, rank))
+    qd = scratch("gla.qd", (n_tiles, n_heads, PAGE, dp), torch.float32)
+    kd = scratch("gla.kd", (n_tiles, n_heads, dp, PAGE), torch.float32)
+    gd = scratch("gla.gd", (n_tiles, n_heads, dp), torch.float32)
+    library.check(library.lib().yalm_gla_tiles(
+        _need(proj, "proj", torch.float32, (T, N)), _need(w2, "w2", torch.float32, (n_heads * d, gla_padded_rank(rank))),
+        _need(bias, "bias", torch.float32, (n_heads * d,)), _need(w_norm, "w_norm", torch.float32, (dv,)),
+        _need(state, "state", torch.float32, (None, n_heads * d * dv)), _need(raw, "raw", torch.float32, (T, n_heads * dv)),
+        qd.data_ptr(), kd.data_ptr(), gd.data_ptr(), _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)),
+        _need(seq_slot, "seq_slot", torch.int32, (B,)), _need(seq_tile0, "seq_tile0", torch.int32, (B + 1,)), n_tiles,
+        _need(out, "out", None, (T, n_heads * dv)), T, B, n_heads, d, dv, rank, float(q_scale), 1.0 / float(tau), float(eps),
+        dtype_code(out.dtype), _stream()), "gla_tiles")
+    return out
+
+
 # ---------------------------------------------------------------------------------------------------------------
 # mixture of experts
 MOE_MAX_EXPERTS = 1024

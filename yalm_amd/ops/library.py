@@ -60,6 +60,8 @@ _SIGNATURES = {
     "yalm_layer_norm": (_I, [_P, _P, _F, _P, _P, _P, _F, _I, _P, _I, _P, _P, _F, _I, _I, _P]),
     "yalm_embed_pairs": (_I, [_P, _P, _I, _P, _P, _P, _P, _P, _P, ctypes.c_long, ctypes.c_long, ctypes.c_long, _F, _P, _I, _I, _I, _P]),
     "yalm_moe_select_groups": (_I, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P]),
+    "yalm_gla_tiles_fit": (_I, [_I, _I]),
+    "yalm_gla_tiles": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]),
     "yalm_gla": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]),
     "yalm_moe_route": (_I, [_P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P]),
     "yalm_moe_select": (_I, [_P, _P, _P, _P, _I, _I, _I, _I, _P]),

@@ -7,12 +7,14 @@ per head
     S <- diag(f) S + k v^T;   o = S^T q
 (the read-out sees the token's own write).  Each head's o is divided by its root mean square, multiplied by a weight
 shared by the heads and by silu(W_g h), and W_o carries the heads to the stream.  q | k | v | g | W_1 h are one product
-with float32 results; everything behind it is float32, the small product with W_2 included (ops.kernels.gla)."""
+with float32 results; everything behind it is float32, the small product with W_2 included (ops.kernels.gla: token by
+token; gla_tiles, steps of prompts: 64 tokens at a time on the matrix cores)."""
 import torch
 
 from ..cache.manager import StateRequest
 from ..ops import kernels
 from ..weights.loader import ParamSpec, place
+from .attention import kv_tiles
 from .base import Part, part
 
 NAMES = {"q": "q", "k": "k", "v": "v", "gate": "g", "decay_in": "a1", "decay_out": "a2", "decay_bias": "a2.b", "norm": "norm",
@@ -21,6 +23,8 @@ NAMES = {"q": "q", "k": "k", "v": "v", "gate": "g", "decay_in": "a1", "decay_out
 
 @part("mixer", "gla")
 class GatedLinearAttention(Part):
+    prompt_tables = (kv_tiles,)
+
     def __init__(self, spec, dim, prefix):
         super().__init__(spec, dim, prefix)
         p = spec.params
@@ -75,8 +79,8 @@ class GatedLinearAttention(Part):
         return 2 * self.qk + 2 * self.vv + self.decay_rank
 
     def describe(self, compute_dtype):
-        return "gated linear attention, %d heads of %d x %d, decays of rank %d: state columns in the registers of a group of " \
-               "lanes, float32" % (self.n_heads, self.key_dim, self.value_dim, self.decay_rank), False
+        return "gated linear attention, %d heads of %d x %d, decays of rank %d: float32, prompts by tiles of 64 tokens on the " \
+               "matrix cores, single tokens with state columns in the registers of a group of lanes" % (self.n_heads, self.key_dim, self.value_dim, self.decay_rank), False
 
     def forward(self, h, x, ctx, line, writes_cache=True):
         """Adds the mixer's result to the stream x."""
@@ -94,6 +98,15 @@ class GatedLinearAttention(Part):
         raw = ws.get("gla.raw", (T, self.vv), torch.float32)
         o = ws.get("gla.o", (T, self.vv), h.dtype)
         state = ctx.cache.group_of(line).line_state(line)
-        kernels.gla(proj, self.w2, self.decay_bias, self.w_norm, state, raw, ctx.cu_seqlens, ctx.seq_slot, o, self.n_heads,
-                    self.key_dim, self.value_dim, self.decay_rank, self.q_scale, self.tau, self.eps)
+        B = ctx.seq_slot.shape[0]
+        sizes = (self.n_heads, self.key_dim, self.value_dim, self.decay_rank, self.q_scale, self.tau, self.eps)
+        # With float32 as the compute dtype prompts go token by token too: the decays' products are then formed one factor
+        # at a time, without the rounding of their logarithms' sums.
+        if ctx.mode == "prefill" and h.dtype == torch.bfloat16 and T >= kernels.GLA_TILES_MIN_TOKENS * B and not kernels.FORCE_SIMPLE \
+                and kernels.gla_tiles_fit(self.key_dim, self.decay_rank):
+            tiles = ctx.tables["kv_tiles"]
+            kernels.gla_tiles(proj, self.w2, self.decay_bias, self.w_norm, state, raw, ctx.cu_seqlens, ctx.seq_slot,
+                              tiles["seq_tile0"], tiles["n_tiles"], o, *sizes, ws.get)
+        else:
+            kernels.gla(proj, self.w2, self.decay_bias, self.w_norm, state, raw, ctx.cu_seqlens, ctx.seq_slot, o, *sizes)
         self._gemm(ctx, o, self.wo, x, epilogue)
