@@ -579,7 +579,10 @@ def masked_attention_float64(q, k, v, n_heads, n_kv, hd, window, bias=None):
                                                          (32, 8, 128, 0, [2048]), (40, 8, 96, 0, [1500]),
                                                          (40, 10, 32, 200, [2200, 70]), (12, 4, 96, 0, [1300]),
                                                          (40, 8, 80, 0, [1500]), (24, 8, 48, 100, [2300, 65]),
-                                                         (12, 4, 16, 0, [1300]), (40, 8, 112, 0, [1700])])
+                                                         (12, 4, 16, 0, [1300]), (40, 8, 112, 0, [1700]),
+                                                         (16, 1, 144, 0, [1500, 70]), (32, 1, 160, 0, [700]), (9, 1, 176, 100, [600, 129]),
+                                                         (20, 4, 192, 0, [900, 1]), (16, 1, 208, 0, [300]), (8, 2, 224, 0, [640]),
+                                                         (5, 1, 240, 70, [400, 65]), (16, 1, 256, 0, [700, 64])])
 def test_attn_prefill_with_many_and_with_few_workgroups(n_heads, n_kv, hd, window, lens):
     """The matrix-core prefill kernel has two forms: workgroups of eight waves that take a tile's keys in two
     halves (launches of at most two workgroups a compute unit, the third case) and of four waves (more, the
@@ -691,7 +694,10 @@ def one_query_reference(q, keys, vals, window):
     (8, 2, 128, 0, [1000, 3], 7), (2, 2, 80, 0, [129], 4), (32, 8, 128, 0, [300], 2), (5, 5, 64, 70, [700, 64], 16),
     (6, 2, 96, 0, [900, 65, 2], 5), (12, 3, 96, 130, [400, 129], 2), (16, 1, 32, 0, [2000, 7], 9),
     (10, 2, 112, 0, [777, 3], 4), (9, 3, 80, 64, [500, 64], 3), (4, 4, 16, 0, [129, 1000], 5),
-    (34, 2, 64, 0, [300, 65], 3), (40, 1, 128, 100, [700], 4), (51, 3, 32, 0, [129, 2], 2)])   # more than 16 heads a group
+    (34, 2, 64, 0, [300, 65], 3), (40, 1, 128, 100, [700], 4), (51, 3, 32, 0, [129, 2], 2),   # more than 16 heads a group
+    (16, 1, 144, 0, [700, 3], 4), (32, 1, 160, 0, [300], 2), (20, 1, 176, 100, [400, 64], 3), (8, 2, 192, 0, [900, 65], 5),
+    (16, 1, 208, 0, [129], 1), (5, 1, 224, 0, [500, 2], 4), (3, 3, 240, 70, [300], 2), (16, 1, 256, 0, [700, 64], 3),
+    (40, 2, 256, 0, [333], 1)])   # one wide head
 def test_attn_decode(n_heads, n_kv, hd, window, lens, splits, dtype, simple):
     _attn_decode_case(n_heads, n_kv, hd, window, lens, splits, dtype, simple, None)
 

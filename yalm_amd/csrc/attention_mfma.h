@@ -36,9 +36,12 @@ __device__ __forceinline__ bf16x8 ld8_once(const bf16* p) {
 // page row that MFMA row i (0..15) of key tile t (0..3) reads
 __device__ __forceinline__ int key_row(int t, int i) { return 32 * (t >> 1) + 8 * (i >> 2) + 4 * (t & 1) + (i & 3); }
 
-// head sizes the kernels are built for: 16 to 128 in steps of 16
-bool mfma_shape_ok(int n_heads, int n_kv_heads, int head_dim) {
-  return head_dim >= 16 && head_dim <= 128 && head_dim % 16 == 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0;
+// head sizes the kernels are built for: 16 to 128 in steps of 16, and without a shape on the scores up to MFMA_WIDE
+// (a latent attention's one wide head)
+constexpr int MFMA_WIDE = 256;
+bool mfma_shape_ok(int n_heads, int n_kv_heads, int head_dim, bool shaped) {
+  return head_dim >= 16 && head_dim <= (shaped ? 128 : MFMA_WIDE) && head_dim % 16 == 0 && n_kv_heads > 0 &&
+         n_heads % n_kv_heads == 0;
 }
 
 }  // namespace

@@ -21,7 +21,7 @@ namespace {
 // BIAS: the scores are shaped (ScoreShape: a cap, a term by the distance of query and key, bias[head][min(distance,
 // n_bias - 1)], a learned logit in the denominator; each optional).
 template <int HD, int NW, bool BLOCKS, bool BIAS>
-__global__ __launch_bounds__(NW * WAVE, NW == 4 ? 2 : 1) void attn_decode_mfma_kernel(   // 2 waves a SIMD: head size 128 needs their registers
+__global__ __launch_bounds__(NW * WAVE, NW == 4 && HD <= 128 ? 2 : 1) void attn_decode_mfma_kernel(   // 2 waves a SIMD: head size 128 needs their registers; a wide head those of one
     const bf16* __restrict__ q, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ block_table, int table_stride, int ring_pages, const int* __restrict__ seq_slot,
     const int* __restrict__ seq_len, float* __restrict__ partial, bf16* __restrict__ out, float* __restrict__ lse,
@@ -257,7 +257,7 @@ int yalm_attn_decode_bf16_mfma(const void* q, const void* k_pages, const void* v
   const bool shaped = shape.any();
   // with sinks the merge kernel always runs: it takes them in, also where there is one split
   const bool merge = n_splits > 1 || sinks.n_sinks > 0;
-  if (!mfma_shape_ok(n_heads, n_kv_heads, head_dim)) return YALM_ERR_ARG;
+  if (!mfma_shape_ok(n_heads, n_kv_heads, head_dim, shaped)) return YALM_ERR_ARG;
   // a score bias: the engine's layout of the pages only (blocks where the head size allows), and no sinks (they are
   // scored without it)
   if ((bias != nullptr && n_bias <= 0) ||
@@ -287,7 +287,25 @@ int yalm_attn_decode_bf16_mfma(const void* q, const void* k_pages, const void* v
     if (shaped) YALM_DECODE(HD_, 4, false, true);                                \
     else YALM_DECODE(HD_, 4, false, false);                                         \
     break
+  // wide heads, never shaped; 256 with two waves, whose results to merge fill 32 KB of LDS where four waves' would pass 64
+#define YALM_DECODE_WIDE32(HD_, NW_)                                                \
+  case HD_:                                                                         \
+    if (blocks) YALM_DECODE(HD_, NW_, true, false);                                 \
+    else YALM_DECODE(HD_, NW_, false, false);                                       \
+    break
+#define YALM_DECODE_WIDE16(HD_)                                                     \
+  case HD_:                                                                         \
+    YALM_DECODE(HD_, 4, false, false);                                              \
+    break
   switch (head_dim) {
+    YALM_DECODE_WIDE16(144);
+    YALM_DECODE_WIDE32(160, 4);
+    YALM_DECODE_WIDE16(176);
+    YALM_DECODE_WIDE32(192, 4);
+    YALM_DECODE_WIDE16(208);
+    YALM_DECODE_WIDE32(224, 4);
+    YALM_DECODE_WIDE16(240);
+    YALM_DECODE_WIDE32(256, 2);
     YALM_DECODE_HD16(16);
     YALM_DECODE_HD32(32);
     YALM_DECODE_HD16(48);
@@ -297,6 +315,8 @@ int yalm_attn_decode_bf16_mfma(const void* q, const void* k_pages, const void* v
     YALM_DECODE_HD16(112);
     YALM_DECODE_HD32(128);
   }
+#undef YALM_DECODE_WIDE16
+#undef YALM_DECODE_WIDE32
 #undef YALM_DECODE_HD32
 #undef YALM_DECODE_HD16
 #undef YALM_DECODE

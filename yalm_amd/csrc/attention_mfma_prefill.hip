@@ -25,7 +25,7 @@ namespace {
 // BIAS: the scores are shaped (ScoreShape: a cap, a term by the distance of query and key, bias[head][min(distance,
 // n_bias - 1)], a learned logit in the denominator; each optional).
 template <int HD, int NC, int KSPL, bool BIAS>
-__global__ __launch_bounds__(256 * KSPL, KSPL == 1 ? 2 : 1) void attn_prefill_mfma_kernel(
+__global__ __launch_bounds__(256 * KSPL, KSPL == 1 && HD <= 144 ? 2 : 1) void attn_prefill_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_stage, const bf16* __restrict__ v_stage,
     bf16* __restrict__ out, float* __restrict__ out_f32, float* __restrict__ lse, const int* __restrict__ cu_seqlens,
     const int* __restrict__ seq_tile0, const int* __restrict__ tile_order, int fold_at, int B, int n_heads,
@@ -362,6 +362,22 @@ int launch_prefill_hd(int head_dim, bool biased, Args... args) {
 #undef YALM_PREFILL_HD
   return YALM_ERR_ARG;
 }
+template <typename... Args>
+int launch_prefill_wide(int head_dim, Args... args) {
+#define YALM_PREFILL_WIDE(HD_) case HD_: return launch_prefill<HD_, 2, 1, false>(args...)
+  switch (head_dim) {
+    YALM_PREFILL_WIDE(144);
+    YALM_PREFILL_WIDE(160);
+    YALM_PREFILL_WIDE(176);
+    YALM_PREFILL_WIDE(192);
+    YALM_PREFILL_WIDE(208);
+    YALM_PREFILL_WIDE(224);
+    YALM_PREFILL_WIDE(240);
+    YALM_PREFILL_WIDE(256);
+  }
+#undef YALM_PREFILL_WIDE
+  return YALM_ERR_ARG;
+}
 }  // namespace
 
 int yalm_attn_prefill_bf16_mfma(const void* q, const void* k_stage, const void* v_stage, void* out, float* out_f32,
@@ -369,14 +385,18 @@ int yalm_attn_prefill_bf16_mfma(const void* q, const void* k_stage, const void* 
                                 const int* cu_seqlens, const int* seq_tile0, const int* tile_order, int n_order,
                                 int T, int B, int n_tiles, int n_heads, int n_kv_heads, int head_dim, int window,
                                 const ScoreShape& shape, hipStream_t stream) {
-  if (!mfma_shape_ok(n_heads, n_kv_heads, head_dim) || n_tiles > 65535) return YALM_ERR_ARG;
-  if (shape.bias != nullptr && shape.n_bias <= 0) return YALM_ERR_ARG;
   const bool biased = shape.any();
+  if (!mfma_shape_ok(n_heads, n_kv_heads, head_dim, biased) || n_tiles > 65535) return YALM_ERR_ARG;
+  if (shape.bias != nullptr && shape.n_bias <= 0) return YALM_ERR_ARG;
   if (tile_order && (n_order <= 0 || n_order > n_tiles)) return YALM_ERR_ARG;
   dim3 grid(n_heads, tile_order ? n_order : n_tiles);
   const long total = (long)grid.x * grid.y;
   const size_t tile_bytes = ((size_t)PAGE * (head_dim + 8) + (size_t)head_dim * (PAGE + 8)) * sizeof(bf16);
   const bf16 *qp = (const bf16*)q, *kp = (const bf16*)k_stage, *vp = (const bf16*)v_stage;
+  // A wide head: two buffers of keys and values fill up to 141 KB of LDS, so four waves a workgroup are the one form.
+  if (head_dim > 128)
+    return launch_prefill_wide(head_dim, grid, 256, 2 * tile_bytes, stream, qp, kp, vp, (bf16*)out, out_f32, lse, cu_seqlens,
+                               seq_tile0, tile_order, (int)total, B, n_heads, n_kv_heads, window, shape);
   // Few workgroups (at most two a compute unit, as a prompt of 2,048 tokens with 32 heads makes): the launch
   // would last as long as the workgroup that sees the most keys, so eight waves take each workgroup's keys
   // in two halves (2,048 tokens: 72 against 78 us; 512 tokens 1.6 % of the prompt step).  More workgroups

@@ -48,10 +48,11 @@ def kv_tiles(n_tok):
 kv_tiles.name = "kv_tiles"
 
 
-def decode_splits(n_heads, n_kv_heads, head_dim, B, max_pages, ragged=False):
+def decode_splits(n_heads, n_kv_heads, head_dim, B, max_pages, ragged=False, shaped=False):
     """Into how many pieces a decode step's attention cuts every sequence, so that about TARGET_WORKGROUPS
-    workgroups run."""
-    mfma = head_dim in kernels.MFMA_HEAD_DIMS and not kernels.FORCE_SIMPLE
+    workgroups run.  shaped: the scores have a shape (a bias, a cap, ...), which the wide heads' kernels do not take."""
+    mfma = (head_dim in kernels.MFMA_HEAD_DIMS or (head_dim in kernels.MFMA_WIDE_HEAD_DIMS and not shaped)) \
+        and not kernels.FORCE_SIMPLE
     if mfma:         # a workgroup of 4 waves per (split, KV head and up to 16 of its query heads, sequence), a page per wave at a time
         per = max(1, B * n_kv_heads * ((n_heads // n_kv_heads + 15) // 16))
         quarters = max(1, min((max_pages + 3) // 4, 4))
@@ -135,13 +136,14 @@ class GQAttention(Part):
             (", window %d" % self.window if self.window else "") + (" + %d sinks" % self.sinks if self.sinks else ""))
         if compute_dtype != torch.bfloat16:
             return what + ": float32-arithmetic kernels", False
-        if self.head_dim in kernels.MFMA_HEAD_DIMS:
+        if self.head_dim in kernels.MFMA_HEAD_DIMS or (self.head_dim in kernels.MFMA_WIDE_HEAD_DIMS
+                                                       and not hasattr(self.position, "score_bias")):
             return what + ": matrix-core kernels", False
         return what + ": float32-arithmetic kernels on bfloat16 storage (the matrix-core kernels take head sizes " \
-                      "of 16 to 128 in steps of 16, not %d): correct, several times slower" % self.head_dim, True
+                      "of 16 to 256 in steps of 16, to 128 with a score bias, not %d): correct, many times slower" % self.head_dim, True
 
     def decode_splits(self, B, max_pages, ragged=False):
-        return decode_splits(self.n_heads, self.n_kv_heads, self.head_dim, B, max_pages, ragged)
+        return decode_splits(self.n_heads, self.n_kv_heads, self.head_dim, B, max_pages, ragged, shaped=hasattr(self.position, "score_bias"))
 
     def fuses_norm(self, norm, x, ctx):
         if not hasattr(norm, "fused") or self.head_dim % 16:

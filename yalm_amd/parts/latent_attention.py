@@ -141,10 +141,10 @@ class LatentAttention(Part):
             self.n_heads, self.padded, self.rot_dim, self.rank, ", window %d" % self.window if self.window else "")
         if compute_dtype != torch.bfloat16:
             return what + ": float32-arithmetic kernels", False
-        if self.padded in kernels.MFMA_HEAD_DIMS:
+        if self.padded in kernels.MFMA_HEAD_DIMS + kernels.MFMA_WIDE_HEAD_DIMS:
             return what + ": matrix-core attention kernels", False
         return what + ": float32-arithmetic attention kernels on bfloat16 storage (the matrix-core kernels take " \
-                      "head sizes up to 128, not %d): correct, several times slower" % self.padded, True
+                      "head sizes up to 256, not %d): correct, a hundred times slower and more" % self.padded, True
 
     # ------------------------------------------------------------------ the step
     def forward(self, h, x, ctx, line, writes_cache=True):

@@ -243,7 +243,7 @@ class ShapedAttention(Part):
                                  tiles.get("tile_order"), score_bias=self.score_bias, softcap=self.softcap,
                                  sink_logit=self.sink, slopes=self.slopes, block=self.block, log_distance=self.log_ab)
         else:
-            n_splits = decode_splits(H, G, P, T, min(group.ring_pages, ctx.pages_bucket), ctx.ragged)
+            n_splits = decode_splits(H, G, P, T, min(group.ring_pages, ctx.pages_bucket), ctx.ragged, shaped=True)
             partial = ws.get("attn.partial", (kernels.attn_decode_workspace_floats(T, H, P, n_splits),), torch.float32)
             kernels.attn_decode(q, k_pages, v_pages, group.table, group.ring_pages, ctx.seq_slot, ctx.seq_len, o, partial,
                                 H, G, P, self.window, n_splits, step_max_len=ctx.step_max_len, seq_order=ctx.seq_order,
