@@ -238,6 +238,49 @@ __global__ __launch_bounds__(4 * WAVE) void heads_norm_kernel(const float* __res
   }
 }
 
+// The gated form for dv a multiple of 4 up to 256: LPR lanes a (token, head), four elements a lane, everything asked for
+// before the first sum.
+template <typename T, int LPR>
+__global__ __launch_bounds__(4 * WAVE) void heads_norm_gate_kernel(const float* __restrict__ raw, const float* __restrict__ w,
+                                                                  const float* __restrict__ gate, long gate_row, T* __restrict__ out,
+                                                                  long n_rows, int n_heads, int dv, float eps) {
+  const long row = (long)blockIdx.x * (4 * WAVE / LPR) + threadIdx.x / LPR;
+  const int i = threadIdx.x % LPR * 4;
+  const bool ok = row < n_rows && i < dv;
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f), g = v, ww = v;
+  if (ok) {
+    v = *reinterpret_cast<const float4*>(raw + row * dv + i);
+    g = *reinterpret_cast<const float4*>(gate + (row / n_heads) * gate_row + (row % n_heads) * dv + i);
+    ww = *reinterpret_cast<const float4*>(w + i);
+  }
+  float ss = (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+#pragma unroll
+  for (int o = LPR / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+  const float f = 1.0f / sqrtf(ss / (float)dv + eps);
+  auto gated = [&](float x, float y, float z) { return x * f * y * (z / (1.0f + expf(-z))); };
+  if (ok) {
+    T* o = out + row * dv + i;
+    o[0] = from_f32<T>(gated(v.x, ww.x, g.x));
+    o[1] = from_f32<T>(gated(v.y, ww.y, g.y));
+    o[2] = from_f32<T>(gated(v.z, ww.z, g.z));
+    o[3] = from_f32<T>(gated(v.w, ww.w, g.w));
+  }
+}
+
+template <typename T>
+int heads_norm_gate_launch(const float* raw, const float* w, const float* gate, long gate_row, void* out, long n_rows, int n_heads,
+                           int dv, float eps, hipStream_t stream) {
+#define HN(LPR_)                                                                                                         \
+  heads_norm_gate_kernel<T, LPR_><<<ceil_div(n_rows, 4 * WAVE / LPR_), 4 * WAVE, 0, stream>>>(raw, w, gate, gate_row, (T*)out, \
+                                                                                             n_rows, n_heads, dv, eps)
+  if (dv <= 32) HN(8);
+  else if (dv <= 64) HN(16);
+  else if (dv <= 128) HN(32);
+  else HN(64);
+#undef HN
+  return launch_status();
+}
+
 template <class Op, int NR, int LANES, int NC, int TOK>
 int diag_scan_launch(const Op& op, float* state, float* raw, const int* cu_seqlens, const int* seq_slot, int B, int n_heads,
                      int d, int dv, size_t low_elements, hipStream_t stream) {
@@ -252,6 +295,10 @@ int diag_scan_launch(const Op& op, float* state, float* raw, const int* cu_seqle
 static inline int heads_norm_launch(const float* raw, const float* w, const float* gate, long gate_row, void* out, int T, int n_heads,
                                     int dv, float eps, int out_dtype, hipStream_t stream) {
   const long n_rows = (long)T * n_heads;
+  if (gate != nullptr && dv % 4 == 0 && dv <= 256 && gate_row % 4 == 0 &&
+      ((((uintptr_t)raw) | ((uintptr_t)w) | ((uintptr_t)gate)) & 15) == 0)
+    return out_dtype == YALM_F32 ? heads_norm_gate_launch<float>(raw, w, gate, gate_row, out, n_rows, n_heads, dv, eps, stream)
+                                 : heads_norm_gate_launch<bf16>(raw, w, gate, gate_row, out, n_rows, n_heads, dv, eps, stream);
   const int blocks = ceil_div(n_rows, 4);
   if (out_dtype == YALM_F32)
     heads_norm_kernel<float><<<blocks, 4 * WAVE, 0, stream>>>(raw, w, gate, gate_row, (float*)out, n_rows, n_heads, dv, eps);
