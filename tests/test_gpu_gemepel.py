@@ -76,7 +76,7 @@ def test_layer_norm_kernels(R_, D, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("D,V,bigram", [(5, 11, (7, 3, 2)), (300, 50, (1, 5, 9)), (1100, 40, (509, 101, 7)), (64, 90000, (65521, 1 << 20, 999983))])
+@pytest.mark.parametrize("D,V,bigram", [(5, 11, (7, 3, 2)), (300, 50, (1, 5, 9)), (1100, 40, (487, 101, 13)), (64, 90000, (65521, 1 << 20, 999983))])
 def test_embedding_of_token_pairs(D, V, bigram, dtype):
     """Two texts in pieces of several tokens and of one, beside a padding row; products of token and multiplier beyond 32
     bits; the previous token is kept per slot."""
@@ -111,7 +111,7 @@ def test_embedding_of_token_pairs(D, V, bigram, dtype):
     assert at == [12, 9] and int(last[0]) == 123 and int(last[2]) == 123
 
 
-@pytest.mark.parametrize("E,top,groups,keep,scale", [(12, 4, 2, 1, 2.0), (12, 3, 4, 2, 1.0), (1, 1, 1, 1, 0.5), (6, 2, 6, 3, 1.5), (6, 6, 1, 1, 1.0),
+@pytest.mark.parametrize("E,top,groups,keep,scale", [(14, 5, 2, 1, 1.8), (12, 3, 4, 2, 1.0), (1, 1, 1, 1, 0.5), (6, 2, 6, 3, 1.5), (6, 6, 1, 1, 1.0),
                                                      (64, 8, 8, 4, 2.5), (256, 8, 8, 4, 2.5), (300, 5, 100, 2, 1.0), (1024, 9, 2, 2, 1.0)])
 def test_choice_inside_groups(E, top, groups, keep, scale):
     """Corrections from strongly negative to strongly positive (all choice scores negative, all positive, mixed), so that
@@ -189,7 +189,7 @@ def test_latent_norm(R_, n, row, dtype):
 @pytest.mark.parametrize("n_first", [3, 40])
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,d,dv,rank,tau", [(1, 4, 4, 1, 1.0), (4, 32, 64, 16, 16.0), (3, 5, 9, 3, 0.5), (2, 64, 40, 20, 16.0), (1, 128, 70, 16, 8.0),
-                                             (1, 200, 33, 64, 16.0), (2, 16, 200, 7, 4.0), (5, 36, 31, 256, 2.0), (2, 256, 16, 256, 16.0), (3, 48, 64, 17, 16.0)])
+                                             (1, 200, 33, 64, 16.0), (2, 16, 200, 7, 4.0), (5, 36, 31, 256, 2.0), (2, 256, 16, 256, 16.0), (3, 44, 60, 17, 12.0)])
 def test_gla_kernel(H, d, dv, rank, tau, dtype, n_first):
     """Two sequences and a padding row: first pieces as a step of prompts, then single tokens, against the plain recurrence
     over the whole texts; the state left behind against the plain one (it is kept column by column)."""

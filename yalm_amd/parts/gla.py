@@ -44,6 +44,7 @@ class GatedLinearAttention(Part):
         self.names.update(p.get("tensors") or {})
         self.qk = self.n_heads * self.key_dim
         self.vv = self.n_heads * self.value_dim
+        self.proj_cols = 2 * self.qk + 2 * self.vv + self.decay_rank
         self.w_in = self.wo = self.w2 = self.decay_bias = self.w_norm = None
 
     def _n(self, key):
@@ -76,7 +77,8 @@ class GatedLinearAttention(Part):
         return StateRequest((kernels.gla_state_elements(self.n_heads, self.key_dim, self.value_dim),), torch.float32)
 
     def row_elements(self):
-        return 2 * self.qk + 2 * self.vv + self.decay_rank
+        padded = next((p for p in (32, 64, 128) if p >= self.key_dim), 0)          # a scaled query's row in gla_tiles
+        return max(self.proj_cols, self.n_heads * padded)
 
     def describe(self, compute_dtype):
         return "gated linear attention, %d heads of %d x %d, decays of rank %d: float32, prompts by tiles of 64 tokens on the " \
@@ -93,7 +95,7 @@ class GatedLinearAttention(Part):
     def _run(self, h, x, ctx, line, epilogue):
         T = h.shape[0]
         ws = ctx.ws
-        proj = ws.get("gla.proj", (T, self.row_elements()), torch.float32)
+        proj = ws.get("gla.proj", (T, self.proj_cols), torch.float32)
         self._gemm(ctx, h, self.w_in, proj, kernels.EPI_STORE_F32)
         raw = ws.get("gla.raw", (T, self.vv), torch.float32)
         o = ws.get("gla.o", (T, self.vv), h.dtype)
