@@ -12,6 +12,7 @@ from .gedunex import GedunexConfig
 from .gemepel import GemepelConfig
 from .rekirax import RekiraxConfig
 from .situlorn import SitulornConfig
+from .zebivik import ZebivikConfig
 
 _ARCHITECTURES = {}
 
@@ -65,6 +66,6 @@ def _folder_shapes(path):
     return shapes.get
 
 
-for _cls in (LlamaConfig, SitulornConfig, GedunexConfig, BovozenConfig, RekiraxConfig, GemepelConfig):
+for _cls in (LlamaConfig, SitulornConfig, GedunexConfig, BovozenConfig, RekiraxConfig, GemepelConfig, ZebivikConfig):
     for _name in _cls.ARCHITECTURES:
         register_architecture(_name, _cls)

@@ -60,10 +60,23 @@ template <> __device__ __forceinline__ bf16 from_f32<bf16>(float v) { return sta
 // (src/infer.cpp:189-195): silu(z) = z / (1 + exp(-z)); gelu(z) = z/2 (1 + tanh(0.797885 (z + 0.044715 z^3))).
 constexpr int EPI_GATED_SILU = 3, EPI_GATED_GELU = 5;
 constexpr bool gated(int epilogue) { return epilogue == EPI_GATED_SILU || epilogue == EPI_GATED_GELU; }
+// What a gated epilogue writes: the columns of its result, and the unit's constants.  limit > 0 clamps the gate from above
+// and the up value on both sides; the unit is then g sigmoid(alpha g) (u + shift) (1 and 0 make it silu(g) u).
+struct GateOut {
+  int n;
+  float limit = 0.f, alpha = 1.f, shift = 0.f;
+  __host__ __device__ explicit GateOut(int n_) : n(n_) {}
+  __host__ __device__ GateOut(int n_, float limit_, float alpha_, float shift_) : n(n_), limit(limit_), alpha(alpha_), shift(shift_) {}
+  __host__ __device__ operator int() const { return n; }
+};
 template <int EPI>
-__device__ __forceinline__ float gate_act(float z) {
-  if constexpr (EPI == EPI_GATED_GELU) return 0.5f * z * (1.0f + tanhf(0.797885f * (z + 0.044715f * z * z * z)));
-  return z / (1.0f + expf(-z));
+__device__ __forceinline__ float gate_unit(float g, float u, const GateOut& out) {
+  if constexpr (EPI == EPI_GATED_GELU) return 0.5f * g * (1.0f + tanhf(0.797885f * (g + 0.044715f * g * g * g))) * u;
+  if (out.limit > 0.f) {
+    g = fminf(g, out.limit);
+    u = fminf(fmaxf(u, -out.limit), out.limit);
+  }
+  return g / (1.0f + expf(-out.alpha * g)) * (u + out.shift);
 }
 
 __device__ __forceinline__ float wave_sum(float v) {

@@ -21,7 +21,7 @@
 //   Row begin(h, r, ok)         what a thread that forms row r of head h keeps in registers
 //   fetch(t, h, r, z)           two floats of token t's projections (plain loads)
 //   form(row, z, low, q, f, k)  the operands from them
-//   value(t, h, j)              v_t[j];  low(t, i) the short vector's elements
+//   value(t, h, j), act(z)      a plain load of what v_t[j] is made of, and v_t[j] from it;  low(t, i) the short vector's elements
 #pragma once
 #include "common.h"
 
@@ -125,7 +125,7 @@ __global__ __launch_bounds__(DS_THREADS) void diag_scan_kernel(Op op, float* __r
     }
 #pragma unroll
     for (int k = 0; k < VL; ++k)
-      if (vt + k * (DS_THREADS / COLS) < TOK) s_v[vt + k * (DS_THREADS / COLS)][vc] = zv[k];
+      if (vt + k * (DS_THREADS / COLS) < TOK) s_v[vt + k * (DS_THREADS / COLS)][vc] = Op::act(zv[k]);
     if (tc + TOK < t1) {
       fetch(tc + TOK);
       if constexpr (Op::LOW) {

@@ -76,13 +76,13 @@ __device__ __forceinline__ bf16x8 load8(const bf16* p, bool ok) {
 // epilogue codes as in yalm_gemm: 0 float32 store, 1 bfloat16 store, 2 float32 add, 3 and 5 gated
 template <int EPI>
 __device__ __forceinline__ void store_tile(void* Cv, const f32x4& v, const f32x4& u, int m_base, int n, int hcol,
-                                           int M, int N, int H) {
+                                           int M, int N, GateOut H) {
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     int m = m_base + r;
     if (m >= M) continue;
     if (gated(EPI)) {
-      if (hcol < H) ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_act<EPI>(v[r]) * u[r]);
+      if (hcol < H) ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_unit<EPI>(v[r], u[r], H));
     } else if (n < N) {
       size_t o = (size_t)m * N + n;
       if (EPI == 0) ((float*)Cv)[o] = v[r];
@@ -98,7 +98,7 @@ __global__ __launch_bounds__(NWAVES * WAVE) void gemm_batch_kernel(const bf16* _
                                                                     const bf16* __restrict__ W,
                                                                     void* __restrict__ Cv,
                                                                     float* __restrict__ partial, int M, int N, int K,
-                                                                    int H, int k_per_slice, int always_partial,
+                                                                    GateOut H, int k_per_slice, int always_partial,
                                                                     RowScale rs) {
   __shared__ __attribute__((aligned(16))) bf16 xs[2][MT * 16 * XROW];
   constexpr int NTHREADS = NWAVES * WAVE;
@@ -234,7 +234,7 @@ __global__ __launch_bounds__(NW * WAVE) void gemm_batch_dma_kernel(const bf16* _
                                                                         const bf16* __restrict__ W,
                                                                         void* __restrict__ Cv,
                                                                         float* __restrict__ partial, int M, int N,
-                                                                        int K, int H, int k_per_slice,
+                                                                        int K, GateOut H, int k_per_slice,
                                                                         int always_partial, RowScale rs) {
   constexpr int KD = 64;
   constexpr int WSTAGE = NTW * 2048;             // a wave's weight rows of a stage
@@ -358,7 +358,7 @@ __global__ __launch_bounds__(NW * WAVE) void gemm_batch_dma_kernel(const bf16* _
 // launches one of the two kernels: the DMA one (NW waves; up to 128 rows) where K and the slices are
 // multiples of 64, else the register one (8 waves; up to 64 rows)
 template <int MT, int NTW, int EPI, int NW>
-int launch_kernel(dim3 grid, const bf16* X, const bf16* W, void* C, float* ws, int M, int N, int K, int H,
+int launch_kernel(dim3 grid, const bf16* X, const bf16* W, void* C, float* ws, int M, int N, int K, GateOut H,
                   int k_per_slice, int always_partial, const RowScale& rs, hipStream_t stream) {
   if (K % 64 == 0 && k_per_slice % 64 == 0) {
     constexpr int XG0 = MT <= 2 ? 4 : (MT <= 4 ? 8 : 16);
@@ -382,7 +382,7 @@ int launch_kernel(dim3 grid, const bf16* X, const bf16* W, void* C, float* ws, i
 
 // adds the K slices in order and applies the epilogue; a thread per (row, 4 columns)
 template <int EPI>
-__global__ void splitk_reduce_kernel(const float* __restrict__ partial, void* __restrict__ Cv, int M, int N, int H,
+__global__ void splitk_reduce_kernel(const float* __restrict__ partial, void* __restrict__ Cv, int M, int N, GateOut H,
                                      int slices) {
   const int cols4 = (gated(EPI)) ? (N / 2) / 4 : (N + 3) / 4;     // gated: N = 32 * blocks, a thread per 4 hidden columns
   const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
@@ -403,7 +403,7 @@ __global__ void splitk_reduce_kernel(const float* __restrict__ partial, void* __
     const float gv[4] = {g.x, g.y, g.z, g.w}, uv[4] = {u.x, u.y, u.z, u.w};
 #pragma unroll
     for (int e = 0; e < 4; ++e)
-      if (c4 + e < H) C[c4 + e] = static_cast<bf16>(gate_act<EPI>(gv[e]) * uv[e]);
+      if (c4 + e < H) C[c4 + e] = static_cast<bf16>(gate_unit<EPI>(gv[e], uv[e], H));
   } else {
     float v[4] = {0.f, 0.f, 0.f, 0.f};
     const float* p = partial + (size_t)m * N + c4;
@@ -447,7 +447,7 @@ void slice_k(int K, int wanted, int* k_per_slice, int* slices) {
 }
 
 template <int MT, int EPI, int NW, int NTW_ = 0>
-int launch_nw(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, int H,
+int launch_nw(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, GateOut H,
               const RowScale& rs, hipStream_t stream) {
   constexpr int NTW = NTW_ ? NTW_ : (gated(EPI) ? 2 : 1);
   if constexpr (NTW_ == 0 && !gated(EPI) && MT <= 4 && NW <= 4) {
@@ -469,7 +469,7 @@ int launch_nw(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, 
 }
 
 template <int MT, int EPI>
-int launch_mt(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, int H,
+int launch_mt(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, GateOut H,
               const RowScale& rs, hipStream_t stream) {
   // waves a workgroup of the DMA kernel (they share the activations' stage): measured at batch 64
   // 8 waves 8120, 4 waves 8580, 2 waves 8410 tokens a second; at batch 32 5490, 5740 and 5870; with more than 64
@@ -703,7 +703,7 @@ int launch_add_norm_nw(const bf16* X, const bf16* W, float* C, float* ws, long w
   if (ws == nullptr || (long)slices * M * N > ws_floats) return YALM_ERR_ARG;
   slice_k(K, slices, &k_per_slice, &slices);
   dim3 grid(n_blocks, slices);
-  int rc = launch_kernel<MT, NTW, 2, NW>(grid, X, W, C, ws, M, N, K, 0, k_per_slice, 1, RowScale{nullptr, 0, 0.f}, stream);
+  int rc = launch_kernel<MT, NTW, 2, NW>(grid, X, W, C, ws, M, N, K, GateOut(0), k_per_slice, 1, RowScale{nullptr, 0, 0.f}, stream);
   if (rc != YALM_OK) return rc;
   return launch_reduce_add_norm(ws, C, norm_w, eps, h, M, N, slices, stream, emit_ss);
 }
@@ -733,7 +733,7 @@ int launch_partial_nw(const bf16* X, const bf16* W, float* ws, long ws_floats, i
   slice_k(K, slices, &k_per_slice, &slices);
   *slices_out = slices;
   dim3 grid(n_blocks, slices);
-  return launch_kernel<MT, NTW, 0, NW>(grid, X, W, ws, ws, M, N, K, 0, k_per_slice, 1, rs, stream);
+  return launch_kernel<MT, NTW, 0, NW>(grid, X, W, ws, ws, M, N, K, GateOut(0), k_per_slice, 1, rs, stream);
 }
 
 template <int MT>
@@ -746,7 +746,7 @@ int launch_partial(const bf16* X, const bf16* W, float* ws, long ws_floats, int 
 }
 
 template <int EPI>
-int dispatch(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, int H,
+int dispatch(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, GateOut H,
              const RowScale& rs, hipStream_t stream) {
   switch ((M + 15) / 16) {
     case 2: return launch_mt<2, EPI>(X, W, C, ws, ws_floats, M, N, K, H, rs, stream);
@@ -765,7 +765,7 @@ int dispatch(const bf16* X, const bf16* W, void* C, float* ws, long ws_floats, i
 // null: one slice then).  ss (may be null): the producer's partial sums of squares [M][n_parts] for the row scale.
 // Refuses (YALM_ERR_ARG) what it does not take.
 static int gemm_batch_scaled(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M,
-                             int N, int K, int epilogue, int H, const float* ss, int n_parts, float eps,
+                             int N, int K, int epilogue, GateOut H, const float* ss, int n_parts, float eps,
                              hipStream_t stream) {
   if (M <= 16 || M > (K % 64 == 0 ? 128 : 64) || K % 8 != 0 || ((uintptr_t)A & 15) || ((uintptr_t)W & 15))
     return YALM_ERR_ARG;
@@ -784,15 +784,16 @@ static int gemm_batch_scaled(const void* A, const void* W, void* C, float* works
 }
 
 int yalm_gemm_bf16_batch(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                         int K, int epilogue, int H, hipStream_t stream) {
+                         int K, int epilogue, GateOut H, hipStream_t stream) {
   return gemm_batch_scaled(A, W, C, workspace, workspace_floats, M, N, K, epilogue, H, nullptr, 0, 0.f, stream);
 }
 
 // yalm_gemm for 17..128 bfloat16 rows (more than 64: K a multiple of 64) whose activations came from yalm_gemm_add_emit:
 // the sums are scaled per row by rsqrt(sum(ss[m, :]) / K + eps).  Refuses (YALM_ERR_ARG) other shapes.
 extern "C" int yalm_gemm_scaled(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M,
-                                int N, int K, int epilogue, int H, const float* ss, int n_parts, float eps,
+                                int N, int K, int epilogue, int hidden, const float* ss, int n_parts, float eps,
                                 hipStream_t stream) {
+  const GateOut H(hidden);
   if (ss == nullptr) return YALM_ERR_ARG;
   if (gated(epilogue) && (H <= 0 || N != 32 * ((H + 15) / 16))) return YALM_ERR_ARG;
   return gemm_batch_scaled(A, W, C, workspace, workspace_floats, M, N, K, epilogue, H, ss, n_parts, eps, stream);
@@ -880,7 +881,7 @@ extern "C" int yalm_gemm_add_emit_parts(int N) { return emit_parts(N); }
 
 // Adds `slices` float32 partial products [slices][M][N] in order and applies the epilogue (for the
 // kernels that split K: this file's and the tiled one of gemm_dma.hip).
-int yalm_splitk_reduce(const float* partial, void* C, int M, int N, int H, int slices, int epilogue,
+int yalm_splitk_reduce(const float* partial, void* C, int M, int N, GateOut H, int slices, int epilogue,
                        hipStream_t stream) {
   const long items = (long)M * (gated(epilogue) ? (N / 2) / 4 : (N + 3) / 4);
   const int blocks = ceil_div(items, 256);

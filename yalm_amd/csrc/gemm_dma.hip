@@ -23,7 +23,7 @@
 #include "yalm_hip.h"
 #include <type_traits>
 
-int yalm_splitk_reduce(const float* partial, void* C, int M, int N, int H, int slices, int epilogue,
+int yalm_splitk_reduce(const float* partial, void* C, int M, int N, GateOut H, int slices, int epilogue,
                        hipStream_t stream);                                  // gemm_batch.hip
 
 namespace {
@@ -50,7 +50,7 @@ template <int EPI, int TM, int TN, int S, int NWM, int NWN, int MINW>
 __global__ __launch_bounds__(NWM * NWN * WAVE, MINW) void gemm_dma_kernel(const bf16* __restrict__ A,
                                                                          const bf16* __restrict__ W,
                                                                          void* __restrict__ Cv, int M, int N, int K,
-                                                                         int H, float* __restrict__ partial,
+                                                                         GateOut H, float* __restrict__ partial,
                                                                          int tiles_per_slice, int n_tile0) {
   constexpr int NW = NWM * NWN;
   constexpr int ROWS = TM + TN;                    // A rows, then W rows
@@ -179,7 +179,7 @@ __global__ __launch_bounds__(NWM * NWN * WAVE, MINW) void gemm_dma_kernel(const 
         for (int pp = 0; pp < FB / 2; ++pp) {
           const int hcol = (n0 + wn * WN + pp * 64) / 2 + li;
           if (hcol < H)
-            ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_act<EPI>(acc[a][2 * pp][r]) * acc[a][2 * pp + 1][r]);
+            ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_unit<EPI>(acc[a][2 * pp][r], acc[a][2 * pp + 1][r], H));
         }
       } else {
 #pragma unroll
@@ -197,7 +197,7 @@ __global__ __launch_bounds__(NWM * NWN * WAVE, MINW) void gemm_dma_kernel(const 
 }
 
 template <int EPI, int TM, int TN, int S, int NWM, int NWN, int MINW>
-int launch_shape(const bf16* A, const bf16* W, void* C, int M, int N, int K, int H, float* partial, int slices,
+int launch_shape(const bf16* A, const bf16* W, void* C, int M, int N, int K, GateOut H, float* partial, int slices,
                  hipStream_t stream, bool add_slices = true, int n_tile0 = 0, int n_tiles = -1) {
   const int tiles_per_slice = ceil_div(K / TK, slices);
   if (n_tiles < 0) n_tiles = ceil_div(N, TN) - n_tile0;     // column tiles n_tile0 ... of this launch
@@ -242,7 +242,7 @@ __host__ __device__ constexpr int dma_place(int d, int n_dma, int n_products) {
 
 template <int EPI, int TN, int MAP>
 __global__ __launch_bounds__(512, 1) void gemm_ring_kernel(const bf16* __restrict__ A, const bf16* __restrict__ W,
-                                                           void* __restrict__ Cv, int M, int N, int K, int H, int n_tile0,
+                                                           void* __restrict__ Cv, int M, int N, int K, GateOut H, int n_tile0,
                                                            int n_tiles, float* __restrict__ partial,
                                                            int tiles_per_slice) {
   constexpr int TM = RING_TM, NW = 8, NWM = 4, NWN = 2, WM = TM / NWM, WN = TN / NWN, FA = WM / 32, FB = WN / 32;
@@ -438,7 +438,7 @@ __global__ __launch_bounds__(512, 1) void gemm_ring_kernel(const bf16* __restric
         for (int pp = 0; pp < FB / 2; ++pp) {
           const int hcol = (n0 + wn * WN + pp * 64) / 2 + li;
           if (hcol < H)
-            ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_act<EPI>(acc[a][2 * pp][r]) * acc[a][2 * pp + 1][r]);
+            ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_unit<EPI>(acc[a][2 * pp][r], acc[a][2 * pp + 1][r], H));
         }
       } else {
 #pragma unroll
@@ -469,7 +469,7 @@ __global__ __launch_bounds__(512, 1) void gemm_ring_kernel(const bf16* __restric
 // ---------------------------------------------------------------------------
 template <int EPI, int TN, int MAP>
 __global__ __launch_bounds__(512, 1) void gemm_ring16_kernel(const bf16* __restrict__ A, const bf16* __restrict__ W,
-                                                             void* __restrict__ Cv, int M, int N, int K, int H,
+                                                             void* __restrict__ Cv, int M, int N, int K, GateOut H,
                                                              int n_tile0, int n_tiles, float* __restrict__ partial,
                                                              int tiles_per_slice) {
   constexpr int TM = RING_TM, NW = 8, NWM = 4, NWN = 2, WM = TM / NWM, WN = TN / NWN, FA = WM / 16, FB = WN / 16;
@@ -662,7 +662,7 @@ __global__ __launch_bounds__(512, 1) void gemm_ring16_kernel(const bf16* __restr
         for (int pp = 0; pp < FB / 2; ++pp) {
           const int hcol = (n0 + wn * WN) / 2 + pp * 16 + l16;
           if (hcol < H)
-            ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_act<EPI>(acc[a][2 * pp][r]) * acc[a][2 * pp + 1][r]);
+            ((bf16*)Cv)[(size_t)m * H + hcol] = static_cast<bf16>(gate_unit<EPI>(acc[a][2 * pp][r], acc[a][2 * pp + 1][r], H));
         }
       } else {
 #pragma unroll
@@ -682,7 +682,7 @@ __global__ __launch_bounds__(512, 1) void gemm_ring16_kernel(const bf16* __restr
 // column tiles n_tile0 ... n_tile0 + n_tiles - 1 (n_tiles < 0: to the last) of a 256 x TN tiling
 // (slices > 1: the slices of K go to `partial` as [slices][M][N], unadded)
 template <int EPI, int TN, int MAP>
-int launch_ring(const bf16* A, const bf16* W, void* C, int M, int N, int K, int H, hipStream_t stream, int n_tile0 = 0,
+int launch_ring(const bf16* A, const bf16* W, void* C, int M, int N, int K, GateOut H, hipStream_t stream, int n_tile0 = 0,
                 int n_tiles = -1, float* partial = nullptr, int slices = 1) {
   if (n_tiles < 0) n_tiles = ceil_div(N, TN) - n_tile0;
   const int mt = ceil_div(M, RING_TM);
@@ -691,7 +691,7 @@ int launch_ring(const bf16* A, const bf16* W, void* C, int M, int N, int K, int 
   const dim3 grid = MAP == 0 ? dim3(n_tiles, mt, slices) : dim3(8 * ceil_div(mt * n_tiles, 8), slices, 1);
   const size_t lds = (size_t)RING_SLOTS * RING_SLOT;
   // tiles of 256 and 192 columns: the kernel with the 16x16x32 products; of 128: the one with 32x32x16
-  void (*kernel)(const bf16*, const bf16*, void*, int, int, int, int, int, int, float*, int);
+  void (*kernel)(const bf16*, const bf16*, void*, int, int, int, GateOut, int, int, float*, int);
   if constexpr (TN == 128) kernel = &gemm_ring_kernel<EPI, TN, MAP>;
   else kernel = &gemm_ring16_kernel<EPI, TN, MAP>;
   static LdsAllowance allowed;                     // more than 64 KB of LDS has to be asked for once a device
@@ -775,7 +775,7 @@ RingPlan ring_plan(int M, int N, int K, long workspace_floats, int consumer) {
 // stay there unadded (one slice: the product itself), *slices_out says how many
 template <int EPI>
 int launch_ring_shape(const bf16* A, const bf16* W, void* C, float* partial, long partial_floats, int M, int N, int K,
-                      int H, hipStream_t stream, int* slices_out = nullptr,
+                      GateOut H, hipStream_t stream, int* slices_out = nullptr,
                       int consumer = EPI == 2 ? RING_RESIDUAL : RING_PLAIN) {
   const bool keep = slices_out != nullptr;
   const RingPlan p = ring_plan(M, N, K, partial != nullptr ? partial_floats : 0, consumer);
@@ -804,7 +804,7 @@ int launch_ring_shape(const bf16* A, const bf16* W, void* C, float* partial, lon
 }
 
 template <int EPI>
-int launch(const bf16* A, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, int H,
+int launch(const bf16* A, const bf16* W, void* C, float* ws, long ws_floats, int M, int N, int K, GateOut H,
            hipStream_t stream) {
   if (takes_ring(M)) return launch_ring_shape<EPI>(A, W, C, ws, ws_floats, M, N, K, H, stream);
   const int slices = ws != nullptr ? slices_for(M, N, K, ws_floats) : 1;
@@ -842,20 +842,20 @@ int yalm_gemm_bf16_dma_partial(const void* A, const void* W, float* workspace, l
     const RingPlan p = ring_plan(M, N, K, workspace_floats, consumer);
     if (p.slices == 1) {
       *slices_out = 1;
-      return launch_ring_shape<0>(a, w, workspace, nullptr, 0, M, N, K, 0, stream);
+      return launch_ring_shape<0>(a, w, workspace, nullptr, 0, M, N, K, GateOut(0), stream);
     }
-    return launch_ring_shape<0>(a, w, nullptr, workspace, workspace_floats, M, N, K, 0, stream, slices_out,
+    return launch_ring_shape<0>(a, w, nullptr, workspace, workspace_floats, M, N, K, GateOut(0), stream, slices_out,
                                 consumer);
   }
   int slices = slices_for(M, N, K, workspace_floats);
   const int tiles_per_slice = ceil_div(K / TK, slices);
   slices = ceil_div(K / TK, tiles_per_slice);          // what the launch makes of it
   *slices_out = slices;
-  return launch_shape<0, 128, 128, 2, 2, 2, 2>(a, w, workspace, M, N, K, 0, workspace, slices, stream, false);
+  return launch_shape<0, 128, 128, 2, 2, 2, 2>(a, w, workspace, M, N, K, GateOut(0), workspace, slices, stream, false);
 }
 
 int yalm_gemm_bf16_dma(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                       int K, int epilogue, int H, hipStream_t stream) {
+                       int K, int epilogue, GateOut H, hipStream_t stream) {
   if (M <= 64 || K < TK || K % TK != 0 || ((uintptr_t)A & 15) || ((uintptr_t)W & 15)) return YALM_ERR_ARG;
   const bf16* a = (const bf16*)A;
   const bf16* w = (const bf16*)W;

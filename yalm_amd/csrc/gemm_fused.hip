@@ -27,7 +27,7 @@ template <int NT, int NWAVES, int EPI>
 __global__ __launch_bounds__(NWAVES * WAVE) void gemm_norm_kernel(const float* __restrict__ X,
                                                                    const float* __restrict__ norm_w, float eps,
                                                                    const bf16* __restrict__ W, void* __restrict__ Cv,
-                                                                   int M, int N, int K, int H, RopeArgs ra) {
+                                                                   int M, int N, int K, GateOut H, RopeArgs ra) {
   constexpr int KC = 128;
   constexpr int NTHREADS = NWAVES * WAVE;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -156,7 +156,7 @@ __global__ __launch_bounds__(NWAVES * WAVE) void gemm_norm_kernel(const float* _
       for (int r = 0; r < 4; ++r) {
         int m = 4 * q + r;
         if (m < M && hcol < H)
-          C[(size_t)m * H + hcol] = static_cast<bf16>(gate_act<EPI>(g[r] * scale[r]) * (u[r] * scale[r]));
+          C[(size_t)m * H + hcol] = static_cast<bf16>(gate_unit<EPI>(g[r] * scale[r], u[r] * scale[r], H));
       }
     } else {
       f32x4 v = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -213,7 +213,7 @@ __global__ __launch_bounds__(NWAVES * WAVE) void gemm_norm_kernel(const float* _
 }
 
 template <int EPI>
-int launch_norm(const float* X, const float* norm_w, float eps, const bf16* W, void* C, int M, int N, int K, int H,
+int launch_norm(const float* X, const float* norm_w, float eps, const bf16* W, void* C, int M, int N, int K, GateOut H,
            const RopeArgs& ra, hipStream_t stream) {
   bool wide = gated(EPI) || N >= 16384;
   size_t lds = (size_t)M * (K + 8) * sizeof(bf16);
@@ -232,7 +232,8 @@ bool shape_ok(const void* X, const void* norm_w, const void* W, int M, int N, in
 }  // namespace
 
 extern "C" int yalm_gemm_norm(const float* x, const float* norm_w, float eps, const void* W, void* C, int M, int N,
-                              int K, int epilogue, int H, hipStream_t stream) {
+                              int K, int epilogue, int hidden, hipStream_t stream) {
+  const GateOut H(hidden);
   if (!shape_ok(x, norm_w, W, M, N, K)) return YALM_ERR_ARG;
   RopeArgs ra = {};
   if (epilogue == EPI_F32) return launch_norm<EPI_F32>(x, norm_w, eps, (const bf16*)W, C, M, N, K, H, ra, stream);
@@ -272,16 +273,17 @@ extern "C" int yalm_gemm_norm_qkv_rope(const float* x, const float* norm_w, floa
   ra.rotary_dim = rotary_dim;
   ra.n_pages = n_pages;
   ra.page_layout = page_layout;
-  return launch_norm<EPI_ROPE>(x, norm_w, eps, (const bf16*)Wqkv, nullptr, M, N, K, 0, ra, stream);
+  return launch_norm<EPI_ROPE>(x, norm_w, eps, (const bf16*)Wqkv, nullptr, M, N, K, GateOut(0), ra, stream);
 }
 
 // ---------------------------------------------------------------------------
 // chained decode GEMMs (skinny_gemm.h): bfloat16 activations that a producer emitted
 // already multiplied by the norm weights, scaled here per row; and the producer side
 // ---------------------------------------------------------------------------
-extern "C" int yalm_gemm_chain(const void* X, const void* W, void* C, int M, int N, int K, int epilogue, int H,
+extern "C" int yalm_gemm_chain(const void* X, const void* W, void* C, int M, int N, int K, int epilogue, int hidden,
                                const float* ss_in, int n_parts_in, float eps, const float* emit_nw, void* emit_xn,
                                float* emit_ss, hipStream_t stream) {
+  const GateOut H(hidden);
   if (M < 1 || M > 64 || N <= 0 || K <= 0 || K % 8 != 0 || ((uintptr_t)X & 15) || ((uintptr_t)W & 15))
     return YALM_ERR_ARG;
   if (ss_in != nullptr && n_parts_in <= 0) return YALM_ERR_ARG;
@@ -344,7 +346,7 @@ extern "C" int yalm_gemm_chain_qkv_rope(const void* X, const float* ss_in, int n
   ra.rotary_dim = rotary_dim;
   ra.n_pages = n_pages;
   ra.page_layout = page_layout;
-  return skinny::launch<EPI_ROPE>((const bf16*)X, (const bf16*)Wqkv, nullptr, M, N, K, 0, ca, stream);
+  return skinny::launch<EPI_ROPE>((const bf16*)X, (const bf16*)Wqkv, nullptr, M, N, K, GateOut(0), ca, stream);
 }
 
 extern "C" int yalm_gemm_chain_parts(int N) { return skinny::parts_of(N); }

@@ -31,7 +31,7 @@ __device__ __forceinline__ bf16x8 load8(const bf16* p, bool ok) {
 // skinny GEMM: see skinny_gemm.h
 // ---------------------------------------------------------------------------
 template <int EPI>
-int skinny_dispatch(const bf16* X, const bf16* W, void* C, int M, int N, int K, int H, hipStream_t stream) {
+int skinny_dispatch(const bf16* X, const bf16* W, void* C, int M, int N, int K, GateOut H, hipStream_t stream) {
   skinny::ChainArgs ca = {};
   return skinny::launch<EPI>(X, W, C, M, N, K, H, ca, stream);
 }
@@ -48,7 +48,7 @@ constexpr int LDS_ROW = TK + 8;                  // bf16 elements; 16 bytes of p
 // One LDS buffer: the next k tile waits in registers while this one is multiplied.
 template <int EPI, int TM, int TN, int NWM, int NWN, int MINW>
 __global__ __launch_bounds__(NWM * NWN * WAVE, MINW) void gemm_tiled_kernel(const bf16* __restrict__ A, const bf16* __restrict__ W,
-                                                            void* __restrict__ Cv, int M, int N, int K, int H) {
+                                                            void* __restrict__ Cv, int M, int N, int K, GateOut H) {
   constexpr int NT = NWM * NWN * WAVE;
   constexpr int WM = TM / NWM, WN = TN / NWN, FA = WM / 32, FB = WN / 32;
   constexpr int RPP = NT / 8;                    // rows covered by one pass of all threads
@@ -151,7 +151,7 @@ __global__ __launch_bounds__(NWM * NWN * WAVE, MINW) void gemm_tiled_kernel(cons
           int hcol = (n0 + wn * WN + pp * 64) / 2 + li;
           if (hcol < H)
             ((bf16*)Cv)[(size_t)m * H + hcol] =
-                static_cast<bf16>(gate_act<EPI>(acc[a][2 * pp][r]) * acc[a][2 * pp + 1][r]);
+                static_cast<bf16>(gate_unit<EPI>(acc[a][2 * pp][r], acc[a][2 * pp + 1][r], H));
         }
       } else {
 #pragma unroll
@@ -169,7 +169,7 @@ __global__ __launch_bounds__(NWM * NWN * WAVE, MINW) void gemm_tiled_kernel(cons
 }
 
 template <int EPI, int TM, int TN, int NWM, int NWN, int MINW>
-int tiled_launch_shape(const bf16* A, const bf16* W, void* C, int M, int N, int K, int H, hipStream_t stream) {
+int tiled_launch_shape(const bf16* A, const bf16* W, void* C, int M, int N, int K, GateOut H, hipStream_t stream) {
   dim3 grid(ceil_div(N, TN), ceil_div(M, TM));
   size_t lds = (size_t)(TM + TN) * LDS_ROW * sizeof(bf16);
   gemm_tiled_kernel<EPI, TM, TN, NWM, NWN, MINW><<<grid, NWM * NWN * WAVE, lds, stream>>>(A, W, C, M, N, K, H);
@@ -177,7 +177,7 @@ int tiled_launch_shape(const bf16* A, const bf16* W, void* C, int M, int N, int 
 }
 
 template <int EPI>
-int tiled_launch(const bf16* A, const bf16* W, void* C, int M, int N, int K, int H, hipStream_t stream) {
+int tiled_launch(const bf16* A, const bf16* W, void* C, int M, int N, int K, GateOut H, hipStream_t stream) {
   // 256x128 tiles move fewer bytes per flop; 128x128 tiles where those would not fill the chip
   if ((long)ceil_div(M, 256) * ceil_div(N, 128) > 1024)
     return tiled_launch_shape<EPI, 256, 128, 2, 2, 2>(A, W, C, M, N, K, H, stream);
@@ -187,13 +187,13 @@ int tiled_launch(const bf16* A, const bf16* W, void* C, int M, int N, int K, int
 }  // namespace
 
 int yalm_gemm_bf16_batch(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                         int K, int epilogue, int H, hipStream_t stream);   // gemm_batch.hip
+                         int K, int epilogue, GateOut H, hipStream_t stream);   // gemm_batch.hip
 
 int yalm_gemm_bf16_dma(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                       int K, int epilogue, int H, hipStream_t stream);      // gemm_dma.hip
+                       int K, int epilogue, GateOut H, hipStream_t stream);      // gemm_dma.hip
 
 int yalm_gemm_bf16_mfma(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                        int K, int epilogue, int H, hipStream_t stream) {
+                        int K, int epilogue, GateOut H, hipStream_t stream) {
   if (K % 8 != 0 || ((uintptr_t)A & 15) || ((uintptr_t)W & 15)) return YALM_ERR_ARG;
   const bf16* a = (const bf16*)A;
   const bf16* w = (const bf16*)W;

@@ -7,7 +7,7 @@
 #include "yalm_hip.h"
 
 int yalm_gemm_bf16_mfma(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                        int K, int epilogue, int H, hipStream_t stream);   // gemm_mfma.hip; YALM_ERR_ARG: shape refused
+                        int K, int epilogue, GateOut H, hipStream_t stream);   // gemm_mfma.hip; YALM_ERR_ARG: shape refused
 
 namespace {
 constexpr int BM = 64, BN = 64, BK = 16;
@@ -15,7 +15,7 @@ constexpr int BM = 64, BN = 64, BK = 16;
 
 template <typename T, int EPI>
 __global__ __launch_bounds__(256) void gemm_simple_kernel(const T* __restrict__ A, const T* __restrict__ W,
-                                                          void* __restrict__ Cv, int M, int N, int K, int H) {
+                                                          void* __restrict__ Cv, int M, int N, int K, GateOut H) {
   __shared__ float As[BK][BM + 4];
   __shared__ float Ws[BK][BN + 4];
   const int tid = threadIdx.x;
@@ -64,7 +64,7 @@ __global__ __launch_bounds__(256) void gemm_simple_kernel(const T* __restrict__ 
 #pragma unroll
       for (int jj = 0; jj < 2; ++jj) {
         int hcol = (n0 / 32 + jj) * 16 + tx;
-        if (hcol < H) C[(size_t)m * H + hcol] = from_f32<T>(gate_act<EPI>(acc[i][2 * jj]) * acc[i][2 * jj + 1]);
+        if (hcol < H) C[(size_t)m * H + hcol] = from_f32<T>(gate_unit<EPI>(acc[i][2 * jj], acc[i][2 * jj + 1], H));
       }
     } else {
 #pragma unroll
@@ -95,7 +95,7 @@ template <int MB, int EPI>
 __global__ __launch_bounds__(gated(EPI) ? 512 : 256) void gemm_rows_f32_kernel(const float* __restrict__ A,
                                                                              const float* __restrict__ W,
                                                                              void* __restrict__ Cv, int M, int N, int K,
-                                                                             int H) {
+                                                                             GateOut H) {
   constexpr int NWV = gated(EPI) ? 8 : 4;
   __shared__ __attribute__((aligned(16))) float xs[2][MB][RK];
   __shared__ float sums[NWV * 4][MB];
@@ -171,7 +171,7 @@ __global__ __launch_bounds__(gated(EPI) ? 512 : 256) void gemm_rows_f32_kernel(c
     for (int e = tid; e < 16 * MB; e += NWV * WAVE) {
       const int j = e % 16, m = e / 16, hcol = base + j;
       if (m < M && hcol < H)
-        ((float*)Cv)[(size_t)m * H + hcol] = gate_act<EPI>(sums[j][m]) * sums[16 + j][m];
+        ((float*)Cv)[(size_t)m * H + hcol] = gate_unit<EPI>(sums[j][m], sums[16 + j][m], H);
     }
   } else {
     const int nb = blockIdx.x * NWV * 4;
@@ -186,7 +186,7 @@ __global__ __launch_bounds__(gated(EPI) ? 512 : 256) void gemm_rows_f32_kernel(c
 }
 
 template <int MB>
-int launch_rows_f32(const float* A, const float* W, void* C, int M, int N, int K, int epilogue, int H,
+int launch_rows_f32(const float* A, const float* W, void* C, int M, int N, int K, int epilogue, GateOut H,
                     hipStream_t stream) {
   switch (epilogue) {
     case 0: gemm_rows_f32_kernel<MB, 0><<<ceil_div(N, 16), 256, 0, stream>>>(A, W, C, M, N, K, H); break;
@@ -201,7 +201,7 @@ int launch_rows_f32(const float* A, const float* W, void* C, int M, int N, int K
 
 // float32, at most 64 rows (16 a pass over the weights: up to four passes still beat the tiles, which
 // are mostly padding then), K a multiple of 4 and 16-byte aligned operands; YALM_ERR_ARG: not taken
-int gemm_rows_f32(const void* A, const void* W, void* C, int M, int N, int K, int epilogue, int H, hipStream_t stream) {
+int gemm_rows_f32(const void* A, const void* W, void* C, int M, int N, int K, int epilogue, GateOut H, hipStream_t stream) {
   if (M > 64 || K % 4 != 0 || ((uintptr_t)A & 15) || ((uintptr_t)W & 15)) return YALM_ERR_ARG;
   const float* w = (const float*)W;
   const int out_cols = gated(epilogue) ? H : N;
@@ -219,7 +219,7 @@ int gemm_rows_f32(const void* A, const void* W, void* C, int M, int N, int K, in
 }
 
 template <typename T>
-int gemm_simple(const void* A, const void* W, void* C, int M, int N, int K, int epilogue, int H, hipStream_t stream) {
+int gemm_simple(const void* A, const void* W, void* C, int M, int N, int K, int epilogue, GateOut H, hipStream_t stream) {
   dim3 grid(ceil_div(N, BN), ceil_div(M, BM));
   const T* a = (const T*)A;
   const T* w = (const T*)W;
@@ -236,7 +236,9 @@ int gemm_simple(const void* A, const void* W, void* C, int M, int N, int K, int 
 }  // namespace
 
 extern "C" int yalm_gemm(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N,
-                         int K, int dtype, int epilogue, int H, int force_simple, hipStream_t stream) {
+                         int K, int dtype, int epilogue, int hidden, float gate_limit, float gate_alpha, float up_shift,
+                         int force_simple, hipStream_t stream) {
+  const GateOut H(hidden, gate_limit, gate_alpha, up_shift);
   if (M <= 0) return YALM_OK;
   if (N <= 0 || K <= 0 || epilogue < 0 || (epilogue > 3 && epilogue != EPI_GATED_GELU)) return YALM_ERR_ARG;
   if (gated(epilogue) && (H <= 0 || N != 32 * ((H + 15) / 16))) return YALM_ERR_ARG;

@@ -200,8 +200,8 @@ int main(int argc, char** argv) {
   for (int rep = 0; rep < 3; ++rep) {
     CK(hipEventRecord(e0, stream));
     for (int c = 0; c < copies; ++c) {
-      int rc = yalm_gemm(x, w[c], out, ws, ws_floats, M, N, K, 1, epilogue, H, 0, stream);
-      if (rc == 0 && ffn) rc = yalm_gemm(out, w2[c], x_out, ws, ws_floats, M, dim, hidden, 1, 2, 0, 0, stream);
+      int rc = yalm_gemm(x, w[c], out, ws, ws_floats, M, N, K, 1, epilogue, H, 0.f, 1.f, 0.f, 0, stream);
+      if (rc == 0 && ffn) rc = yalm_gemm(out, w2[c], x_out, ws, ws_floats, M, dim, hidden, 1, 2, 0, 0.f, 1.f, 0.f, 0, stream);
       if (rc != 0) {
         fprintf(stderr, "yalm_gemm failed: %s\n", yalm_error_string(rc));
         return 1;

@@ -2,7 +2,8 @@
 //
 //  * yalm_moe_route: per token, logits = W_router h in float32, scores = softmax over all experts, the
 //    `top` largest (the lowest index on ties), with their scores as weights (optionally renormalised
-//    to sum 1).  One wave a token.  yalm_moe_select_groups: sigmoid scores, choice inside the best groups.
+//    to sum 1).  One wave a token.  yalm_moe_select_groups: sigmoid or softmax scores, a
+//    correction, choice inside the best groups.
 //  * yalm_moe_pair_gate_up / yalm_moe_pair_down: every pair reads its expert's weights: a wave per output
 //    row, the lanes along K with 16-byte loads.  What a decode step needs (few pairs, each bound by
 //    the one pass over its expert), and correct for any number of tokens.
@@ -124,10 +125,11 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const T* __restrict__ h
     for (int k = lane; k < top; k += WAVE) wts[(size_t)t * top + k] /= total;
 }
 
-// Sigmoid scores and choice inside the best groups: s = sigmoid(logit), c = s + correction; experts e of neighbours form
-// n_groups equal groups, a group's score is the sum of its two largest c, the `keep` best groups stay (the others'
-// c counts as minus infinity), the `top` largest c are chosen, and their weights are s / (sum of the chosen s + 1e-20) *
-// scale.  One wave a token; ties go to the lower index.
+// Choice inside the best groups: scores s = sigmoid(logit), or with SOFTMAX the softmax over all experts, c = s + correction;
+// experts e of neighbours form n_groups equal groups, a group's score is the sum of its two largest c (with GROUP_MAX its
+// largest c), the `keep` best groups stay (the others' c counts as minus infinity), the `top` largest c are chosen, and their
+// weights are s / (sum of the chosen s + 1e-20) * scale.  One wave a token; ties go to the lower index.
+template <bool SOFTMAX, bool GROUP_MAX>
 __global__ __launch_bounds__(WAVE) void moe_select_groups_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
                                                                  int* __restrict__ ids, float* __restrict__ wts, int E, int top,
                                                                  int n_groups, int keep, float scale) {
@@ -135,8 +137,18 @@ __global__ __launch_bounds__(WAVE) void moe_select_groups_kernel(const float* __
   __shared__ float choice[MOE_MAX_EXPERTS];       // c
   __shared__ float group[MOE_MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x, per = E / n_groups;
+  const float* z = logits + (size_t)t * E;
+  float m = 0.f, inv = 1.f;
+  if constexpr (SOFTMAX) {
+    m = -INFINITY;
+    for (int e = lane; e < E; e += WAVE) m = fmaxf(m, z[e]);
+    m = wave_max(m);
+    float sum = 0.f;
+    for (int e = lane; e < E; e += WAVE) sum += expf(z[e] - m);
+    inv = 1.0f / wave_sum(sum);
+  }
   for (int e = lane; e < E; e += WAVE) {
-    const float s = 1.0f / (1.0f + expf(-logits[(size_t)t * E + e]));
+    const float s = SOFTMAX ? expf(z[e] - m) * inv : 1.0f / (1.0f + expf(-z[e]));
     score[e] = s;
     choice[e] = s + (correction != nullptr ? correction[e] : 0.f);
   }
@@ -170,7 +182,7 @@ __global__ __launch_bounds__(WAVE) void moe_select_groups_kernel(const float* __
         const float x = choice[e];
         if (x > a) { b = a; a = x; } else if (x > b) { b = x; }
       }
-      group[g] = per > 1 ? a + b : a;
+      group[g] = !GROUP_MAX && per > 1 ? a + b : a;
     }
     __syncthreads();
     for (int e = lane; e < E; e += WAVE)
@@ -496,12 +508,20 @@ extern "C" int yalm_moe_select(const float* logits, const float* bias, int* ids,
 }
 
 extern "C" int yalm_moe_select_groups(const float* logits, const float* correction, int* ids, float* wts, int T, int E, int top,
-                                      int n_groups, int keep, float scale, hipStream_t stream) {
+                                      int n_groups, int keep, float scale, int softmax, int group_max, hipStream_t stream) {
   if (T <= 0) return YALM_OK;
   if (E <= 0 || E > MOE_MAX_EXPERTS || n_groups <= 0 || E % n_groups || keep <= 0 || keep > n_groups || top <= 0 ||
       top > keep * (E / n_groups))
     return YALM_ERR_ARG;
-  moe_select_groups_kernel<<<T, WAVE, 0, stream>>>(logits, correction, ids, wts, E, top, n_groups, keep, scale);
+#define SEL(S_, M_) moe_select_groups_kernel<S_, M_><<<T, WAVE, 0, stream>>>(logits, correction, ids, wts, E, top, n_groups, keep, scale)
+  if (softmax) {
+    if (group_max) SEL(true, true);
+    else SEL(true, false);
+  } else {
+    if (group_max) SEL(false, true);
+    else SEL(false, false);
+  }
+#undef SEL
   return launch_status();
 }
 

@@ -2,7 +2,8 @@
 // the previous and the present token, an activation between the two products of an
 // ungated feed-forward (or of a gated one whose products carry biases), the add of a sublayer's result under a gate
 // of one number a token, a short causal convolution over time on every channel with its carried inputs, a sigmoid
-// gate on an attention's heads, and the way into a walk of looped layers.
+// gate on an attention's heads (a number an element, or a number a head), the way into a walk of looped layers, and the cap
+// on logits.
 #include "common.h"
 #include "yalm_hip.h"
 
@@ -105,9 +106,11 @@ __global__ __launch_bounds__(NW * WAVE) void gated_add_kernel(const float* __res
 // that neighbouring channels' weights are neighbours): a causal convolution over the tokens
 // of a sequence, the last tap on the token itself.  Inputs in front of the step's first token of a sequence come from
 // carried[slot][taps - 1][D] (the sequence's last taps - 1 inputs, the newest last; zeros for a new sequence), and a
-// padding row (slot -1) reads zeros there.  A thread a (token, channel).
+// padding row (slot -1) reads zeros there.  The rows of h are h_row apart; in_bias (may be null) is a part of every input (of
+// the carried ones too, and not of the zeros in front of a text), out_bias is added to the sum.  A thread a (token, channel).
 template <typename T, int MAX_TAPS>
-__global__ void time_conv_kernel(const T* __restrict__ h, const float* __restrict__ w, const float* __restrict__ carried,
+__global__ void time_conv_kernel(const T* __restrict__ h, long h_row, const float* __restrict__ in_bias,
+                                 const float* __restrict__ out_bias, const float* __restrict__ w, const float* __restrict__ carried,
                                  T* __restrict__ out, const int* __restrict__ tok_seq, const int* __restrict__ cu_seqlens,
                                  const int* __restrict__ seq_slot, int D, int taps, int residual) {
   const int t = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
@@ -115,11 +118,12 @@ __global__ void time_conv_kernel(const T* __restrict__ h, const float* __restric
   const int b = tok_seq[t];
   const int first = b >= 0 ? cu_seqlens[b] : t, slot = b >= 0 ? seq_slot[b] : -1;
   const int l = t - first;                        // the token's place among its sequence's tokens of this step
-  float acc = residual ? to_f32(h[(size_t)t * D + c]) : 0.f;
+  const float ib = in_bias != nullptr ? in_bias[c] : 0.f;
+  float acc = (residual ? to_f32(h[(size_t)t * h_row + c]) + ib : 0.f) + (out_bias != nullptr ? out_bias[c] : 0.f);
   for (int j = 0; j < taps; ++j) {
     const int src = l - (taps - 1) + j;
     float v = 0.f;
-    if (src >= 0) v = to_f32(h[(size_t)(first + src) * D + c]);
+    if (src >= 0) v = to_f32(h[(size_t)(first + src) * h_row + c]) + ib;
     else if (slot >= 0) v = carried[((size_t)slot * (taps - 1) + (taps - 1 + src)) * D + c];
     acc = fmaf(w[(size_t)j * D + c], v, acc);
   }
@@ -154,12 +158,21 @@ template <> struct Chunk<bf16, 8> {
   }
 };
 template <typename E, int VEC>
-__global__ void time_conv_vec_kernel(const E* __restrict__ h, const float* __restrict__ w, float* __restrict__ carried,
+__global__ void time_conv_vec_kernel(const E* __restrict__ h, long h_row, const float* __restrict__ in_bias,
+                                     const float* __restrict__ out_bias, const float* __restrict__ w, float* __restrict__ carried,
                                      E* __restrict__ out, const int* __restrict__ tok_seq,
                                      const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slot, int D, int taps,
                                      int residual, int one_each, int n_tokens, int per_block) {
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
   if (c >= D) return;
+  float ib[VEC], ob[VEC];
+#pragma unroll
+  for (int k = 0; k < VEC; ++k) ib[k] = ob[k] = 0.f;
+#pragma unroll
+  for (int k = 0; k < VEC; k += 4) {
+    if (in_bias != nullptr) Chunk<float, 4>::load(in_bias + c + k, ib + k);
+    if (out_bias != nullptr) Chunk<float, 4>::load(out_bias + c + k, ob + k);
+  }
   // a workgroup takes per_block tokens that follow each other: a token's earlier inputs are then lines that the
   // same threads have just read
   for (int t = blockIdx.x * per_block; t < min(n_tokens, (int)(blockIdx.x + 1) * per_block); ++t) {
@@ -167,13 +180,18 @@ __global__ void time_conv_vec_kernel(const E* __restrict__ h, const float* __res
   const int first = one_each ? t : (b >= 0 ? cu_seqlens[b] : t), slot = b >= 0 ? seq_slot[b] : -1;
   const int l = t - first, keep = taps - 1;
   float own[VEC], acc[VEC], v[VEC];
-  Chunk<E, VEC>::load(h + (size_t)t * D + c, own);
+  Chunk<E, VEC>::load(h + (size_t)t * h_row + c, own);
 #pragma unroll
-  for (int k = 0; k < VEC; ++k) acc[k] = residual ? own[k] : 0.f;
+  for (int k = 0; k < VEC; ++k) {
+    own[k] += ib[k];
+    acc[k] = (residual ? own[k] : 0.f) + ob[k];
+  }
   for (int j = 0; j < taps; ++j) {
     const int src = l - keep + j;
     if (src >= 0) {
-      Chunk<E, VEC>::load(h + (size_t)(first + src) * D + c, v);
+      Chunk<E, VEC>::load(h + (size_t)(first + src) * h_row + c, v);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) v[k] += ib[k];
     } else if (slot >= 0) {
       const float* row = carried + ((size_t)slot * keep + (keep + src)) * D + c;
 #pragma unroll
@@ -205,7 +223,7 @@ __global__ void time_conv_vec_kernel(const E* __restrict__ h, const float* __res
 // carried[slot] <- the last taps - 1 inputs of each sequence after this step's tokens; a thread a (sequence, channel)
 // reads what it needs of the old rows before it writes the new ones
 template <typename T, int MAX_TAPS>
-__global__ void time_conv_carry_kernel(const T* __restrict__ h, float* __restrict__ carried,
+__global__ void time_conv_carry_kernel(const T* __restrict__ h, long h_row, const float* __restrict__ in_bias, float* __restrict__ carried,
                                        const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slot, int D,
                                        int taps) {
   const int b = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
@@ -214,12 +232,13 @@ __global__ void time_conv_carry_kernel(const T* __restrict__ h, float* __restric
   if (slot < 0) return;
   const int first = cu_seqlens[b], n = cu_seqlens[b + 1] - first, keep = taps - 1;
   float* rows = carried + (size_t)slot * keep * D + c;
+  const float ib = in_bias != nullptr ? in_bias[c] : 0.f;
   float fresh[MAX_TAPS];
 #pragma unroll
   for (int i = 0; i < MAX_TAPS; ++i) {
     if (i < keep) {
       const int src = n - keep + i;               // place among this step's tokens; negative: an older input
-      fresh[i] = src >= 0 ? to_f32(h[(size_t)(first + src) * D + c]) : rows[(size_t)(keep + src) * D];
+      fresh[i] = src >= 0 ? to_f32(h[(size_t)(first + src) * h_row + c]) + ib : rows[(size_t)(keep + src) * D];
     }
   }
 #pragma unroll
@@ -257,6 +276,23 @@ __global__ void sigmoid_gate_kernel(T* __restrict__ o, const float* __restrict__
     T* p = o + ((size_t)t * n_heads + h) * pad + e;
     *p = from_f32<T>(to_f32(*p) / (1.0f + expf(-g[(size_t)t * g_stride + i])));
   }
+}
+
+// out[t, h, e] = o[t, h, e] * sigmoid(g[t * g_row + h]) * scale, e < dv (a gate of one number a head): rows of out are out_row
+// apart and may be o's own; a workgroup a token, or several where the tokens are few
+template <typename T>
+__global__ void head_gate_kernel(const T* __restrict__ o, const float* __restrict__ g, long g_row, float scale, T* __restrict__ out,
+                                 long out_row, int n_heads, int dv) {
+  const int t = blockIdx.x;
+  const T* src = o + (size_t)t * n_heads * dv;
+  T* dst = out + (size_t)t * out_row;
+  for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < n_heads * dv; i += gridDim.y * blockDim.x)
+    dst[i] = from_f32<T>(to_f32(src[i]) * (scale / (1.0f + expf(-g[(size_t)t * g_row + i / dv]))));
+}
+
+// z[i] = cap tanh(z[i] / cap)
+__global__ void softcap_kernel(float* __restrict__ z, long n, float cap, float inv) {
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) z[i] = cap * tanhf(z[i] * inv);
 }
 
 // both[t] = [x[t] | x0[t]] in the compute dtype, then x[t] = start: what the product that enters a walk of looped
@@ -340,44 +376,47 @@ extern "C" int yalm_gated_add(const float* y, const void* h, const void* w, int 
 }
 
 constexpr int CONV_MAX_TAPS = 16;
-extern "C" int yalm_time_conv(const void* h, const float* w, float* carried, void* out, const int* tok_seq,
+extern "C" int yalm_time_conv(const void* h, long h_row, const float* in_bias, const float* out_bias, const float* w, float* carried, void* out, const int* tok_seq,
                               const int* cu_seqlens, const int* seq_slot, int T, int B, int D, int taps, int residual,
                               int one_each, int dtype, hipStream_t stream) {
   if (T <= 0) return YALM_OK;
   if (one_each && T != B) return YALM_ERR_ARG;
+  if (h_row < D) return YALM_ERR_ARG;
   if (D <= 0 || B <= 0 || taps <= 0 || taps > CONV_MAX_TAPS || h == out ||
       (taps > 1 && carried == nullptr) || ceil_div(D, 256) > 65535)
     return YALM_ERR_ARG;
   const int vec = dtype == YALM_F32 ? 4 : 8;
-  if (D % vec == 0 && (((uintptr_t)h | (uintptr_t)out | (uintptr_t)carried) & 15) == 0 && (dtype == YALM_F32 || dtype == YALM_BF16)) {
+  if (D % vec == 0 && h_row % vec == 0 &&
+      (((uintptr_t)h | (uintptr_t)out | (uintptr_t)carried | (uintptr_t)w | (uintptr_t)in_bias | (uintptr_t)out_bias) & 15) == 0 &&
+      (dtype == YALM_F32 || dtype == YALM_BF16)) {
     const int lanes = D / vec, vthreads = lanes >= 256 ? 256 : 64;
     const int per_block = (long)T * D >= 2048L * 4096 ? 4 : 1;      // measured: 20.1 -> 15.8 us at 2,048 x 4,096, no gain below
     dim3 vgrid(ceil_div(T, per_block), ceil_div(lanes, vthreads)), vcgrid(B, ceil_div(D, 256));
     if (dtype == YALM_F32) {
-      time_conv_vec_kernel<float, 4><<<vgrid, vthreads, 0, stream>>>((const float*)h, w, carried, (float*)out, tok_seq, cu_seqlens,
+      time_conv_vec_kernel<float, 4><<<vgrid, vthreads, 0, stream>>>((const float*)h, h_row, in_bias, out_bias, w, carried, (float*)out, tok_seq, cu_seqlens,
                                                                     seq_slot, D, taps, residual, one_each, T, per_block);
       if (taps > 1 && !one_each)
-        time_conv_carry_kernel<float, CONV_MAX_TAPS><<<vcgrid, 256, 0, stream>>>((const float*)h, carried, cu_seqlens, seq_slot, D, taps);
+        time_conv_carry_kernel<float, CONV_MAX_TAPS><<<vcgrid, 256, 0, stream>>>((const float*)h, h_row, in_bias, carried, cu_seqlens, seq_slot, D, taps);
     } else {
-      time_conv_vec_kernel<bf16, 8><<<vgrid, vthreads, 0, stream>>>((const bf16*)h, w, carried, (bf16*)out, tok_seq, cu_seqlens,
+      time_conv_vec_kernel<bf16, 8><<<vgrid, vthreads, 0, stream>>>((const bf16*)h, h_row, in_bias, out_bias, w, carried, (bf16*)out, tok_seq, cu_seqlens,
                                                                    seq_slot, D, taps, residual, one_each, T, per_block);
       if (taps > 1 && !one_each)
-        time_conv_carry_kernel<bf16, CONV_MAX_TAPS><<<vcgrid, 256, 0, stream>>>((const bf16*)h, carried, cu_seqlens, seq_slot, D, taps);
+        time_conv_carry_kernel<bf16, CONV_MAX_TAPS><<<vcgrid, 256, 0, stream>>>((const bf16*)h, h_row, in_bias, carried, cu_seqlens, seq_slot, D, taps);
     }
     return launch_status();
   }
   const int threads = D >= 256 ? 256 : 64;
   dim3 grid(T, ceil_div(D, threads)), cgrid(B, ceil_div(D, threads));
   if (dtype == YALM_F32) {
-    time_conv_kernel<float, CONV_MAX_TAPS><<<grid, threads, 0, stream>>>((const float*)h, w, carried, (float*)out, tok_seq,
+    time_conv_kernel<float, CONV_MAX_TAPS><<<grid, threads, 0, stream>>>((const float*)h, h_row, in_bias, out_bias, w, carried, (float*)out, tok_seq,
                                                                          cu_seqlens, seq_slot, D, taps, residual);
     if (taps > 1)
-      time_conv_carry_kernel<float, CONV_MAX_TAPS><<<cgrid, threads, 0, stream>>>((const float*)h, carried, cu_seqlens, seq_slot, D, taps);
+      time_conv_carry_kernel<float, CONV_MAX_TAPS><<<cgrid, threads, 0, stream>>>((const float*)h, h_row, in_bias, carried, cu_seqlens, seq_slot, D, taps);
   } else if (dtype == YALM_BF16) {
-    time_conv_kernel<bf16, CONV_MAX_TAPS><<<grid, threads, 0, stream>>>((const bf16*)h, w, carried, (bf16*)out, tok_seq,
+    time_conv_kernel<bf16, CONV_MAX_TAPS><<<grid, threads, 0, stream>>>((const bf16*)h, h_row, in_bias, out_bias, w, carried, (bf16*)out, tok_seq,
                                                                         cu_seqlens, seq_slot, D, taps, residual);
     if (taps > 1)
-      time_conv_carry_kernel<bf16, CONV_MAX_TAPS><<<cgrid, threads, 0, stream>>>((const bf16*)h, carried, cu_seqlens, seq_slot, D, taps);
+      time_conv_carry_kernel<bf16, CONV_MAX_TAPS><<<cgrid, threads, 0, stream>>>((const bf16*)h, h_row, in_bias, carried, cu_seqlens, seq_slot, D, taps);
   } else {
     return YALM_ERR_DTYPE;
   }
@@ -426,5 +465,29 @@ extern "C" int yalm_loop_pack(float* x, const float* x0, const float* start, voi
     loop_pack_kernel<bf16><<<T, threads, 0, stream>>>(x, x0, start, (bf16*)both, D);
   else
     return YALM_ERR_DTYPE;
+  return launch_status();
+}
+
+extern "C" int yalm_head_gate(const void* o, const float* g, long g_row, float scale, void* out, long out_row, int T, int n_heads,
+                              int dv, int dtype, hipStream_t stream) {
+  if (T <= 0) return YALM_OK;
+  if (n_heads <= 0 || dv <= 0 || g_row < n_heads || out_row < (long)n_heads * dv || (o == out && T > 1 && out_row != (long)n_heads * dv))
+    return YALM_ERR_ARG;
+  const int cols = n_heads * dv, slices = T >= 256 ? 1 : ceil_div(cols, 1024);
+  const dim3 grid(T, slices < 64 ? slices : 64);
+  if (dtype == YALM_F32)
+    head_gate_kernel<float><<<grid, 256, 0, stream>>>((const float*)o, g, g_row, scale, (float*)out, out_row, n_heads, dv);
+  else if (dtype == YALM_BF16)
+    head_gate_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)o, g, g_row, scale, (bf16*)out, out_row, n_heads, dv);
+  else
+    return YALM_ERR_DTYPE;
+  return launch_status();
+}
+
+extern "C" int yalm_softcap(float* z, long n, float cap, hipStream_t stream) {
+  if (n <= 0) return YALM_OK;
+  if (!(cap > 0.f)) return YALM_ERR_ARG;
+  const int blocks = (int)((n + 1023) / 1024 < 4096 ? (n + 1023) / 1024 : 4096);
+  softcap_kernel<<<blocks, 256, 0, stream>>>(z, n, cap, 1.0f / cap);
   return launch_status();
 }

@@ -1,6 +1,7 @@
 // Kernels of layers that norm a sublayer's OUTPUT before it joins the residual stream
-// (x <- x + rms(y) * w) or the SUM of both (x <- LN(alpha x + y)), and of the PolyNorm activation.  Everything is float32 arithmetic on a row
-// per workgroup; inputs from GEMMs are float32, outputs go to the compute dtype.
+// (x <- x + rms(y) * w) or the SUM of both (x <- LN(alpha x + y)), of the PolyNorm activation, of an elementwise squash in
+// a norm's place (tanh(alpha x) * w + b), and of a row's RMS norm under a sigmoid gate.  Everything is float32 arithmetic, on a
+// row per workgroup where a row has sums; inputs from GEMMs are float32, outputs go to the compute dtype.
 #include "common.h"
 #include "yalm_hip.h"
 
@@ -148,6 +149,89 @@ __global__ __launch_bounds__(NT) void layer_norm_kernel(float* __restrict__ x, c
   each([&](int i, int j) { h[row + i] = from_f32<T>(fmaf((normed(i, j) - mean2) * r2, next_w[i], next_b[i])); });
 }
 
+// An elementwise squash in a norm's place, n(v) = tanh(alpha v) * w + b.  y null: h[r] = T(n(x[row(r)])).  Else x[r] += mult *
+// n(y[r] + y_bias), and h (may be null) receives the new x, or with next_w the squash that reads the stream next, of the new
+// x.  A thread has VEC neighbours of a row.
+template <typename T, int VEC>
+__global__ __launch_bounds__(ROW_THREADS) void squash_kernel(float* __restrict__ x, const float* __restrict__ y,
+                                                             const float* __restrict__ y_bias, float mult,
+                                                             const int* __restrict__ row_index, float alpha,
+                                                             const float* __restrict__ w, const float* __restrict__ b,
+                                                             T* __restrict__ h, float next_alpha, const float* __restrict__ next_w,
+                                                             const float* __restrict__ next_b, int D) {
+  struct __attribute__((aligned(VEC * sizeof(float)))) F { float v[VEC]; };
+  struct __attribute__((aligned(VEC * sizeof(T)))) O { T v[VEC]; };
+  const int i = (blockIdx.y * ROW_THREADS + threadIdx.x) * VEC;
+  if (i >= D) return;
+  auto load = [&](const float* p) { return *reinterpret_cast<const F*>(p); };
+  const size_t at = (size_t)blockIdx.x * D + i;
+  float* xp = x + (row_index != nullptr ? (size_t)row_index[blockIdx.x] * D + i : at);
+  const F ww = load(w + i), bb = load(b + i);
+  F xv = load(xp);
+  O o;
+  if (y == nullptr) {
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) o.v[k] = from_f32<T>(fmaf(tanhf(alpha * xv.v[k]), ww.v[k], bb.v[k]));
+    *reinterpret_cast<O*>(h + at) = o;
+    return;
+  }
+  F yv = load(y + at);
+  if (y_bias != nullptr) {
+    const F yb = load(y_bias + i);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) yv.v[k] += yb.v[k];
+  }
+#pragma unroll
+  for (int k = 0; k < VEC; ++k) xv.v[k] = fmaf(mult, fmaf(tanhf(alpha * yv.v[k]), ww.v[k], bb.v[k]), xv.v[k]);
+  *reinterpret_cast<F*>(xp) = xv;
+  if (h == nullptr) return;
+  if (next_w != nullptr) {
+    const F nw = load(next_w + i), nb = load(next_b + i);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) o.v[k] = from_f32<T>(fmaf(tanhf(next_alpha * xv.v[k]), nw.v[k], nb.v[k]));
+  } else {
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) o.v[k] = from_f32<T>(xv.v[k]);
+  }
+  *reinterpret_cast<O*>(h + at) = o;
+}
+
+// out[r, i] = x[r, i] / sqrt(mean(x[r]^2) + eps) * w[i] * sigmoid(gate[r, i]), i < n: a workgroup a row; the rows of gate and
+// out are gate_row and out_row apart.  PER > 0: the row fits PER values a thread; PER = 0: any length.
+template <typename T, int NT, int PER>
+__global__ __launch_bounds__(NT) void rms_gate_kernel(const float* __restrict__ x, const float* __restrict__ w, float eps,
+                                                      const float* __restrict__ gate, long gate_row, T* __restrict__ out,
+                                                      long out_row, int n) {
+  __shared__ float red[NT / WAVE];
+  const float* xr = x + (size_t)blockIdx.x * n;
+  const float* gr = gate + (size_t)blockIdx.x * gate_row;
+  T* o = out + (size_t)blockIdx.x * out_row;
+  float ss = 0.f;
+  auto gated = [&](float v, float s, float wi, float z) { return from_f32<T>(v * s * wi / (1.0f + expf(-z))); };
+  if constexpr (PER > 0) {
+    float v[PER], z[PER], g[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int i = threadIdx.x + j * NT;
+      v[j] = i < n ? xr[i] : 0.f;
+      z[j] = i < n ? gr[i] : 0.f;
+      g[j] = i < n ? w[i] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < PER; ++j) ss = fmaf(v[j], v[j], ss);
+    const float s = 1.0f / sqrtf(block_sum<NT / WAVE>(ss, red) / (float)n + eps);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int i = threadIdx.x + j * NT;
+      if (i < n) o[i] = gated(v[j], s, g[j], z[j]);
+    }
+  } else {
+    for (int i = threadIdx.x; i < n; i += NT) ss = fmaf(xr[i], xr[i], ss);
+    const float s = 1.0f / sqrtf(block_sum<NT / WAVE>(ss, red) / (float)n + eps);
+    for (int i = threadIdx.x; i < n; i += NT) o[i] = gated(xr[i], s, w[i], gr[i]);
+  }
+}
+
 // out = a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + eps) over the row.  PER > 0: the row fits PER
 // values a thread and is read once (kept in registers between the sums and the result); PER = 0: any width, read twice.
 template <typename T, int NT, int PER>
@@ -285,5 +369,55 @@ extern "C" int yalm_polynorm(const float* z, const float* coef, float eps, void*
   if (F <= 0) return YALM_ERR_ARG;
   if (out_dtype == YALM_BF16) return polynorm_launch<bf16>(z, coef, eps, out, R, F, stream);
   if (out_dtype == YALM_F32) return polynorm_launch<float>(z, coef, eps, out, R, F, stream);
+  return YALM_ERR_DTYPE;
+}
+
+template <typename T>
+static int squash_launch(float* x, const float* y, const float* y_bias, float mult, const int* row_index, float alpha,
+                         const float* w, const float* b, void* h, float next_alpha, const float* next_w, const float* next_b,
+                         int R, int D, hipStream_t stream) {
+  const bool vec = D % 4 == 0 && ((((uintptr_t)x) | ((uintptr_t)y) | ((uintptr_t)y_bias) | ((uintptr_t)w) | ((uintptr_t)b) |
+                                   ((uintptr_t)h) | ((uintptr_t)next_w) | ((uintptr_t)next_b)) & 15) == 0;
+  const dim3 grid(R, ceil_div(D, ROW_THREADS * (vec ? 4 : 1)));
+#define SQ(V_) \
+  squash_kernel<T, V_><<<grid, ROW_THREADS, 0, stream>>>(x, y, y_bias, mult, row_index, alpha, w, b, (T*)h, next_alpha, next_w, next_b, D)
+  if (vec) SQ(4);
+  else SQ(1);
+#undef SQ
+  return launch_status();
+}
+
+extern "C" int yalm_squash(float* x, const float* y, const float* y_bias, float mult, const int* row_index, float alpha,
+                           const float* w, const float* b, void* h, int h_dtype, float next_alpha, const float* next_w,
+                           const float* next_b, int R, int D, hipStream_t stream) {
+  if (R <= 0) return YALM_OK;
+  if (D <= 0 || ceil_div(D, ROW_THREADS) > 65535 || w == nullptr || b == nullptr || (y == nullptr && h == nullptr) ||
+      (y == nullptr && (y_bias != nullptr || next_w != nullptr)) || (y != nullptr && row_index != nullptr) ||
+      (next_w != nullptr && (next_b == nullptr || h == nullptr)))
+    return YALM_ERR_ARG;
+  if (h != nullptr && h_dtype != YALM_F32 && h_dtype != YALM_BF16) return YALM_ERR_DTYPE;
+  if (h != nullptr && h_dtype == YALM_BF16)
+    return squash_launch<bf16>(x, y, y_bias, mult, row_index, alpha, w, b, h, next_alpha, next_w, next_b, R, D, stream);
+  return squash_launch<float>(x, y, y_bias, mult, row_index, alpha, w, b, h, next_alpha, next_w, next_b, R, D, stream);
+}
+
+template <typename T>
+static int rms_gate_launch(const float* x, const float* w, float eps, const float* gate, long gate_row, void* out, long out_row,
+                           int R, int n, hipStream_t stream) {
+#define RG(NT_, PER_) rms_gate_kernel<T, NT_, PER_><<<R, NT_, 0, stream>>>(x, w, eps, gate, gate_row, (T*)out, out_row, n)
+  if (n <= 1024) RG(256, 4);
+  else if (n <= 2048) RG(512, 4);
+  else if (n <= 8192) RG(1024, 8);
+  else RG(1024, 0);
+#undef RG
+  return launch_status();
+}
+
+extern "C" int yalm_rms_gate(const float* x, const float* w, float eps, const float* gate, long gate_row, void* out,
+                             long out_row, int out_dtype, int R, int n, hipStream_t stream) {
+  if (R <= 0) return YALM_OK;
+  if (n <= 0 || gate_row < n || out_row < n || w == nullptr || gate == nullptr) return YALM_ERR_ARG;
+  if (out_dtype == YALM_F32) return rms_gate_launch<float>(x, w, eps, gate, gate_row, out, out_row, R, n, stream);
+  if (out_dtype == YALM_BF16) return rms_gate_launch<bf16>(x, w, eps, gate, gate_row, out, out_row, R, n, stream);
   return YALM_ERR_DTYPE;
 }

@@ -3,6 +3,7 @@
 // with those an earlier layer made for the same token, and the way into the cache.  A workgroup a token; the row
 // waits in LDS between its sums and its results.
 //
+// The rows of qkv are qkv_row apart (a product may hold more behind them).
 //   q = (qkv[:Q] + b_q);  q <- q / rms(q) * w_q            (w_q null: no norm)
 //   q <- q * (1 + coef ln(floor((p + 1) / every) + 1)) * q_scale      (every 0: no factor)
 //   k likewise with w_k (no factor);  v = qkv[Q + K:] + b_v
@@ -21,7 +22,7 @@ namespace {
 // thread's loads wait for each other's results in turn: the fewer rounds the better)
 template <typename T, int PACK_THREADS>
 __global__ __launch_bounds__(PACK_THREADS) void qkv_pack_kernel(
-    const float* __restrict__ qkv, const float* __restrict__ bias, const float* __restrict__ w_q,
+    const float* __restrict__ qkv, long qkv_row, const float* __restrict__ bias, const float* __restrict__ w_q,
     const float* __restrict__ w_k, float eps, float temp_coef, int temp_every, float q_scale, float* __restrict__ v_first,
     int blend, const float* __restrict__ lam_p, T* __restrict__ q_out, T* __restrict__ k_stage, T* __restrict__ v_stage,
     const int* __restrict__ seq_tile0, T* __restrict__ k_pages, T* __restrict__ v_pages,
@@ -34,7 +35,7 @@ __global__ __launch_bounds__(PACK_THREADS) void qkv_pack_kernel(
   const int t = blockIdx.x, tid = threadIdx.x;
   const int Q = n_heads * d, K = n_kv_heads * d, V = n_kv_heads * dv, N = Q + K + (v_from_k ? 0 : V);
   float* head_f = row + N;                        // head_norm: 1 / rms of each query head, then of each key head
-  const float* src = qkv + (size_t)t * N;
+  const float* src = qkv + (size_t)t * qkv_row;
   float sq = 0.f, sk = 0.f;
 #pragma unroll 4
   for (int i = tid; i < N; i += PACK_THREADS) {
@@ -150,7 +151,7 @@ constexpr int PW_WAVES = 4;
 // SHAPED: with norms a head, values that are the keys, or the rotation (the other models run the code without them)
 template <typename T, int NV, bool SHAPED>
 __global__ __launch_bounds__(PW_WAVES * WAVE) void qkv_pack_wave_kernel(
-    const float* __restrict__ qkv, const float* __restrict__ bias, const float* __restrict__ w_q,
+    const float* __restrict__ qkv, long qkv_row, const float* __restrict__ bias, const float* __restrict__ w_q,
     const float* __restrict__ w_k, float eps, float temp_coef, int temp_every, float q_scale, float* __restrict__ v_first,
     int blend, const float* __restrict__ lam_p, T* __restrict__ q_out, T* __restrict__ k_stage, T* __restrict__ v_stage,
     const int* __restrict__ seq_tile0, T* __restrict__ k_pages, T* __restrict__ v_pages,
@@ -163,7 +164,7 @@ __global__ __launch_bounds__(PW_WAVES * WAVE) void qkv_pack_wave_kernel(
   const int t = blockIdx.x * PW_WAVES + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   if (t >= n_tokens) return;
   const int Q = n_heads * d, K = n_kv_heads * d, V = n_kv_heads * dv, N = Q + K + (v_from_k ? 0 : V);
-  const float* src = qkv + (size_t)t * N;
+  const float* src = qkv + (size_t)t * qkv_row;
   float4 r[NV], wt[NV];                           // the row and the norm weights of its elements: every load asked for at once
   float sq = 0.f, sk = 0.f;
 #pragma unroll
@@ -394,7 +395,7 @@ extern "C" int yalm_v_tiles(const void* v_rows, void* v_stage, void* v_pages, co
   return launch_status();
 }
 
-extern "C" int yalm_qkv_pack(const float* qkv, const float* bias, const float* w_q, const float* w_k, float eps,
+extern "C" int yalm_qkv_pack(const float* qkv, long qkv_row, const float* bias, const float* w_q, const float* w_k, float eps,
                              float temp_coef, int temp_every, float q_scale, float* v_first, int blend,
                              const float* lam, void* q_out, void* k_stage, void* v_stage, const int* seq_tile0,
                              void* k_pages, void* v_pages, const int* block_table, int table_stride, int ring_pages,
@@ -414,11 +415,11 @@ extern "C" int yalm_qkv_pack(const float* qkv, const float* bias, const float* w
     return YALM_ERR_ARG;
   const int n_row = n_heads * d + n_kv_heads * (d + (v_from_k ? 0 : dv));
   const size_t lds = (size_t)(n_row + n_heads + n_kv_heads) * sizeof(float);
-  if (lds > 64 * 1024) return YALM_ERR_ARG;
+  if (lds > 64 * 1024 || qkv_row < n_row) return YALM_ERR_ARG;
   // a wave a token where a lane can take four elements at a time and the row fits its registers, and where the tokens
   // are many: a few tokens are done sooner by 1,024 threads each (8 tokens of 6,144 numbers: 12 against 25 us)
   const bool heads_fit = !head_norm || (d >= 4 && d <= 256 && (d & (d - 1)) == 0);      // a head in neighbouring lanes
-  const bool by_wave = heads_fit && T >= 32 && d % 4 == 0 && dv % 4 == 0 && n_row <= 256 * 32 &&
+  const bool by_wave = heads_fit && T >= 32 && d % 4 == 0 && dv % 4 == 0 && qkv_row % 4 == 0 && n_row <= 256 * 32 &&
                        ((((uintptr_t)qkv) | ((uintptr_t)bias) | ((uintptr_t)w_q) | ((uintptr_t)w_k) | ((uintptr_t)v_first) |
                          ((uintptr_t)q_out) | ((uintptr_t)k_stage) | ((uintptr_t)k_pages) | ((uintptr_t)v_rows)) & 15) == 0;
   if (by_wave) {
@@ -428,7 +429,7 @@ extern "C" int yalm_qkv_pack(const float* qkv, const float* bias, const float* w
   do { if (shaped) YALM_PACK_WS(TYPE, NV_, true); else YALM_PACK_WS(TYPE, NV_, false); } while (0)
 #define YALM_PACK_WS(TYPE, NV_, SHAPED_)                                                                                 \
   qkv_pack_wave_kernel<TYPE, NV_, SHAPED_><<<blocks, PW_WAVES * WAVE, 0, stream>>>(                                               \
-      qkv, bias, w_q, w_k, eps, temp_coef, temp_every, q_scale, v_first, blend, lam, (TYPE*)q_out, (TYPE*)k_stage,        \
+      qkv, qkv_row, bias, w_q, w_k, eps, temp_coef, temp_every, q_scale, v_first, blend, lam, (TYPE*)q_out, (TYPE*)k_stage,        \
       (TYPE*)v_stage, seq_tile0, (TYPE*)k_pages, (TYPE*)v_pages, block_table, table_stride, ring_pages, tok_seq,         \
       tok_pos, seq_slot, seq_len, T, n_heads, n_kv_heads, d, dv, pad, n_pages, page_layout, (TYPE*)v_rows, head_norm,    \
       v_from_k, (const float2*)cos_sin, rot_dims, n_positions)
@@ -455,7 +456,7 @@ extern "C" int yalm_qkv_pack(const float* qkv, const float* bias, const float* w
   if (wide) YALM_PACK_N(TYPE, 1024); else YALM_PACK_N(TYPE, 256)
 #define YALM_PACK_N(TYPE, NT)                                                                                        \
   qkv_pack_kernel<TYPE, NT><<<T, NT, lds, stream>>>(                                                                 \
-      qkv, bias, w_q, w_k, eps, temp_coef, temp_every, q_scale, v_first, blend, lam, (TYPE*)q_out, (TYPE*)k_stage,    \
+      qkv, qkv_row, bias, w_q, w_k, eps, temp_coef, temp_every, q_scale, v_first, blend, lam, (TYPE*)q_out, (TYPE*)k_stage,    \
       (TYPE*)v_stage, seq_tile0, (TYPE*)k_pages, (TYPE*)v_pages, block_table, table_stride, ring_pages, tok_seq,     \
       tok_pos, seq_slot, seq_len, n_heads, n_kv_heads, d, dv, pad, n_pages, page_layout, (TYPE*)v_rows, head_norm,    \
       v_from_k, (const float2*)cos_sin, rot_dims, n_positions)

@@ -93,7 +93,7 @@ template <int MT, int NT, int NWAVES, int EPI, int KS, bool PREFETCH = true, int
 __global__ __launch_bounds__(NWAVES * WAVE) void gemm_skinny_kernel(const bf16* __restrict__ X,
                                                                      const bf16* __restrict__ W,
                                                                      void* __restrict__ Cv, int M, int N, int K,
-                                                                     int H, ChainArgs ca) {
+                                                                     GateOut H, ChainArgs ca) {
   constexpr int KC = 32 * KS;                    // k per wave iteration
   constexpr int G = NT / TW;                     // groups of waves, each with TW tiles
   constexpr int KW = NWAVES / G;                 // waves of a group: they split K
@@ -332,7 +332,7 @@ __global__ __launch_bounds__(NWAVES * WAVE) void gemm_skinny_kernel(const bf16* 
       for (int r = 0; r < 4; ++r) {
         int m = mt * 16 + 4 * q + r;
         if (m < M && hcol < H)
-          C[(size_t)m * H + hcol] = static_cast<bf16>(gate_act<EPI>(g[r] * scale[r]) * (u[r] * scale[r]));
+          C[(size_t)m * H + hcol] = static_cast<bf16>(gate_unit<EPI>(g[r] * scale[r], u[r] * scale[r], H));
       }
       continue;
     }
@@ -432,7 +432,7 @@ __global__ __launch_bounds__(NWAVES * WAVE) void gemm_skinny_kernel(const bf16* 
 // batch rows (only when the split-K kernel refused the shape) keep 128-wide chunks for the registers.
 // the LDS-DMA variant: its ring of stages is dynamic LDS, which has to be allowed once beyond 64 KB
 template <int NT, int NWAVES, int EPI, int TW, int S, int XR, int RW = 16 * NT>
-int launch_dma(const bf16* X, const bf16* W, void* C, int M, int N, int K, int H, const ChainArgs& ca,
+int launch_dma(const bf16* X, const bf16* W, void* C, int M, int N, int K, GateOut H, const ChainArgs& ca,
                hipStream_t stream) {
   constexpr size_t lds = (size_t)NWAVES * S * (16 * TW + XR) * 128;
   static_assert(lds + NWAVES * TW * WAVE * 16 + 1024 <= 160 * 1024, "the ring and the partial sums fit the LDS of a CU");
@@ -444,7 +444,7 @@ int launch_dma(const bf16* X, const bf16* W, void* C, int M, int N, int K, int H
 }
 
 template <int MT, int EPI>
-int launch_mt(const bf16* X, const bf16* W, void* C, int M, int N, int K, int H, const ChainArgs& ca,
+int launch_mt(const bf16* X, const bf16* W, void* C, int M, int N, int K, GateOut H, const ChainArgs& ca,
               hipStream_t stream) {
   constexpr int E = gated(EPI) ? EPI_F32 : EPI;   // the gated epilogue needs pairs of tiles
   const bool emit = ca.emit_nw != nullptr;
@@ -492,7 +492,7 @@ int launch_mt(const bf16* X, const bf16* W, void* C, int M, int N, int K, int H,
 }
 
 template <int EPI>
-int launch(const bf16* X, const bf16* W, void* C, int M, int N, int K, int H, const ChainArgs& ca,
+int launch(const bf16* X, const bf16* W, void* C, int M, int N, int K, GateOut H, const ChainArgs& ca,
            hipStream_t stream) {
   switch ((M + 15) / 16) {
     case 1: return launch_mt<1, EPI>(X, W, C, M, N, K, H, ca, stream);

@@ -36,8 +36,11 @@ int yalm_rmsnorm(const float* x, const void* w, int w_dtype, void* out, int out_
 // fused_ffn_w1_w3_glu_act (src/infer.cu:250-337, 610-634)
 // workspace: float32 scratch (may be null) for kernels that split K across workgroups; they
 // use as many slices as it holds (slices * M * N floats).
+// gate_limit, gate_alpha, up_shift (epilogue 3 only): with gate_limit > 0 the gate is min(gate, limit) and up is clamped to
+// +-limit; the unit is gate / (1 + exp(-gate_alpha gate)) * (up + up_shift) (0, 1, 0: silu(gate) * up).
 int yalm_gemm(const void* A, const void* W, void* C, float* workspace, long workspace_floats, int M, int N, int K,
-              int dtype, int epilogue, int H, int force_simple, hipStream_t stream);
+              int dtype, int epilogue, int H, float gate_limit, float gate_alpha, float up_shift, int force_simple,
+              hipStream_t stream);
 
 // Floats of workspace with which the tiled bfloat16 kernel for more than 64 rows splits K (0: it does
 // not; the output's tiles fill the chip).
@@ -301,11 +304,12 @@ int yalm_moe_route(const void* h, const void* w_router, int dtype, int* ids, flo
 // weighted by the softmax over the chosen logits alone.
 int yalm_moe_select(const float* logits, const float* bias, int* ids, float* wts, int T, int E, int top, int renorm,
                     hipStream_t stream);
-// Sigmoid scores and choice inside the best groups: s = sigmoid(logit), c = s + correction (float32 [E], may be null);
-// neighbours form n_groups equal groups, a group's score is the sum of its two largest c, experts outside the `keep` best
+// Choice inside the best groups: s = sigmoid(logit), or with `softmax` the softmax over all experts, c = s + correction
+// (float32 [E], may be null); neighbours form n_groups equal groups, a group's score is the sum of its two largest c (with
+// `group_max` its largest c), experts outside the `keep` best
 // groups are out, the `top` (<= keep * E / n_groups) largest c are chosen and weigh s / (sum of the chosen s + 1e-20) * scale.
 int yalm_moe_select_groups(const float* logits, const float* correction, int* ids, float* wts, int T, int E, int top,
-                           int n_groups, int keep, float scale, hipStream_t stream);
+                           int n_groups, int keep, float scale, int softmax, int group_max, hipStream_t stream);
 // w_gate null (here and in yalm_moe_grouped): experts of two matrices, mid = relu(w_up h)^2.
 // up_shift: the number added to the clamped up value (mid = g sigmoid(alpha g) (u + up_shift); the text above has 1;
 // alpha 1, limit 0 and up_shift 0 give silu(gate) * up).
@@ -339,8 +343,8 @@ int yalm_embed_sinusoid(const void* table, int table_dtype, const int* tokens, c
 // over each head's d elements instead, with w_q and w_k of d elements shared by the heads.  v_from_k != 0: qkv has no value
 // part, [T, H d + G d], and a head's values are its keys as projected, before their norm (dv = d, no blend).  rot_dims > 0:
 // behind the norms, the neighbours (2p, 2p + 1), p < rot_dims / 2, of every query and key head are turned by the angle
-// cos_sin[position][p] ((cos, sin) float32 [n_positions, rot_dims / 2, 2]).
-int yalm_qkv_pack(const float* qkv, const float* bias, const float* w_q, const float* w_k, float eps, float temp_coef,
+// cos_sin[position][p] ((cos, sin) float32 [n_positions, rot_dims / 2, 2]).  The rows of qkv are qkv_row apart.
+int yalm_qkv_pack(const float* qkv, long qkv_row, const float* bias, const float* w_q, const float* w_k, float eps, float temp_coef,
                   int temp_every, float q_scale, float* v_first, int blend, const float* lam, void* q_out, void* k_stage,
                   void* v_stage, const int* seq_tile0, void* k_pages, void* v_pages, const int* block_table,
                   int table_stride, int ring_pages, const int* tok_seq, const int* tok_pos, const int* seq_slot,
@@ -411,8 +415,9 @@ int yalm_gated_add(const float* y, const void* h, const void* w, int dtype, floa
 // each sequence (h, out [T, D] of `dtype`, not the same memory; w float32 [taps, D], tap by tap, the last tap on the token itself).
 // carried, float32 [n_slots, taps - 1, D], holds each sequence's last taps - 1 inputs (the newest last): read for the
 // places in front of the step's first token, then left advanced.  Rows of padding (slot -1) read zeros and keep nothing.
-// one_each != 0: every sequence brings one token (T = B, row t is sequence t), which lets one launch do both.
-int yalm_time_conv(const void* h, const float* w, float* carried, void* out, const int* tok_seq, const int* cu_seqlens,
+// one_each != 0: every sequence brings one token (T = B, row t is sequence t), which lets one launch do both.  The rows of h
+// are h_row apart; in_bias (float32 [D], may be null) is added to every input (the carried ones hold it), out_bias to every sum.
+int yalm_time_conv(const void* h, long h_row, const float* in_bias, const float* out_bias, const float* w, float* carried, void* out, const int* tok_seq, const int* cu_seqlens,
                    const int* seq_slot, int T, int B, int D, int taps, int residual, int one_each, int dtype, hipStream_t stream);
 // out[t, i] = act(z[t, i] + bias[i]) * (z[t, F + i] + bias[F + i]), i < F: z float32 [T, 2 F] (gate | up), bias float32
 // [2 F] or null, out of `out_dtype`, kind as yalm_activate; with x_bias (float32 [D]) also x[t, :] += x_bias (x float32 [T, D]).
@@ -449,6 +454,50 @@ int yalm_gla_tiles(const float* proj, const float* w2, const float* bias, const 
                    float* kd, float* gd, const int* cu_seqlens, const int* seq_slot, const int* seq_tile0, int n_tiles, void* out,
                    int T, int B, int n_heads, int d, int dv, int rank, float q_scale, float inv_tau, float eps, int out_dtype,
                    hipStream_t stream);
+
+// out[t, h, e] = o[t, h, e] * sigmoid(g[t * g_row + h]) * scale, e < dv: o of `dtype` [T, n_heads, dv], g float32, rows of out
+// out_row apart (out may be o itself where they are o's).
+int yalm_head_gate(const void* o, const float* g, long g_row, float scale, void* out, long out_row, int T, int n_heads, int dv,
+                   int dtype, hipStream_t stream);
+// z[i] = cap tanh(z[i] / cap), in place.
+int yalm_softcap(float* z, long n, float cap, hipStream_t stream);
+
+// An elementwise squash in a norm's place, n(v) = tanh(alpha v) * w + b (w, b float32 [D]).  y null: h[r] = n(x[row_index[r] or
+// r]) in `h_dtype`.  Else x[r] += mult * n(y[r] + y_bias) (x, y float32 [R, D]; y_bias float32 [D] or null), and h (may be null)
+// receives the new x, or with next_w that squash (next_alpha, next_w, next_b) of the new x.
+int yalm_squash(float* x, const float* y, const float* y_bias, float mult, const int* row_index, float alpha, const float* w,
+                const float* b, void* h, int h_dtype, float next_alpha, const float* next_w, const float* next_b, int R, int D,
+                hipStream_t stream);
+// out[r] = x[r] / sqrt(mean(x[r]^2) + eps) * w * sigmoid(gate[r]): x float32 [R, n], w float32 [n], rows of gate (float32) and
+// out (`out_dtype`) gate_row and out_row apart.
+int yalm_rms_gate(const float* x, const float* w, float eps, const float* gate, long gate_row, void* out, long out_row, int out_dtype,
+                  int R, int n, hipStream_t stream);
+
+// Linear attention under a fixed decay a head (lightning.hip): proj float32, rows `row` apart, their first columns z_q | z_k |
+// z_v (H d, H d, H dv); q, k, v = silu of them; per head S <- g S + k v^T, raw [T, H dv] = S^T q.  powers float32 [H, 65]: g^0 ..
+// g^64 of every head.  State, sequences and padding rows as for yalm_hgrn2.  d <= 256.
+int yalm_lightning(const float* proj, long row, const float* powers, float* state, float* raw, const int* cu_seqlens,
+                   const int* seq_slot, int T, int B, int n_heads, int d, int dv, hipStream_t stream);
+// The same for steps of prompts, a tile of 64 tokens at a time (seq_tile0, n_tiles and scratch as for yalm_gla_tiles, DP =
+// yalm_lightning_tiles_fit(d); 0: not taken).
+int yalm_lightning_tiles_fit(int d);
+int yalm_lightning_tiles(const float* proj, long row, const float* powers, float* state, float* raw, float* qd, float* kd, float* gd,
+                         const int* cu_seqlens, const int* seq_slot, const int* seq_tile0, int n_tiles, int T, int B, int n_heads,
+                         int d, int dv, hipStream_t stream);
+
+// The gated linear recurrence on every channel (lru.hip): u float32 [T, W] in blocks of n channels; r, i = sigmoid of the blocks'
+// products with w (`w_dtype` [2, W / n, n, n], [out, in] each; bias float32 [2, W]); a = exp(slope r), S <- a S + sqrt(1 - a^2) i
+// u, out (`out_dtype` [T, W]) = S gelu(z + z_bias) (gelu in its tanh form; z float32, rows z_row apart).  state float32 [slots,
+// W], read and left advanced.  Steps of prompts: seq_tile0 int32 [B + 1] (tiles of 64 tokens, n_tiles in all), scratch ends
+// float32 [n_tiles, 2, W]; seq_tile0 null: a step of single tokens (T = B, row t is sequence t; slot -1: zeros, no state).  Scratch
+// P, Q float32 [T, W].  yalm_lru_step: single tokens in one launch.
+int yalm_lru(const float* u, const void* w, int w_dtype, const float* bias, const float* slope, const float* z, long z_row,
+             const float* z_bias, float* state, float* P, float* Q, float* ends, const int* tok_seq, const int* cu_seqlens,
+             const int* seq_slot, const int* seq_tile0, int n_tiles, void* out, int out_dtype, int T, int B, int W, int n,
+             int force_simple, hipStream_t stream);
+int yalm_lru_step(const float* u, const void* w, int w_dtype, const float* bias, const float* slope, const float* z, long z_row,
+                  const float* z_bias, float* state, const int* seq_slot, void* out, int out_dtype, int B, int W, int n,
+                  hipStream_t stream);
 
 // Yardsticks for the measurement (probes.hip): a kernel that only reads `bytes` bytes once with `workgroups`
 // workgroups (out: 1,024 words of scratch), and a loop of matrix-core instructions on registers (shape 32:

@@ -71,6 +71,14 @@ def _need(t, name, dtype=None, shape=None):
     return t.data_ptr()
 
 
+def _rows(t, name, T, width):
+    """(address, elements from row to row) of a float32 [T, width] on the device whose rows may be parts of wider rows."""
+    if not isinstance(t, torch.Tensor) or t.dtype != torch.float32 or t.dim() != 2 or tuple(t.shape) != (T, width) \
+            or t.stride(1) != 1 or not t.is_cuda:
+        raise ValueError("%s: float32 [%d, %d] on the device with contiguous rows is expected" % (name, T, width))
+    return t.data_ptr(), t.stride(0)
+
+
 def _opt(t, name, dtype=None, shape=None):
     return None if t is None else _need(t, name, dtype, shape)
 
@@ -133,14 +141,16 @@ def gemm_workspace_floats(M, N, K):
     return 0
 
 
-def gemm(a, w, out, epilogue, hidden=0, workspace=None, scale_from=None):
+def gemm(a, w, out, epilogue, hidden=0, workspace=None, scale_from=None, unit=None):
     """out = a[M,K] @ w[N,K]^T with float32 accumulation and one of four epilogues:
     EPI_STORE_F32 (float32 out), EPI_STORE (out in a's dtype), EPI_ADD_F32
     (float32 out += product), EPI_GATED (w = gate/up rows interleaved in blocks of
     16; out[M, hidden] = silu(gate) * up in a's dtype; EPI_GATED_GELU: gelu(gate) * up).  workspace: float32 scratch of
     gemm_workspace_floats(M, N, K) elements, with which small batches split K.
     scale_from = (ss float32 [M, parts], eps), 17..128 bfloat16 rows only (can_add_emit): a was emitted by
-    gemm_add_emit, and the sums are scaled by rsqrt(sum(ss[m]) / K + eps) per row before the epilogue."""
+    gemm_add_emit, and the sums are scaled by rsqrt(sum(ss[m]) / K + eps) per row before the epilogue.
+    unit = (limit, alpha, shift), EPI_GATED only: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g)
+    (u + shift) (limit 0: unclamped; None: silu(gate) * up)."""
     M, K = a.shape
     N = w.shape[0]
     dt = a.dtype
@@ -159,6 +169,9 @@ def gemm(a, w, out, epilogue, hidden=0, workspace=None, scale_from=None):
     p_ws, n_ws = None, 0
     if workspace is not None:
         p_ws, n_ws = _need(workspace, "workspace", torch.float32), workspace.numel()
+    if unit is not None and (epilogue != EPI_GATED or scale_from is not None):
+        raise ValueError("gemm: a unit's constants go with the gated epilogue and without a row scale")
+    limit, alpha, shift = unit if unit is not None else (0.0, 1.0, 0.0)
     if scale_from is not None:
         ss, eps = scale_from
         if dt != torch.bfloat16:
@@ -168,7 +181,7 @@ def gemm(a, w, out, epilogue, hidden=0, workspace=None, scale_from=None):
                                                      ss.shape[1], float(eps), _stream()), "gemm with a row scale")
         return out
     library.check(library.lib().yalm_gemm(p_a, p_w, p_o, p_ws, n_ws, M, N, K, dtype_code(dt), epilogue, hidden,
-                                          1 if FORCE_SIMPLE else 0, _stream()), "gemm")
+                                          float(limit), float(alpha), float(shift), 1 if FORCE_SIMPLE else 0, _stream()), "gemm")
     return out
 
 
@@ -826,6 +839,50 @@ def layer_norm_sum(y, weight, bias, eps, alpha, x, h_out=None, next_norm=None):
     return x
 
 
+def squash(x, alpha, weight, bias, out, row_index=None):
+    """out[r] = tanh(alpha x[row(r)]) * weight + bias; x, weight and bias float32, out [R, D] float32 or the compute dtype,
+    row(r) = row_index[r] (int32) or r."""
+    D = x.shape[1]
+    R = x.shape[0] if row_index is None else row_index.shape[0]
+    library.check(library.lib().yalm_squash(
+        _need(x, "x", torch.float32, (None, D)), None, None, 1.0, _opt(row_index, "row_index", torch.int32, (R,)), float(alpha),
+        _need(weight, "weight", torch.float32, (D,)), _need(bias, "bias", torch.float32, (D,)), _need(out, "out", None, (R, D)),
+        dtype_code(out.dtype), 0.0, None, None, R, D, _stream()), "squash")
+    return out
+
+
+def squash_add(y, alpha, weight, bias, mult, x, h_out=None, next_norm=None, y_bias=None):
+    """x += mult * (tanh(alpha (y + y_bias)) * weight + bias), row by row (x, y float32 [R, D]; y_bias float32 [D] or None);
+    h_out (optional, the compute dtype) receives the new x, or with next_norm = (alpha, float32 weight, bias) that squash of it."""
+    R, D = y.shape
+    p_h, h_code = None, 0
+    if h_out is not None:
+        p_h, h_code = _need(h_out, "h_out", None, (R, D)), dtype_code(h_out.dtype)
+    n_alpha, p_w, p_b = 0.0, None, None
+    if next_norm is not None:
+        if h_out is None:
+            raise ValueError("squash_add: the next norm's output needs h_out")
+        n_alpha = float(next_norm[0])
+        p_w, p_b = (_need(t, "next norm", torch.float32, (D,)) for t in next_norm[1:])
+    library.check(library.lib().yalm_squash(
+        _need(x, "x", torch.float32, (R, D)), _need(y, "y", torch.float32, (R, D)), _opt(y_bias, "y_bias", torch.float32, (D,)),
+        float(mult), None, float(alpha), _need(weight, "weight", torch.float32, (D,)), _need(bias, "bias", torch.float32, (D,)),
+        p_h, h_code, n_alpha, p_w, p_b, R, D, _stream()), "squash_add")
+    return x
+
+
+def rms_gate(x, weight, eps, gate, out):
+    """out[r] = x[r] / sqrt(mean(x[r]^2) + eps) * weight * sigmoid(gate[r]): x float32 [R, n], weight float32 [n]; gate (float32)
+    and out (the compute dtype) [R, n], whose rows may be parts of wider ones."""
+    R, n = x.shape
+    if tuple(out.shape) != (R, n) or out.stride(1) != 1 or not out.is_cuda:
+        raise ValueError("rms_gate: out must be [%d, %d] on the device with contiguous rows" % (R, n))
+    library.check(library.lib().yalm_rms_gate(
+        _need(x, "x", torch.float32, (R, n)), _need(weight, "weight", torch.float32, (n,)), float(eps), *_rows(gate, "gate", R, n),
+        out.data_ptr(), out.stride(0), dtype_code(out.dtype), R, n, _stream()), "rms_gate")
+    return out
+
+
 def polynorm(z, coef, eps, out):
     """out[r] = a N(z[r]) + b N(z[r]^2) + c N(z[r]^3) + e, powers element by element, N(v) = v / sqrt(mean(v^2) + eps);
     z float32 [R, F], coef float32 [4] = (a, b, c, e) on the device, out [R, F] in the compute dtype."""
@@ -942,7 +999,7 @@ def v_tiles(v_rows, v_stage, v_pages, cu_seqlens, seq_tile0, block_table, ring_p
 def qkv_pack(qkv, bias, w_q, w_k, eps, q_temp, q_scale, v_first, blend, lam, q_out, k_stage, v_stage, seq_tile0, k_pages,
              v_pages, block_table, ring_pages, tok_seq, tok_pos, seq_slot, seq_len, n_heads, n_kv_heads, d, dv, pad,
              v_rows=None, head_norm=False, v_from_k=False, cos_sin=None, rot_dims=0):
-    """From a q/k/v product to an attention without rotation.  qkv float32 [T, H d + G d + G dv] (+ bias, float32 of
+    """From a q/k/v product to an attention without rotation.  qkv float32 [T, H d + G d + G dv] (its rows may be parts of wider ones; + bias, float32 of
     that width or None); RMS norms over the WHOLE query and key projections with the weights w_q [H d], w_k [G d]
     (float32; None: no norm); the queries times q_scale and, with q_temp = (coef, every), times 1 + coef ln(floor((p + 1)
     / every) + 1) at position p; blend 1 stores the values in v_first (float32 [T, G dv]), blend 2 replaces them by
@@ -978,7 +1035,7 @@ def qkv_pack(qkv, bias, w_q, w_k, eps, q_temp, q_scale, v_first, blend, lam, q_o
         if ring_pages <= 0 or ring_pages > stride:
             raise ValueError("ring_pages %d does not fit the block table (%d columns)" % (ring_pages, stride))
     library.check(library.lib().yalm_qkv_pack(
-        _need(qkv, "qkv", torch.float32, (T, N)), _opt(bias, "bias", torch.float32, (N,)),
+        *_rows(qkv, "qkv", T, N), _opt(bias, "bias", torch.float32, (N,)),
         _opt(w_q, "w_q", torch.float32, (d if head_norm else Q,)), _opt(w_k, "w_k", torch.float32, (d if head_norm else K,)),
         float(eps), float(coef), int(every),
         float(q_scale), _opt(v_first, "v_first", torch.float32, (T, V)), int(blend), _opt(lam, "lam", torch.float32),
@@ -1154,10 +1211,11 @@ def gated_add(y, h, w, x, accumulate=True):
 TIME_CONV_MAX_TAPS = 16
 
 
-def time_conv(h, w, carried, out, tok_seq, cu_seqlens, seq_slot, residual=True, one_token_each=False):
-    """out[t, c] = (h[t, c] if residual) + sum_j w[j, c] in(t - (taps - 1) + j, c): a causal convolution over the tokens
-    of each sequence of the step, the last tap on the token itself (h, out [T, D] of one dtype and not the same
-    memory; w float32 [taps, D], tap by tap).  carried (float32 [slots, taps - 1, D]; None with one tap) holds each sequence's last
+def time_conv(h, w, carried, out, tok_seq, cu_seqlens, seq_slot, residual=True, one_token_each=False, in_bias=None, bias=None):
+    """out[t, c] = (in(t, c) if residual) + sum_j w[j, c] in(t - (taps - 1) + j, c) + bias[c], in = h + in_bias: a causal
+    convolution over the tokens of each sequence of the step, the last tap on the token itself (h, out [T, D] of one dtype and not the same
+    memory, the rows of h may be parts of wider ones; w float32 [taps, D], tap by tap; in_bias, bias float32 [D] or None).
+    carried (float32 [slots, taps - 1, D]; None with one tap) holds each sequence's last
     taps - 1 inputs, read for the places in front of the step's first token and left advanced.  one_token_each: the caller
     knows that every sequence brings one token (row t is sequence t), which saves a launch."""
     T, D = h.shape
@@ -1167,11 +1225,14 @@ def time_conv(h, w, carried, out, tok_seq, cu_seqlens, seq_slot, residual=True, 
         raise ValueError("time_conv: %d taps (at most %d)" % (taps, TIME_CONV_MAX_TAPS))
     if h.data_ptr() == out.data_ptr():
         raise ValueError("time_conv: the result needs memory of its own")
+    if not h.is_cuda or h.stride(1) != 1:
+        raise ValueError("time_conv: the inputs' rows are contiguous and on the device")
     p_c = None
     if taps > 1:
         p_c = _need(carried, "carried", torch.float32, (None, taps - 1, D))
     library.check(library.lib().yalm_time_conv(
-        _need(h, "h", None, (T, D)), _need(w, "w", torch.float32, (taps, D)), p_c, _need(out, "out", h.dtype, (T, D)),
+        h.data_ptr(), h.stride(0), _opt(in_bias, "in_bias", torch.float32, (D,)), _opt(bias, "bias", torch.float32, (D,)),
+        _need(w, "w", torch.float32, (taps, D)), p_c, _need(out, "out", h.dtype, (T, D)),
         _need(tok_seq, "tok_seq", torch.int32, (T,)), _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)),
         _need(seq_slot, "seq_slot", torch.int32, (B,)), T, B, D, taps, 1 if residual else 0,
         1 if one_token_each and T == B else 0, dtype_code(h.dtype), _stream()),
@@ -1208,6 +1269,25 @@ def sigmoid_gate(o, g, n_heads, dv, pad):
         _need(o, "o", None, (T, n_heads * pad)), g.data_ptr(), int(g.stride(0)), T, n_heads, dv, pad, dtype_code(o.dtype),
         _stream()), "sigmoid_gate")
     return o
+
+
+def head_gate(o, g, n_heads, scale=1.0, out=None):
+    """out[t, h, :] = o[t, h, :] * sigmoid(g[t, h]) * scale: o [T, n_heads dv], g float32 [T, n_heads] (its rows may be parts of
+    wider ones), out [T, n_heads dv] of o's dtype, rows likewise (None: in place)."""
+    T, W = o.shape
+    out = o if out is None else out
+    if out.dtype != o.dtype or tuple(out.shape) != (T, W) or out.stride(1) != 1 or not out.is_cuda or W % n_heads:
+        raise ValueError("head_gate: %s does not hold the result of %d heads in %s" % (list(out.shape), n_heads, list(o.shape)))
+    library.check(library.lib().yalm_head_gate(
+        _need(o, "o", None, (T, W)), *_rows(g, "g", T, n_heads), float(scale), out.data_ptr(), out.stride(0), T, n_heads, W // n_heads,
+        dtype_code(o.dtype), _stream()), "head_gate")
+    return out
+
+
+def softcap(z, cap):
+    """z = cap tanh(z / cap), in place (float32)."""
+    library.check(library.lib().yalm_softcap(_need(z, "z", torch.float32), z.numel(), float(cap), _stream()), "softcap")
+    return z
 
 
 def loop_pack(x, x0, start, both):
@@ -1298,9 +1378,9 @@ def gla_tiles(proj, w2, bias, w_norm, state, raw, cu_seqlens, seq_slot, seq_tile
     dp = gla_tiles_fit(d, rank)
     if not dp:
         raise ValueError("gla_tiles: key heads of %d with decays of rank %d are not taken" % (d, rank))
-    qd = scratch("gla.qd", (n_tiles, n_heads, PAGE, dp), torch.float32)
-    kd = scratch("gla.kd", (n_tiles, n_heads, dp, PAGE), torch.float32)
-    gd = scratch("gla.gd", (n_tiles, n_heads, dp), torch.float32)
+    qd = scratch("scan.qd", (n_tiles, n_heads, PAGE, dp), torch.float32)
+    kd = scratch("scan.kd", (n_tiles, n_heads, dp, PAGE), torch.float32)
+    gd = scratch("scan.gd", (n_tiles, n_heads, dp), torch.float32)
     library.check(library.lib().yalm_gla_tiles(
         _need(proj, "proj", torch.float32, (T, N)), _need(w2, "w2", torch.float32, (n_heads * d, gla_padded_rank(rank))),
         _need(bias, "bias", torch.float32, (n_heads * d,)), _need(w_norm, "w_norm", torch.float32, (dv,)),
@@ -1309,6 +1389,107 @@ def gla_tiles(proj, w2, bias, w_norm, state, raw, cu_seqlens, seq_slot, seq_tile
         _need(seq_slot, "seq_slot", torch.int32, (B,)), _need(seq_tile0, "seq_tile0", torch.int32, (B + 1,)), n_tiles,
         _need(out, "out", None, (T, n_heads * dv)), T, B, n_heads, d, dv, rank, float(q_scale), 1.0 / float(tau), float(eps),
         dtype_code(out.dtype), _stream()), "gla_tiles")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------------------------
+# linear attention under a fixed decay a head
+LIGHTNING_MAX_KEY_DIM = 256
+LIGHTNING_POWERS = PAGE + 1
+
+
+def lightning_state_elements(n_heads, d, dv):
+    return n_heads * d * dv
+
+
+def lightning_tiles_fit(d):
+    """The padded key size with which lightning_tiles takes key heads of d, or 0: it does not."""
+    return library.lib().yalm_lightning_tiles_fit(int(d))
+
+
+def _lightning_args(proj, powers, state, raw, n_heads, d, dv):
+    T = raw.shape[0]
+    if not 0 < d <= LIGHTNING_MAX_KEY_DIM:
+        raise ValueError("lightning: key heads of %d (at most %d)" % (d, LIGHTNING_MAX_KEY_DIM))
+    return T, (*_rows(proj, "proj", T, n_heads * (2 * d + dv)), _need(powers, "powers", torch.float32, (n_heads, LIGHTNING_POWERS)),
+               _need(state, "state", torch.float32, (None, n_heads * d * dv)), _need(raw, "raw", torch.float32, (T, n_heads * dv)))
+
+
+def lightning(proj, powers, state, raw, cu_seqlens, seq_slot, n_heads, d, dv):
+    """Linear attention under a fixed decay a head, over a step's tokens.  proj float32 [T, 2 H d + H dv] = z_q | z_k | z_v (rows
+    may be parts of wider ones); q, k, v = silu of them; per head S <- g S + k v^T, raw float32 [T, H dv] = S^T q; powers
+    float32 [H, 65]: g^0 .. g^64 of every head.  state float32 [slots, H dv d] (a head's S column by column) is read and left
+    advanced.  Sequence b's tokens are cu_seqlens[b] .. cu_seqlens[b + 1] - 1."""
+    B = seq_slot.shape[0]
+    T, args = _lightning_args(proj, powers, state, raw, n_heads, d, dv)
+    library.check(library.lib().yalm_lightning(
+        *args, _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)), _need(seq_slot, "seq_slot", torch.int32, (B,)), T, B, n_heads,
+        d, dv, _stream()), "lightning")
+    return raw
+
+
+def lightning_tiles(proj, powers, state, raw, cu_seqlens, seq_slot, seq_tile0, n_tiles, n_heads, d, dv, scratch):
+    """lightning for a step of prompts, a tile of 64 tokens at a time on the matrix cores in float32; seq_tile0 int32 [B + 1],
+    the first tile of every sequence (n_tiles in all).  scratch(name, shape, dtype) hands out the buffers."""
+    B = seq_slot.shape[0]
+    T, args = _lightning_args(proj, powers, state, raw, n_heads, d, dv)
+    dp = lightning_tiles_fit(d)
+    if not dp:
+        raise ValueError("lightning_tiles: key heads of %d are not taken" % d)
+    qd = scratch("scan.qd", (n_tiles, n_heads, PAGE, dp), torch.float32)
+    kd = scratch("scan.kd", (n_tiles, n_heads, dp, PAGE), torch.float32)
+    gd = scratch("scan.gd", (n_tiles, n_heads, dp), torch.float32)
+    library.check(library.lib().yalm_lightning_tiles(
+        *args, qd.data_ptr(), kd.data_ptr(), gd.data_ptr(), _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)),
+        _need(seq_slot, "seq_slot", torch.int32, (B,)), _need(seq_tile0, "seq_tile0", torch.int32, (B + 1,)), n_tiles, T, B, n_heads,
+        d, dv, _stream()), "lightning_tiles")
+    return raw
+
+
+# ---------------------------------------------------------------------------------------------------------------
+# a gated linear recurrence on every channel
+LRU_STEP_MAX_ROWS = 16           # bfloat16 steps of more single tokens form the gates on the matrix cores
+
+
+def _lru_args(u, w, bias, slope, z, z_bias):
+    T, W = u.shape
+    n = w.shape[-1]
+    if w.dim() != 4 or w.shape[0] != 2 or w.shape[2] != n or w.shape[1] * n != W:
+        raise ValueError("lru: the gates' matrices %s do not fit %d channels" % (list(w.shape), W))
+    return (_need(u, "u", torch.float32, (T, W)), _need(w, "w"), dtype_code(w.dtype), _need(bias, "bias", torch.float32, (2, W)),
+            _need(slope, "slope", torch.float32, (W,)), *_rows(z, "z", T, W), _need(z_bias, "z_bias", torch.float32, (W,)))
+
+
+def lru(u, w, bias, slope, z, z_bias, state, out, tok_seq, cu_seqlens, seq_slot, scratch, seq_tile0=None, n_tiles=0):
+    """The gated linear recurrence over a step's tokens.  u float32 [T, W] in blocks of n channels; r, i = sigmoid(w[0], w[1] in
+    every block, plus bias) (w [2, W / n, n, n], [out, in] each; bias float32 [2, W]); a = exp(slope r) (slope float32 [W],
+    negative); S <- a S + sqrt(1 - a^2) i u; out [T, W] (the compute dtype) = S gelu(z + z_bias), the gelu in its tanh form (z float32,
+    rows may be parts of wider ones).  state float32 [slots, W] is read and left advanced.  seq_tile0 int32 [B + 1]: a step of
+    prompts, every sequence's first tile of 64 tokens, n_tiles in all; None: single tokens (row t is sequence t)."""
+    T, W = u.shape
+    B = seq_slot.shape[0]
+    args = _lru_args(u, w, bias, slope, z, z_bias)
+    P, Q = scratch("lru.p", (T, W), torch.float32), scratch("lru.q", (T, W), torch.float32)
+    ends = None
+    if seq_tile0 is not None:
+        ends = scratch("lru.ends", (n_tiles, 2, W), torch.float32)
+    elif T != B:
+        raise ValueError("lru: %d tokens of %d sequences are not single tokens" % (T, B))
+    library.check(library.lib().yalm_lru(
+        *args, _need(state, "state", torch.float32, (None, W)), P.data_ptr(), Q.data_ptr(), None if ends is None else ends.data_ptr(),
+        _need(tok_seq, "tok_seq", torch.int32, (T,)), _need(cu_seqlens, "cu_seqlens", torch.int32, (B + 1,)),
+        _need(seq_slot, "seq_slot", torch.int32, (B,)), _opt(seq_tile0, "seq_tile0", torch.int32, (B + 1,)), int(n_tiles),
+        _need(out, "out", None, (T, W)), dtype_code(out.dtype), T, B, W, w.shape[-1], 1 if FORCE_SIMPLE else 0, _stream()), "lru")
+    return out
+
+
+def lru_step(u, w, bias, slope, z, z_bias, state, out, seq_slot):
+    """lru for a step of single tokens in one launch (row t is sequence t)."""
+    B, W = u.shape
+    library.check(library.lib().yalm_lru_step(
+        *_lru_args(u, w, bias, slope, z, z_bias), _need(state, "state", torch.float32, (None, W)),
+        _need(seq_slot, "seq_slot", torch.int32, (B,)), _need(out, "out", None, (B, W)), dtype_code(out.dtype), B, W, w.shape[-1],
+        _stream()), "lru_step")
     return out
 
 
@@ -1346,9 +1527,10 @@ def moe_select(logits, ids, wts, renormalize=False, bias=None):
         "moe_select")
 
 
-def moe_select_groups(logits, correction, ids, wts, n_groups=1, keep=1, scale=1.0):
-    """ids, wts [T, top] from float32 logits [T, E]: scores s = sigmoid(logit), choice scores c = s + correction (float32 [E]
-    or None); E experts form n_groups equal groups of neighbours, a group's score is the sum of its two largest c; among
+def moe_select_groups(logits, correction, ids, wts, n_groups=1, keep=1, scale=1.0, softmax=False, group_max=False):
+    """ids, wts [T, top] from float32 logits [T, E]: scores s = sigmoid(logit) (softmax: the softmax over all experts), choice
+    scores c = s + correction (float32 [E]
+    or None); E experts form n_groups equal groups of neighbours, a group's score is the sum of its two largest c (group_max: its largest c); among
     the experts of the `keep` best groups the top largest c are chosen (the lower index on ties) and weigh s / (sum of the
     chosen s + 1e-20) * scale."""
     T, E = logits.shape
@@ -1359,7 +1541,7 @@ def moe_select_groups(logits, correction, ids, wts, n_groups=1, keep=1, scale=1.
     library.check(library.lib().yalm_moe_select_groups(
         _need(logits, "logits", torch.float32, (T, E)), _opt(correction, "correction", torch.float32, (E,)),
         _need(ids, "ids", torch.int32, (T, top)), _need(wts, "wts", torch.float32, (T, top)), T, E, top, n_groups, keep,
-        float(scale), _stream()), "moe_select_groups")
+        float(scale), 1 if softmax else 0, 1 if group_max else 0, _stream()), "moe_select_groups")
 
 
 def moe_pair_gate_up(h, w_gate, w_up, ids, limit, alpha, mid, up_shift=1.0):

@@ -19,7 +19,7 @@ _SIGNATURES = {
     "yalm_error_string": (ctypes.c_char_p, [_I]),
     "yalm_embed": (_I, [_P, _I, _P, _P, _I, _I, _I, _P]),
     "yalm_rmsnorm": (_I, [_P, _P, _I, _P, _I, _P, _I, _I, _F, _P]),
-    "yalm_gemm": (_I, [_P, _P, _P, _P, ctypes.c_long, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "yalm_gemm": (_I, [_P, _P, _P, _P, ctypes.c_long, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]),
     "yalm_gemm_norm": (_I, [_P, _P, _F, _P, _P, _I, _I, _I, _I, _I, _P]),
     "yalm_gemm_norm_qkv_rope": (_I, [_P, _P, _F, _P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P]),
     "yalm_gemm_chain": (_I, [_P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _F, _P, _P, _P, _P]),
@@ -59,7 +59,7 @@ _SIGNATURES = {
     "yalm_latent_norm": (_I, [_P, ctypes.c_long, _P, _I, _F, _P, _I, _I, _I, _P]),
     "yalm_layer_norm": (_I, [_P, _P, _F, _P, _P, _P, _F, _I, _P, _I, _P, _P, _F, _I, _I, _P]),
     "yalm_embed_pairs": (_I, [_P, _P, _I, _P, _P, _P, _P, _P, _P, ctypes.c_long, ctypes.c_long, ctypes.c_long, _F, _P, _I, _I, _I, _P]),
-    "yalm_moe_select_groups": (_I, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P]),
+    "yalm_moe_select_groups": (_I, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P]),
     "yalm_gla_tiles_fit": (_I, [_I, _I]),
     "yalm_gla_tiles": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]),
     "yalm_gla": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]),
@@ -70,7 +70,7 @@ _SIGNATURES = {
     "yalm_moe_grouped_tiles": (_I, [_I, _I]),
     "yalm_moe_grouped": (_I, [_P, _P, _P, _P, _P, _P, _F, _F, _F, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P]),
     "yalm_embed_sinusoid": (_I, [_P, _I, _P, _P, _P, _F, _P, _I, _I, _I, _P]),
-    "yalm_qkv_pack": (_I, [_P, _P, _P, _P, _F, _F, _I, _F, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _P,
+    "yalm_qkv_pack": (_I, [_P, ctypes.c_long, _P, _P, _P, _F, _F, _I, _F, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _P,
                            _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _I, _I, _P, _I, _I, _P]),
     "yalm_v_tiles": (_I, [_P, _P, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
     "yalm_mlstm_chunks": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _F, _F, _I, _I, _I, _P]),
@@ -80,16 +80,25 @@ _SIGNATURES = {
     "yalm_embed_learned": (_I, [_P, _P, _I, _P, _P, _F, _P, _I, _I, _I, _I, _P]),
     "yalm_activate": (_I, [_P, _P, ctypes.c_long, _I, _I, _P]),
     "yalm_gated_add": (_I, [_P, _P, _P, _I, _P, _I, _I, _I, _P]),
-    "yalm_time_conv": (_I, [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "yalm_time_conv": (_I, [_P, ctypes.c_long, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
     "yalm_gated_bias_act": (_I, [_P, _P, _P, _I, _I, _I, _I, _P, _P, _I, _P]),
     "yalm_sigmoid_gate": (_I, [_P, _P, ctypes.c_long, _I, _I, _I, _I, _I, _P]),
     "yalm_loop_pack": (_I, [_P, _P, _P, _P, _I, _I, _I, _P]),
     "yalm_hgrn2": (_I, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P]),
+    "yalm_head_gate": (_I, [_P, _P, ctypes.c_long, _F, _P, ctypes.c_long, _I, _I, _I, _I, _P]),
+    "yalm_softcap": (_I, [_P, ctypes.c_long, _F, _P]),
+    "yalm_squash": (_I, [_P, _P, _P, _F, _P, _F, _P, _P, _P, _I, _F, _P, _P, _I, _I, _P]),
+    "yalm_rms_gate": (_I, [_P, _P, _F, _P, ctypes.c_long, _P, ctypes.c_long, _I, _I, _I, _P]),
+    "yalm_lightning": (_I, [_P, ctypes.c_long, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P]),
+    "yalm_lightning_tiles_fit": (_I, [_I]),
+    "yalm_lightning_tiles": (_I, [_P, ctypes.c_long, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P]),
+    "yalm_lru": (_I, [_P, _P, _I, _P, _P, _P, ctypes.c_long, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P]),
+    "yalm_lru_step": (_I, [_P, _P, _I, _P, _P, _P, ctypes.c_long, _P, _P, _P, _P, _I, _I, _I, _I, _P]),
     "yalm_probe_read": (_I, [_P, ctypes.c_long, _P, _I, _P]),
     "yalm_probe_mfma": (_I, [_I, _I, _I, _P, _P, _P]),
 }
 
-ABI_VERSION = 36
+ABI_VERSION = 37
 
 
 class KernelError(RuntimeError):

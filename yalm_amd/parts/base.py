@@ -12,7 +12,10 @@ it is in.  Kinds of parts and the methods each must have:
                  the cache line (line, name) for each of them
   input_filter   cache_request() as a mixer's; forward(h[T, dim], out[T, dim], ctx, line): what a sublayer reads in h's place
                  forward(h[T, dim], x_f32[T, dim], ctx, line, writes_cache): adds its output to x
-  feed_forward   forward(h[T, dim], x_f32[T, dim], ctx): adds its output to x
+                 optional: forward_to(h, y_f32[T, dim], ctx, line, writes_cache), which writes its output to y instead; a
+                 `late_bias` (float32 [dim]) that its output lacks and that whoever reads y adds to every row (forward_to
+                 is then told so with late_bias_taken=True)
+  feed_forward   forward(h[T, dim], x_f32[T, dim], ctx): adds its output to x; optional: forward_to(h, y_f32, ctx)
   block          forward(x_f32[T, dim], ctx, line, writes_cache): one layer on the residual stream;
                  optional: a `next_norm` argument (the norm that reads the stream after this layer, whose
                  activations the layer may prepare) and first_norm() (the norm it applies first)
@@ -135,7 +138,7 @@ class Part:
         return type(self).__name__, False
 
     @staticmethod
-    def _gemm(ctx, a, w, out, epilogue, hidden=0, scale_from=None):
+    def _gemm(ctx, a, w, out, epilogue, hidden=0, scale_from=None, unit=None):
         """kernels.gemm with the scratch that lets small batches split K."""
         from ..ops import kernels
         import torch
@@ -143,7 +146,7 @@ class Part:
         n = kernels.gemm_workspace_floats(a.shape[0], w.shape[0], a.shape[1]) if a.dtype == torch.bfloat16 else 0
         if n and ctx is not None:
             ws = ctx.ws.get("gemm.partial", (n,), torch.float32)
-        return kernels.gemm(a, w, out, epilogue, hidden=hidden, workspace=ws, scale_from=scale_from)
+        return kernels.gemm(a, w, out, epilogue, hidden=hidden, workspace=ws, scale_from=scale_from, unit=unit)
 
     def _emit_args(self, emit_for, ctx, T, width):
         """Operands for a residual-add GEMM that also prepares the activations of the norm
@@ -193,3 +196,57 @@ class Part:
         """True if this part can take the float32 residual stream x and do `norm` itself
         (it then offers forward_prenorm in place of forward)."""
         return False
+
+
+class JoinableMixer(Part):
+    """A mixer of the form: one product in front, something in between, one product behind.  What such a mixer says:
+      n_in, in_rows(get)          the first product's matrix [n_in, dim] from the folder's tensors
+      n_out, out_columns(get)     the last product's matrix [dim, n_out]
+      load_rest(get, compute_dtype, device, scale=1.0)      everything else it loads; scale: what its result counts for
+      between(h, proj, o, ctx, line, writes_cache, scale=1.0)   fills o [T, n_out] (compute dtype) from proj [T, n_in] (float32)
+      late_bias                   the last product's bias, or None
+    Alone it runs its two products itself.  A mixer made of several (side_by_side) may set `joined` on those whose class
+    says `joinable`: it then makes one product of their first ones and one of their last ones, hands them their columns of
+    the wider rows, and they load no matrices of their own."""
+    joinable = False
+
+    def __init__(self, spec, dim, prefix):
+        super().__init__(spec, dim, prefix)
+        self.joined = False
+        self.share = 1.0                  # of a joined mixer in the common result
+        self.w_in = self.wo = None
+        self.late_bias = None
+
+    def load(self, get, compute_dtype, device):
+        from ..weights.loader import place
+        if not self.joined:
+            self.w_in = place(self.in_rows(get), compute_dtype, device)
+            self.wo = place(self.out_columns(get), compute_dtype, device)
+        self.load_rest(get, compute_dtype, device, self.share)
+
+    def weight_bytes(self):
+        return 0 if self.joined else (self.w_in.numel() + self.wo.numel()) * self.w_in.element_size()
+
+    def forward(self, h, x, ctx, line, writes_cache=True):
+        """Adds the mixer's result to the stream x."""
+        from ..ops import kernels
+        if self.late_bias is not None:
+            raise ValueError("a mixer whose last product has a bias writes its result (forward_to); it does not add to the stream")
+        return self._run(h, x, ctx, line, writes_cache, kernels.EPI_ADD_F32)
+
+    def forward_to(self, h, y, ctx, line, writes_cache=True, late_bias_taken=False):
+        """Writes the mixer's result to y (float32 [T, dim]), without its late_bias."""
+        from ..ops import kernels
+        if self.late_bias is not None and not late_bias_taken:
+            raise ValueError("this mixer's result lacks a bias that nobody adds")
+        return self._run(h, y, ctx, line, writes_cache, kernels.EPI_STORE_F32)
+
+    def _run(self, h, x, ctx, line, writes_cache, epilogue):
+        import torch
+        from ..ops import kernels
+        T = h.shape[0]
+        proj = ctx.ws.get("joinable.proj", (T, self.n_in), torch.float32)
+        self._gemm(ctx, h, self.w_in, proj, kernels.EPI_STORE_F32)
+        o = ctx.ws.get("joinable.o", (T, self.n_out), h.dtype)
+        self.between(h, proj, o, ctx, line, writes_cache)
+        self._gemm(ctx, o, self.wo, x, epilogue)

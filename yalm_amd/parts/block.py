@@ -183,6 +183,67 @@ class PostNormResidualBlock(Part):
             ctx.normed[id(next_norm)] = (hand_on, None, None)
 
 
+@part("block", "sandwich_residual")
+class SandwichResidualBlock(Part):
+    """x += mixer_out_norm(mixer(mixer_norm(x))); x += feed_forward_out_norm(feed_forward(feed_forward_norm(x))): a norm on
+    either side of every sublayer (a norm's own scale on what it adds is its parameter).  Members: mixer, mixer_norm,
+    mixer_out_norm, and optionally feed_forward with feed_forward_norm and feed_forward_out_norm.  The sublayers offer
+    forward_to; the norm behind a sublayer brings its result (and the bias it may lack) into the stream and, where it can,
+    leaves the output of the norm that reads the stream next: the feed-forward's, or next_norm."""
+
+    def __init__(self, layer_spec, dim, prefix=""):
+        super().__init__(None, dim, layer_spec.prefix)
+        p = layer_spec.prefix
+        self.mixer = build_part("mixer", layer_spec.mixer, dim, p)
+        self.mixer_norm = build_part("norm", layer_spec.mixer_norm, dim, p)
+        self.mixer_out_norm = build_part("norm", layer_spec.mixer_out_norm, dim, p)
+        self.feed_forward = self.feed_forward_norm = self.feed_forward_out_norm = None
+        if layer_spec.part("feed_forward") is not None:
+            self.feed_forward = build_part("feed_forward", layer_spec.feed_forward, dim, p)
+            self.feed_forward_norm = build_part("norm", layer_spec.feed_forward_norm, dim, p)
+            self.feed_forward_out_norm = build_part("norm", layer_spec.feed_forward_out_norm, dim, p)
+
+    def children(self):
+        return [c for c in (self.mixer_norm, self.mixer, self.mixer_out_norm, self.feed_forward_norm, self.feed_forward,
+                            self.feed_forward_out_norm) if c is not None]
+
+    def first_norm(self):
+        return self.mixer_norm
+
+    def forward(self, x, ctx, line, writes_cache=True, next_norm=None):
+        import torch
+        T = x.shape[0]
+        y = ctx.ws.get("block.y", (T, self.dim), torch.float32)
+        h = ctx.ws.get("block.h", (T, self.dim), ctx.act_dtype)
+        left = ctx.normed.pop(id(self.mixer_norm), None)
+        if left is None:
+            self.mixer_norm.forward(x, h, ctx)
+        else:                                             # the layer before has left this norm's output
+            h = left[0]
+        bias = getattr(self.mixer, "late_bias", None)
+        self.mixer.forward_to(h, y, ctx, line, writes_cache, **({} if bias is None else {"late_bias_taken": True}))
+        after = next_norm if self.feed_forward is None else self.feed_forward_norm
+        h = self._join(self.mixer_out_norm, y, x, ctx, after, bias)
+        if self.feed_forward is not None:
+            if h is None:
+                h = ctx.ws.get("block.h", (T, self.dim), ctx.act_dtype)
+                self.feed_forward_norm.forward(x, h, ctx)
+            self.feed_forward.forward_to(h, y, ctx)
+            h = self._join(self.feed_forward_out_norm, y, x, ctx, next_norm, None)
+        if h is not None:
+            ctx.normed[id(next_norm)] = (h, None, None)
+
+    def _join(self, norm, y, x, ctx, after, bias):
+        """The result y into the stream; returns the output of the norm `after` for the new stream, or None."""
+        kw = {} if bias is None else {"y_bias": bias}
+        if after is None or not norm.can_hand_to(after):
+            norm.join(y, x, ctx, **kw)
+            return None
+        h = ctx.ws.get("block.h", (x.shape[0], self.dim), ctx.act_dtype)      # the sublayer has read what it holds
+        norm.join(y, x, ctx, h_out=h, next_norm=after, **kw)
+        return h
+
+
 @part("block", "loop_entry")
 class LoopEntryBlock(Part):
     """The way into a walk of looped layers: x <- W [x; x0] + start, x0 being what the embedding left (it keeps a copy

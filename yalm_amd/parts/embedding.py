@@ -101,12 +101,16 @@ class TokenEmbedding(Part):
 
 @part("head", "lm_head")
 class LMHead(Part):
-    """logits = W h in float32; W is the embedding table when tied (src/infer.cpp:508-521)."""
+    """logits = W h in float32; W is the embedding table when tied (src/infer.cpp:508-521).  With `softcap` c every logit is
+    c tanh(logit / c)."""
 
     def __init__(self, spec, dim, prefix, embedding=None):
         super().__init__(spec, dim, prefix)
         self.vocab_size = int(spec.params["vocab_size"])
         self.tied = bool(spec.params.get("tied", False))
+        self.softcap = float(spec.params.get("softcap") or 0.0)
+        if self.softcap < 0.0:
+            raise ValueError("a cap on the logits is positive (0: none)")
         self.tensor = self.prefix + str(spec.params.get("tensor", "weight"))
         self.embedding = embedding
         self.weight = None
@@ -135,6 +139,12 @@ class LMHead(Part):
 
     def forward_prenorm(self, x, norm, logits, ctx):
         """logits for every row of x (no row selection)."""
+        return self._capped(self._product_prenorm(x, norm, logits, ctx))
+
+    def _capped(self, logits):
+        return kernels.softcap(logits, self.softcap) if self.softcap else logits
+
+    def _product_prenorm(self, x, norm, logits, ctx):
         src = ctx.normed.pop(id(norm), None)
         if src is not None and src[1] is None:            # the norm's output is ready
             return self._gemm(ctx, src[0], self.weight, logits, kernels.EPI_STORE_F32)
@@ -147,4 +157,4 @@ class LMHead(Part):
         return kernels.gemm_norm(x, nw, eps, self.weight, logits, kernels.EPI_STORE_F32)
 
     def forward(self, h, logits, ctx):
-        return self._gemm(ctx, h, self.weight, logits, kernels.EPI_STORE_F32)
+        return self._capped(self._gemm(ctx, h, self.weight, logits, kernels.EPI_STORE_F32))

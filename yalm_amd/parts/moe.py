@@ -9,8 +9,8 @@ make silu(gate) * up).  The part's result is the weighted sum over
 a token's chosen experts, in the order of their scores.  `unit` "relu2": experts of two matrices, out = W_down
 relu(W_up h)^2.  `scores` "sigmoid": s = sigmoid(W_router h); experts are chosen by s plus a correction (the tensor
 `correction`, one number an expert), among the `keep_groups` best of `groups` equal groups of neighbouring experts (a
-group's score is the sum of its two largest corrected scores), and weigh s over the sum of the chosen s, times
-`weight_scale`.  With `shared` = {hidden, prefix, gate} one more expert of the
+group's score is the sum of its two largest corrected scores, or with `group_score` "max" its largest), and weigh s over the sum
+of the chosen s, times `weight_scale`.  Softmax scores with `renormalize` take a correction, groups and weight_scale likewise.  With `shared` = {hidden, prefix, gate} one more expert of the
 same form (its tensors behind `prefix`, its own hidden size) runs for every token and is added, times sigmoid(w . h), one
 number a token (w: the tensor `gate` behind the prefix, [1, width]; no `gate`: added as it is).
 
@@ -64,8 +64,13 @@ class MixtureOfExperts(Part):
             raise ValueError("mixture of experts: %d of %d experts from %d of %d groups is not offered"
                              % (self.top, self.n_experts, self.keep_groups, self.groups))
         self.correction_name = self.names.get("correction")        # a tensor's name, or no correction
-        if not self.sigmoid and (self.groups > 1 or self.weight_scale != 1.0 or self.correction_name):
-            raise ValueError("groups, a correction and weight_scale go with sigmoid scores")
+        if p.get("group_score", "top2") not in ("top2", "max"):
+            raise ValueError("mixture of experts: a group's score %r is neither 'top2' nor 'max'" % (p.get("group_score"),))
+        self.group_max = p.get("group_score", "top2") == "max"
+        # whether the choice is made by corrected scores inside groups (a kernel of its own)
+        self.corrected = self.sigmoid or self.groups > 1 or self.weight_scale != 1.0 or bool(self.correction_name)
+        if self.corrected and not self.sigmoid and (self.renormalize is not True or self.router_bias):
+            raise ValueError("groups, a correction and weight_scale go with sigmoid scores, or with softmax scores brought to one sum")
         if self.sigmoid and (self.renormalize or self.router_bias):
             raise ValueError("sigmoid scores are always brought to one sum and take no router bias")
         self.correction = None
@@ -155,8 +160,9 @@ class MixtureOfExperts(Part):
         wts = ws.get("moe.weights", (T, self.top), torch.float32)
         logits = ws.get("moe.logits", (T, self.n_experts), torch.float32)        # products exact, sums in float32
         self._gemm(ctx, h, self.w_router, logits, kernels.EPI_STORE_F32)
-        if self.sigmoid:
-            kernels.moe_select_groups(logits, self.correction, ids, wts, self.groups, self.keep_groups, self.weight_scale)
+        if self.corrected:
+            kernels.moe_select_groups(logits, self.correction, ids, wts, self.groups, self.keep_groups, self.weight_scale,
+                                      softmax=not self.sigmoid, group_max=self.group_max)
         else:
             kernels.moe_select(logits, ids, wts, self.renormalize, bias=self.b_router)
         if T >= GROUPED_MIN_ROWS and kernels.can_moe_grouped(self.dim, self.hidden, h.dtype, T * self.top, self.n_experts):

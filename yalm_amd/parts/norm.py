@@ -6,7 +6,11 @@ the norm of a layer that norms a sublayer's OUTPUT: x += norm(y).
 
 LayerNorm: out = (x - mean) / sqrt(mean of the squared deviations + eps) * weight + bias, everything in float32; the bias is
 the tensor of the weight's name with `bias_suffix` (default ".b") behind it.  Its `join` norms the SUM of the stream,
-times `stream_scale` (default 1), and the sublayer's result: x = norm(stream_scale x + y)."""
+times `stream_scale` (default 1), and the sublayer's result: x = norm(stream_scale x + y).
+
+DynamicTanh stands in a norm's place and forms no mean: out = tanh(alpha x) * weight + bias, everything in float32; alpha is one
+number, the tensor of the weight's name with `alpha_suffix` (default ".alpha") behind it, the bias as LayerNorm's.  Its `join`
+adds the squashed result of a sublayer, times `result_scale` (default 1): x += result_scale norm(y)."""
 import torch
 
 from ..ops import kernels
@@ -88,3 +92,41 @@ class LayerNorm(Part):
     def can_hand_to(self, next_norm):
         """True if `join` can apply next_norm to the stream it leaves."""
         return hasattr(next_norm, "joined")
+
+
+@part("norm", "dynamic_tanh")
+class DynamicTanh(Part):
+    def __init__(self, spec, dim, prefix):
+        super().__init__(spec, dim, prefix)
+        self.tensor = self.prefix + str(spec.params.get("tensor", "weight"))
+        self.bias_tensor = self.tensor + str(spec.params.get("bias_suffix", ".b"))
+        self.alpha_tensor = self.tensor + str(spec.params.get("alpha_suffix", ".alpha"))
+        self.result_scale = float(spec.params.get("result_scale", 1.0))
+        self.weight = self.bias = self.alpha = None
+
+    def param_specs(self):
+        return [ParamSpec(self.tensor, (self.dim,), init="norm"), ParamSpec(self.bias_tensor, (self.dim,), init="bias"),
+                ParamSpec(self.alpha_tensor, (), init="fraction")]
+
+    def load(self, get, compute_dtype, device):
+        self.weight, self.bias = (get(n).to(torch.float32).to(device).contiguous() for n in (self.tensor, self.bias_tensor))
+        self.alpha = float(get(self.alpha_tensor))
+
+    def weight_bytes(self):
+        return 2 * self.dim * 4
+
+    def squash(self):
+        """(alpha, weight, bias) for a norm whose `join` applies this one to the stream it leaves."""
+        return self.alpha, self.weight, self.bias
+
+    def forward(self, x, out, ctx, row_index=None):
+        return kernels.squash(x, *self.squash(), out, row_index)
+
+    def join(self, y, x, ctx, h_out=None, next_norm=None, y_bias=None):
+        """x += result_scale norm(y + y_bias) (x, y float32 [T, dim]; y_bias float32 [dim] or None); h_out, if given, receives the
+        new x in the compute dtype, or with next_norm (a DynamicTanh) that norm's output for the new x."""
+        return kernels.squash_add(y, *self.squash(), self.result_scale, x, h_out, None if next_norm is None else next_norm.squash(), y_bias)
+
+    def can_hand_to(self, next_norm):
+        """True if `join` can apply next_norm to the stream it leaves."""
+        return hasattr(next_norm, "squash")

@@ -15,7 +15,9 @@ heads); `values` "keys": no value projection, a head's values are its keys as pr
 that is a rotation (kind "rope": behind the norms, the first rotary_dim elements of every query and key head are
 turned; the projections' rows and the norms' weights are brought into the kernel's order of pairs at load);
 `log_distance`: two numbers a head (tensors), a and b, take a ln(1 + b (i - j)) off the score of query i and key j,
-behind the cap; `gate`: the heads' results are multiplied by sigmoid(W_g h) before the output projection.
+behind the cap; `gate` true or "elements": the heads' results are multiplied by sigmoid(W_g h) before the output projection;
+"heads": a head's result by one number, W_g having a row a head (its rows then stand behind q, k and v in the first product);
+`out_bias`: the output projection has a bias, which is left to whoever takes the result (late_bias).
 forward_to writes the mixer's result instead of adding it to the stream.
 
 The cache and the attention kernels are the library's grouped-query ones: a head is stored `pad` elements wide
@@ -29,7 +31,7 @@ from ..cache.manager import KVRequest
 from ..ops import kernels
 from ..weights.loader import ParamSpec, place
 from .attention import decode_splits, kv_tiles
-from .base import Part, build_part, part
+from .base import JoinableMixer, build_part, part
 
 # A prompt step of at least this many tokens leaves its values row by row and transposes them a tile of 64 tokens at a
 # time (whole lines into the staging tiles and pages instead of two bytes a token and element)
@@ -38,11 +40,11 @@ V_TILES_MIN_TOKENS = 64
 NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "out": "o_proj.weight",
          "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "q_norm": "q_norm.weight",
          "k_norm": "k_norm.weight", "sink": "sink", "blend": "value_blend", "gate": "g_proj.weight", "log_a": "log_a",
-         "log_b": "log_b"}
+         "log_b": "log_b", "out_bias": "o_proj.bias"}
 
 
 @part("mixer", "shaped_attention")
-class ShapedAttention(Part):
+class ShapedAttention(JoinableMixer):
     prompt_tables = (kv_tiles,)
 
     def __init__(self, spec, dim, prefix):
@@ -64,7 +66,10 @@ class ShapedAttention(Part):
         self.values_from_keys = p.get("values", "own") == "keys"
         if p.get("values", "own") not in ("own", "keys"):
             raise ValueError("values %r are neither 'own' nor 'keys'" % (p.get("values"),))
-        self.has_gate = bool(p.get("gate", False))
+        self.gate = {False: None, None: None, True: "elements"}.get(p.get("gate"), p.get("gate"))
+        if self.gate not in (None, "elements", "heads"):
+            raise ValueError("an output gate %r is neither 'elements' nor 'heads'" % (p.get("gate"),))
+        self.has_out_bias = bool(p.get("out_bias", False))
         self.has_log_distance = bool(p.get("log_distance", False))
         self.eps = float(p.get("eps", 1e-6))
         self.biases = bool(p.get("biases", False))
@@ -84,7 +89,9 @@ class ShapedAttention(Part):
         if self.pad > kernels.MAX_HEAD_DIM:
             raise ValueError("heads of %d are not supported (at most %d)" % (self.pad, kernels.MAX_HEAD_DIM))
         self.q_dim, self.k_dim, self.v_dim = self.n_heads * self.key_dim, self.n_kv_heads * self.key_dim, self.n_kv_heads * self.value_dim
-        self.n_proj = self.q_dim + self.k_dim + (0 if self.values_from_keys else self.v_dim)      # a token's row of the first product
+        self.n_proj = self.q_dim + self.k_dim + (0 if self.values_from_keys else self.v_dim)      # what the packing kernel reads of a token's row
+        self.gate_rows = (self.n_heads + 3) // 4 * 4 if self.gate == "heads" else 0               # behind it, zero rows up to whole fours
+        self.joinable = self.gate == "heads"      # the gate's kernel brings the result to its place in a wider row
         if (self.q_dim + self.k_dim + self.v_dim) * 4 > 64 * 1024:
             raise ValueError("a token's queries, keys and values (%d numbers) are more than the packing kernel holds"
                              % (self.q_dim + self.k_dim + self.v_dim))
@@ -94,7 +101,7 @@ class ShapedAttention(Part):
         self.rot_dims = int(getattr(self.position, "rotary_dim", 0) or 0)
         if self.rot_dims > self.key_dim:
             raise ValueError("%d turned elements do not fit key heads of %d" % (self.rot_dims, self.key_dim))
-        self.wqkv = self.wo = self.bias = self.w_qn = self.w_kn = self.sink = self.lam = self.wg = self.log_ab = None
+        self.bias = self.w_qn = self.w_kn = self.sink = self.lam = self.wg = self.log_ab = None
 
     def children(self):
         return [self.position] if self.position is not None else []
@@ -108,8 +115,10 @@ class ShapedAttention(Part):
                ParamSpec(self._n("out"), (D, self.n_heads * self.value_dim), fan_in=self.n_heads * self.value_dim)]
         if not self.values_from_keys:
             out.append(ParamSpec(self._n("v"), (self.v_dim, D), fan_in=D))
-        if self.has_gate:
-            out.append(ParamSpec(self._n("gate"), (self.n_heads * self.value_dim, D), fan_in=D))
+        if self.gate:
+            out.append(ParamSpec(self._n("gate"), (self.n_heads * (self.value_dim if self.gate == "elements" else 1), D), fan_in=D))
+        if self.has_out_bias:
+            out.append(ParamSpec(self._n("out_bias"), (D,), init="bias"))
         if self.head_norm:
             out += [ParamSpec(self._n("q_norm"), (self.key_dim,), init="norm"), ParamSpec(self._n("k_norm"), (self.key_dim,), init="norm")]
         if self.has_log_distance:
@@ -126,26 +135,46 @@ class ShapedAttention(Part):
             out.append(ParamSpec(self._n("blend"), (), init="fraction"))
         return out
 
-    def load(self, get, compute_dtype, device):
-        def f32(key):
-            return get(self._n(key)).to(torch.float32).reshape(-1).to(device).contiguous()
-        def paired(t, n_heads):            # rows (or a norm's weights) in the order in which the rotation kernel pairs them
-            if not self.rot_dims:
-                return t
-            flat = t.dim() == 1
-            out = self.position.arrange_projection_rows(t.reshape(n_heads * self.key_dim, -1), n_heads)
-            return out.reshape(-1) if flat else out
-        rows = [paired(get(self._n("q")), self.n_heads), paired(get(self._n("k")), self.n_kv_heads)]
+    @property
+    def n_in(self):
+        return self.n_proj + self.gate_rows
+
+    @property
+    def n_out(self):
+        return self.n_heads * self.pad
+
+    def _paired(self, t, n_heads):
+        """Rows (or a norm's weights) in the order in which the rotation kernel pairs them."""
+        if not self.rot_dims:
+            return t
+        flat = t.dim() == 1
+        out = self.position.arrange_projection_rows(t.reshape(n_heads * self.key_dim, -1), n_heads)
+        return out.reshape(-1) if flat else out
+
+    def in_rows(self, get):
+        rows = [self._paired(get(self._n("q")), self.n_heads), self._paired(get(self._n("k")), self.n_kv_heads)]
         if not self.values_from_keys:
             rows.append(get(self._n("v")))
-        self.wqkv = place(torch.cat(rows, dim=0), compute_dtype, device)
-        self.wg = place(get(self._n("gate")), compute_dtype, device) if self.has_gate else None
+        if self.gate == "heads":
+            g = get(self._n("gate"))
+            rows += [g, g.new_zeros((self.gate_rows - self.n_heads, self.dim))]
+        return torch.cat(rows, dim=0)
+
+    def out_columns(self, get):
         wo = get(self._n("out"))
         if self.pad != self.value_dim:                    # the attention's result is `pad` wide a head, zeros behind
-            spread = torch.zeros((self.dim, self.n_heads, self.pad), dtype=wo.dtype)
+            spread = wo.new_zeros((self.dim, self.n_heads, self.pad))
             spread[:, :, :self.value_dim] = wo.reshape(self.dim, self.n_heads, self.value_dim)
             wo = spread.reshape(self.dim, self.n_heads * self.pad)
-        self.wo = place(wo, compute_dtype, device)
+        return wo
+
+    def load_rest(self, get, compute_dtype, device, scale=1.0):
+        paired = self._paired
+
+        def f32(key):
+            return get(self._n(key)).to(torch.float32).reshape(-1).to(device).contiguous()
+        self.wg = place(get(self._n("gate")), compute_dtype, device) if self.gate == "elements" else None
+        self.late_bias = f32("out_bias") * scale if self.has_out_bias else None
         self.bias = None
         if self.biases:
             b = [paired(get(self._n("q_bias")).reshape(-1), self.n_heads), paired(get(self._n("k_bias")).reshape(-1), self.n_kv_heads)]
@@ -164,7 +193,7 @@ class ShapedAttention(Part):
         self.lam = f32("blend") if self.value_blend == "later" else None
 
     def weight_bytes(self):
-        return (self.wqkv.numel() + self.wo.numel() + (self.wg.numel() if self.wg is not None else 0)) * self.wqkv.element_size()
+        return super().weight_bytes() + (self.wg.numel() * self.wg.element_size() if self.wg is not None else 0)
 
     def cache_request(self):
         # a query inside a block sees fewer than `block` keys back: the ring of a window of that width holds them
@@ -172,7 +201,7 @@ class ShapedAttention(Part):
         return KVRequest(self.n_kv_heads, self.pad, reach, 0)
 
     def row_elements(self):
-        return max(self.q_dim + self.k_dim + self.v_dim, self.n_heads * self.pad)
+        return max(self.q_dim + self.k_dim + self.v_dim + self.gate_rows, self.n_heads * self.pad)
 
     def describe(self, compute_dtype):
         what = "shaped attention, %d heads in %d groups, keys of %d and values of %d in heads of %d%s" % (
@@ -180,10 +209,16 @@ class ShapedAttention(Part):
             (", window %d" % self.window if self.window else "") + (", blocks of %d" % self.block if self.block else ""))
         if compute_dtype != torch.bfloat16:
             return what + ": float32-arithmetic kernels", False
-        if self.pad in kernels.MFMA_HEAD_DIMS:
+        if self.pad in kernels.MFMA_HEAD_DIMS or (self.pad in kernels.MFMA_WIDE_HEAD_DIMS and not self.shaped_scores):
             return what + ": matrix-core kernels", False
         return what + ": float32-arithmetic kernels on bfloat16 storage (the matrix-core kernels take head sizes " \
-                      "of 16 to 128 in steps of 16, not %d): correct, several times slower" % self.pad, True
+                      "of 16 to 256 in steps of 16, to 128 where the scores have a shape, not %d): correct, several times slower" % self.pad, True
+
+    @property
+    def shaped_scores(self):
+        """Whether the scores are more than scaled products (which the wide heads' kernels do not take)."""
+        return bool(self.softcap or self.block or self.has_sink or self.has_log_distance
+                    or hasattr(self.position, "score_bias") or hasattr(self.position, "slopes"))
 
     @property
     def score_bias(self):
@@ -193,24 +228,16 @@ class ShapedAttention(Part):
     def slopes(self):
         return getattr(self.position, "slopes", None)
 
-    def forward(self, h, x, ctx, line, writes_cache=True):
-        """Adds the mixer's result to the stream x."""
-        return self._run(h, x, ctx, line, writes_cache, kernels.EPI_ADD_F32)
-
-    def forward_to(self, h, y, ctx, line, writes_cache=True):
-        """Writes the mixer's result to y (float32 [T, dim])."""
-        return self._run(h, y, ctx, line, writes_cache, kernels.EPI_STORE_F32)
-
-    def _run(self, h, x, ctx, line, writes_cache, epilogue):
+    def between(self, h, proj, o, ctx, line, writes_cache, scale=1.0):
         T = h.shape[0]
+        joint = o                         # where the result belongs: maybe columns of a wider row
         act, ws = h.dtype, ctx.ws
         H, G, P = self.n_heads, self.n_kv_heads, self.pad
         if self.position is not None and ctx.max_position >= self.position.n_positions:
             raise ValueError("position %d is beyond the %d distances the score table holds"
                              % (ctx.max_position, self.position.n_positions))
         prefill = ctx.mode == "prefill"
-        qkv = ws.get("attn.qkv", (T, self.n_proj), torch.float32)
-        self._gemm(ctx, h, self.wqkv, qkv, kernels.EPI_STORE_F32)
+        qkv = proj[:, :self.n_proj]
         q = ws.get("attn.q", (T, H * P), act)
         group = ctx.cache.group_of(line)
         k_pages, v_pages = group.line_pages(line)
@@ -237,20 +264,22 @@ class ShapedAttention(Part):
         if v_rows is not None:
             kernels.v_tiles(v_rows, vst, v_pages if writes_cache else None, ctx.cu_seqlens, seq_tile0, group.table,
                             group.ring_pages, ctx.seq_slot, ctx.seq_len, G, P)
-        o = ws.get("attn.o", (T, H * P), act)
+        if not joint.is_contiguous():
+            o = ws.get("attn.o", (T, H * P), act)
         if prefill:
             kernels.attn_prefill(q, kst, vst, o, ctx.cu_seqlens, seq_tile0, ctx.tok_seq, ctx.tok_pos, H, G, P, self.window,
                                  tiles.get("tile_order"), score_bias=self.score_bias, softcap=self.softcap,
                                  sink_logit=self.sink, slopes=self.slopes, block=self.block, log_distance=self.log_ab)
         else:
-            n_splits = decode_splits(H, G, P, T, min(group.ring_pages, ctx.pages_bucket), ctx.ragged, shaped=True)
+            n_splits = decode_splits(H, G, P, T, min(group.ring_pages, ctx.pages_bucket), ctx.ragged, shaped=self.shaped_scores)
             partial = ws.get("attn.partial", (kernels.attn_decode_workspace_floats(T, H, P, n_splits),), torch.float32)
             kernels.attn_decode(q, k_pages, v_pages, group.table, group.ring_pages, ctx.seq_slot, ctx.seq_len, o, partial,
                                 H, G, P, self.window, n_splits, step_max_len=ctx.step_max_len, seq_order=ctx.seq_order,
                                 score_bias=self.score_bias, softcap=self.softcap, sink_logit=self.sink, slopes=self.slopes,
                                 block=self.block, log_distance=self.log_ab)
-        if self.has_gate:
+        if self.gate == "heads":
+            kernels.head_gate(o, proj[:, self.n_proj:self.n_proj + H], H, scale, joint)
+        elif self.gate == "elements":
             gates = ws.get("attn.gate", (T, H * self.value_dim), torch.float32)
             self._gemm(ctx, h, self.wg, gates, kernels.EPI_STORE_F32)
             kernels.sigmoid_gate(o, gates, H, self.value_dim, P)
-        self._gemm(ctx, o, self.wo, x, epilogue)

@@ -1,7 +1,8 @@
 """Gated feed-forward, dense: x += down( act(gate h) * (up h) )
 (src/infer.cpp:356-385 with one expert of weight 1).  act is silu(z) = z / (1 + exp(-z)) (SwiGLU) or, with the
 parameter `activation` = "gelu", gelu(z) = z/2 (1 + tanh(0.797885 (z + 0.044715 z^3))): the two the reference
-knows (src/infer.cpp:189-195, convert.py:51-52).
+knows (src/infer.cpp:189-195, convert.py:51-52).  With `limit` (silu only): g = min(gate h, limit), u = clamp(up h, -limit, limit) and the
+middle is g sigmoid(alpha g) (u + up_shift) (`alpha` and `up_shift` default to 1 and 0).
 Gate and up rows are interleaved in blocks of 16 at load so that one GEMM
 produces both and its epilogue multiplies them (the reference fuses the two
 products by pointer, src/infer.cu:610-634)."""
@@ -39,6 +40,10 @@ class SwiGLU(Part):
         if self.activation not in ACTIVATIONS:
             raise ValueError("feed-forward activation %r is not offered (%s)" % (self.activation, ", ".join(ACTIVATIONS)))
         self.gated = ACTIVATIONS[self.activation]          # the GEMM epilogue that applies it
+        unit = (float(spec.params.get("limit", 0.0) or 0.0), float(spec.params.get("alpha", 1.0)), float(spec.params.get("up_shift", 0.0)))
+        self.unit = None if unit == (0.0, 1.0, 0.0) else unit          # the epilogue's constants, where they are not silu's
+        if self.unit is not None and (self.activation != "silu" or unit[0] <= 0.0):
+            raise ValueError("feed-forward: alpha and up_shift go with silu and a positive limit")
         # the tensors' names behind the part's prefix (parameter `tensors`: {gate, up, down})
         self.names = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
         self.names.update(spec.params.get("tensors") or {})
@@ -63,7 +68,7 @@ class SwiGLU(Part):
         return self.hidden
 
     def fuses_norm(self, norm, x, ctx):
-        if not hasattr(norm, "fused") or ctx.mode not in ("decode", "prefill"):
+        if not hasattr(norm, "fused") or ctx.mode not in ("decode", "prefill") or self.unit is not None:
             return False
         T = x.shape[0]
         if ctx.mode == "prefill":             # takes the norm's output where the product before has left it
@@ -108,7 +113,15 @@ class SwiGLU(Part):
             self._gemm(ctx, mid, self.w_down, x, kernels.EPI_ADD_F32)
 
     def forward(self, h, x, ctx):
+        """Adds the result to x."""
+        return self._run(h, x, ctx, kernels.EPI_ADD_F32)
+
+    def forward_to(self, h, y, ctx):
+        """Writes the result to y (float32 [T, dim])."""
+        return self._run(h, y, ctx, kernels.EPI_STORE_F32)
+
+    def _run(self, h, x, ctx, epilogue):
         T = h.shape[0]
         mid = ctx.ws.get("ffn.hidden", (T, self.hidden), h.dtype)
-        self._gemm(ctx, h, self.w_gate_up, mid, self.gated, hidden=self.hidden)
-        self._gemm(ctx, mid, self.w_down, x, kernels.EPI_ADD_F32)
+        self._gemm(ctx, h, self.w_gate_up, mid, self.gated, hidden=self.hidden, unit=self.unit)
+        self._gemm(ctx, mid, self.w_down, x, epilogue)
