@@ -8,7 +8,7 @@ shape with its window of 4,096 positions and prompts of 6,000 tokens).
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers N] [--dtype bf16|fp32] [--shape NAME]
                     [--prompt-len N] [--prefill-len N] [--batch B] [--points B,B] [--no-prefill]
                     [--kernels] [--ragged] [--sweep]
-    python bench.py --design situlorn|gedunex|bovozen|rekirax|gemepel [--sizes 2048,4096] [--kernels] [--steps K] [--warmup W]
+    python bench.py --design situlorn|gedunex|bovozen|rekirax|gemepel|zebivik [--sizes 2048,4096] [--kernels] [--steps K] [--warmup W]
 
 --kernels adds the time of every kernel of a decode step and of a prompt step, each taken alone at the
 shape's sizes (src/test.cpp:340-405 times single kernels so), with its rate against the peak;
@@ -24,7 +24,9 @@ dense and mixture-of-experts feed-forwards) beside the Situlorn and the Llama la
 of the Rekirax design (three side-by-side mixers of a chunked rotary attention and HGRN2, one window attention, gated
 feed-forwards with biases, a way into looped layers) beside the Bovozen and the Llama layers, --design gemepel for four
 layers of the Gemepel design (two latent attentions with latent queries, one on the other's keys, two gated linear
-attentions, mixtures of two-matrix experts) beside the Situlorn, the Rekirax and the Llama layers, --design bovozen for four layers
+attentions, mixtures of two-matrix experts) beside the Situlorn, the Rekirax and the Llama layers, --design zebivik for four
+layers of the Zebivik design (two recurrent blocks, two side-by-side mixers of a rotary attention and a lightning attention, a
+clamped dense feed-forward and mixtures beside a shared expert) beside the Rekirax, the Gemepel and the Llama layers, --design bovozen for four layers
 of the Bovozen design (two gated delta rules, two attentions inside blocks of positions, a two-matrix feed-forward and
 mixtures of experts beside a shared expert) beside the Gedunex and the Llama layers.  The default workload and its
 line stay as they are.
@@ -121,8 +123,9 @@ KERNEL_FACES = ("embed", "rmsnorm", "gemm", "gemm_norm", "gemm_norm_qkv_rope", "
                 "latent_pack", "moe_route", "moe_select", "moe_pair_gate_up", "moe_pair_down", "moe_grouped", "embed_sinusoid",
                 "qkv_pack", "v_tiles", "mlstm_scan", "mlstm_chunks", "gated_delta", "embed_learned", "activate", "gated_add",
                 "time_conv", "gated_bias_act", "sigmoid_gate", "loop_pack", "hgrn2", "layer_norm", "layer_norm_sum", "embed_pairs",
-                "latent_norm", "moe_select_groups", "gla", "gla_tiles")
-FP32_FACES = ("mlstm_scan", "mlstm_chunks", "gated_delta", "hgrn2", "gla", "gla_tiles")     # kernels of float32 multiply-adds whatever the model's dtype: priced against that peak
+                "latent_norm", "moe_select_groups", "gla", "gla_tiles", "squash", "squash_add", "rms_gate", "head_gate", "softcap",
+                "lightning", "lightning_tiles", "lru", "lru_step")
+FP32_FACES = ("mlstm_scan", "mlstm_chunks", "gated_delta", "hgrn2", "gla", "gla_tiles", "lightning", "lightning_tiles")     # kernels of float32 multiply-adds whatever the model's dtype: priced against that peak
 
 
 def record_kernel_calls(run):
@@ -261,6 +264,33 @@ def kernel_cost(name, a, kw, kv_tokens, torch):
         T, B = proj.shape[0], seq_slot.shape[0]
         # per token and head: the decay, the rank-one write and the read-out, each over the d x dv state; the rest as for hgrn2
         return "gla %d tokens" % T, nbytes(proj, out) + 2 * nbytes(raw) + 2 * B * H * d * dv * 4, 5.0 * T * H * d * dv
+    if name == "lightning_tiles":
+        proj, raw, seq_slot, n_tiles = a[0], a[3], a[5], a[7]
+        H, d, dv = a[8], a[9], a[10]
+        T, B = proj.shape[0], seq_slot.shape[0]
+        return "lightning_tiles %d tokens" % T, nbytes(proj) + 4 * n_tiles * 64 * H * d * 4 + 3 * nbytes(raw) + 2 * B * H * d * dv * 4, \
+            T * H * (64.0 * (d + dv) + 4.0 * d * dv)
+    if name == "lightning":
+        proj, raw, seq_slot = a[0], a[3], a[5]
+        H, d, dv = a[6], a[7], a[8]
+        T, B = proj.shape[0], seq_slot.shape[0]
+        return "lightning %d tokens" % T, nbytes(proj, raw) + 2 * B * H * d * dv * 4, 5.0 * T * H * d * dv
+    if name in ("lru", "lru_step"):
+        u, w, z, out = a[0], a[1], a[4], a[7]
+        T, B = u.shape[0], (a[10] if name == "lru" else a[8]).shape[0]
+        # the two gates' products; the decays' products and the tiles' own states pass through memory once each way
+        return "%s %d tokens" % (name, T), nbytes(u, w, z, out) + (4 * nbytes(u) if name == "lru" else 0) + 8 * B * u.shape[1], \
+            4.0 * u.numel() * w.shape[-1]
+    if name == "squash":
+        return "squash %dx%d" % tuple(a[4].shape), a[4].numel() * 4 + nbytes(a[4]), 0.0
+    if name == "squash_add":
+        return "squash_add %dx%d" % tuple(a[0].shape), 3 * nbytes(a[0]) + (nbytes(a[6]) if len(a) > 6 and a[6] is not None else 0), 0.0
+    if name == "rms_gate":
+        return "rms_gate %dx%d" % tuple(a[0].shape), 2 * nbytes(a[0]) + nbytes(a[4]), 0.0
+    if name == "head_gate":
+        return "head_gate %dx%d" % tuple(a[0].shape), 2 * nbytes(a[0]) + a[1].numel() * 4, 0.0
+    if name == "softcap":
+        return "softcap %dx%d" % tuple(a[0].shape), 2 * nbytes(a[0]), 0.0
     if name == "time_conv":
         return "time_conv %dx%d" % tuple(a[0].shape), nbytes(a[0], a[3]), 0.0
     if name == "gated_bias_act":
@@ -434,6 +464,26 @@ def gemepel_config(width, n_layers=4):
             "layers": [pattern[i % 4] for i in range(n_layers)]}
 
 
+def zebivik_config(width, n_layers=4):
+    """Layers of the Zebivik design at a real model's sizes: recurrent blocks as wide as the model, in blocks of 256 channels
+    behind four taps; side-by-side mixers whose attention has heads of 128 in groups of four, turned whole, and whose linear
+    attention has heads of 128 x 128; a dense feed-forward of llama_config's size and mixtures of bovozen_config's experts, chosen
+    inside four of eight groups, beside a shared one."""
+    heads = width // 128
+    left = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+            "rot": {"dims": 128, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    right = {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 0.5 ** (1 + 9.0 * i / heads) for i in range(heads)]}
+    side = {"left": left, "right": right, "left_scale": 1.0, "right_scale": 1.0}
+    rec = {"width": width, "blocks": max(1, width // 256), "conv": 4}
+    dense = {"kind": "dense", "ff": width * 7 // 2, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "shared": {"ff": width // 2},
+           "router": {"experts": 32, "top": 4, "scale": 2.5, "groups": {"count": 8, "keep": 4}}}
+    pattern = [{"type": "rglru", "mixer": rec, "mlp": dense}, {"type": "parallel", "mixer": side, "mlp": moe},
+               {"type": "rglru", "mixer": rec, "mlp": moe}, {"type": "parallel", "mixer": side, "mlp": moe}]
+    return {"architecture": "Zebivik", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+            "logit_softcap": 30.0, "layers": [pattern[i % 4] for i in range(n_layers)]}
+
+
 def llama_config(width, n_layers=4):
     return {"architectures": ["LlamaForCausalLM"], "hidden_size": width, "intermediate_size": width * 7 // 2,
             "num_hidden_layers": n_layers, "num_attention_heads": width // 128, "num_key_value_heads": width // 512,
@@ -453,11 +503,12 @@ def bench_design(args):
     out = {}
     for width in [int(w) for w in args.sizes.split(",") if w]:
         own = {"gedunex": gedunex_config, "situlorn": situlorn_config, "bovozen": bovozen_config, "rekirax": rekirax_config,
-               "gemepel": gemepel_config}[args.design]
+               "gemepel": gemepel_config, "zebivik": zebivik_config}[args.design]
         own = (args.design, own(width))
         beside = {"gedunex": (("situlorn", situlorn_config(width)),), "bovozen": (("gedunex", gedunex_config(width)),),
                   "rekirax": (("bovozen", bovozen_config(width)),),
-                  "gemepel": (("situlorn", situlorn_config(width)), ("rekirax", rekirax_config(width)))}.get(args.design, ())
+                  "gemepel": (("situlorn", situlorn_config(width)), ("rekirax", rekirax_config(width))),
+                  "zebivik": (("rekirax", rekirax_config(width)), ("gemepel", gemepel_config(width)))}.get(args.design, ())
         for design, cfg in (own,) + beside + (("llama", llama_config(width)),):
             model = Model.random(cfg, seed=0, dtype=dtype, device="cuda:0")
             V = model.vocab_size
@@ -561,7 +612,7 @@ def main():
     ap.add_argument("--context", type=int, default=0,
                     help="the reference's -T: past this many positions two attention sinks and the last "
                          "<context> - 2 positions are attended to (0: the shape's own window, if any)")
-    ap.add_argument("--design", default="", choices=["", "situlorn", "gedunex", "bovozen", "rekirax", "gemepel"],
+    ap.add_argument("--design", default="", choices=["", "situlorn", "gedunex", "bovozen", "rekirax", "gemepel", "zebivik"],
                     help="measure layers of this design beside Llama layers of equal width instead of the default workload")
     ap.add_argument("--sizes", default="2048,4096", help="widths for --design")
     args = ap.parse_args()
