@@ -279,15 +279,18 @@ __global__ void sigmoid_gate_kernel(T* __restrict__ o, const float* __restrict__
 }
 
 // out[t, h, e] = o[t, h, e] * sigmoid(g[t * g_row + h]) * scale, e < dv (a gate of one number a head): rows of out are out_row
-// apart and may be o's own; a workgroup a token, or several where the tokens are few
-template <typename T>
-__global__ void head_gate_kernel(const T* __restrict__ o, const float* __restrict__ g, long g_row, float scale, T* __restrict__ out,
-                                 long out_row, int n_heads, int dv) {
-  const int t = blockIdx.x;
-  const T* src = o + (size_t)t * n_heads * dv;
-  T* dst = out + (size_t)t * out_row;
-  for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < n_heads * dv; i += gridDim.y * blockDim.x)
-    dst[i] = from_f32<T>(to_f32(src[i]) * (scale / (1.0f + expf(-g[(size_t)t * g_row + i / dv]))));
+// apart and may be o's own; a thread VEC neighbours of a head
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ o, const float* __restrict__ g, long g_row, float scale,
+                                                        T* __restrict__ out, long out_row, int n_heads, int dv) {
+  struct __attribute__((aligned(VEC * sizeof(T)))) V { T v[VEC]; };
+  const int t = blockIdx.x, i = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (i >= n_heads * dv) return;
+  const float f = scale / (1.0f + expf(-g[(size_t)t * g_row + i / dv]));
+  V x = *reinterpret_cast<const V*>(o + (size_t)t * n_heads * dv + i);
+#pragma unroll
+  for (int k = 0; k < VEC; ++k) x.v[k] = from_f32<T>(to_f32(x.v[k]) * f);
+  *reinterpret_cast<V*>(out + (size_t)t * out_row + i) = x;
 }
 
 // z[i] = cap tanh(z[i] / cap)
@@ -473,14 +476,21 @@ extern "C" int yalm_head_gate(const void* o, const float* g, long g_row, float s
   if (T <= 0) return YALM_OK;
   if (n_heads <= 0 || dv <= 0 || g_row < n_heads || out_row < (long)n_heads * dv || (o == out && T > 1 && out_row != (long)n_heads * dv))
     return YALM_ERR_ARG;
-  const int cols = n_heads * dv, slices = T >= 256 ? 1 : ceil_div(cols, 1024);
-  const dim3 grid(T, slices < 64 ? slices : 64);
-  if (dtype == YALM_F32)
-    head_gate_kernel<float><<<grid, 256, 0, stream>>>((const float*)o, g, g_row, scale, (float*)out, out_row, n_heads, dv);
-  else if (dtype == YALM_BF16)
-    head_gate_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)o, g, g_row, scale, (bf16*)out, out_row, n_heads, dv);
-  else
+  const int cols = n_heads * dv, bytes = dtype == YALM_F32 ? 4 : 2, wide = 16 / bytes;
+  if (ceil_div(cols, 256) > 65535) return YALM_ERR_ARG;
+  const bool vec = dv % wide == 0 && out_row % wide == 0 && ((((uintptr_t)o) | ((uintptr_t)out)) & 15) == 0;
+  const dim3 grid(T, ceil_div(cols, 256 * (vec ? wide : 1)));
+#define HG(T_, V_) head_gate_kernel<T_, V_><<<grid, 256, 0, stream>>>((const T_*)o, g, g_row, scale, (T_*)out, out_row, n_heads, dv)
+  if (dtype == YALM_F32) {
+    if (vec) HG(float, 4);
+    else HG(float, 1);
+  } else if (dtype == YALM_BF16) {
+    if (vec) HG(bf16, 8);
+    else HG(bf16, 1);
+  } else {
     return YALM_ERR_DTYPE;
+  }
+#undef HG
   return launch_status();
 }
 
