@@ -86,7 +86,7 @@ def test_declared_tensors():
     assert "l0.mix.left.out" not in shapes and "l0.mix.right.q.b" not in shapes
     assert shapes["l1.mix.y"] == (120, 80) and shapes["l1.mix.conv"] == (120, 4) and shapes["l1.mix.ra"] == (5, 24, 24)
     assert shapes["l1.mix.ri.b"] == (5, 24) and shapes["l1.mix.lam"] == (120,) and shapes["l1.mix.o"] == (80, 120)
-    assert shapes["l0.mlp.gate"] == (96, 80) and shapes["l1.mlp.correction"] == (12,) and shapes["l1.mlp.e11.down"] == (80, 48)
+    assert shapes["l0.mlp.gate"] == (96, 80) and shapes["l1.mlp.correction"] == (15,) and shapes["l1.mlp.e14.down"] == (80, 48)
     assert shapes["l1.mlp.shared.up"] == (40, 80) and "l3.mlp.shared.up" not in shapes
 
 
@@ -107,7 +107,7 @@ def test_declared_tensors():
     (lambda c: c["layers"][0]["mlp"].update(limit=0.0), "limit"),
     (lambda c: c["layers"][0]["mlp"].update(kind="mlp"), "neither"),
     (lambda c: c["layers"][1]["mlp"]["router"].update(top=7), "do not go together"),
-    (lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(count=5), "do not go together"),
+    (lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(count=4), "do not go together"),
     (lambda c: c["layers"][1]["mlp"]["shared"].update(ff=0), "do not go together"),
 ])
 def test_configurations_that_are_refused(change, message):

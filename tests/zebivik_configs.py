@@ -2,7 +2,7 @@
 heads alone and in groups, keys above and below values, heads turned whole, in part and not at all, with and without slowed
 frequencies, linear-attention heads of 3 to 150 channels under decays from 0 to 1, recurrent blocks wider and narrower than the
 model, in one block and in many (of one channel too), behind one to seven taps, dense and mixed feed-forwards, layers without one,
-one to four groups of experts (of one expert and of more) with some or all kept, top from one to all, with and without a shared
+one to eight groups of experts (of one expert and of more) with some or all kept, top from one to all, with and without a shared
 expert, with and without a cap on the logits, scales on either side of one."""
 import copy
 
@@ -55,7 +55,7 @@ def model(vocab, width, eps, mult, layers, softcap=None):
 
 MIXED = model(211, 80, 1e-6, 0.7, [
     layer(side(attention(6, 2, 24, 40, 0.2, dims=16, scaling=(4.0, 1.0, 4.0, 64)), lightning(12, 20, 0.3, 0.9, 0.999), 0.8, 1.3), dense(96, 0.6)),
-    layer(rglru(120, 5, 4), moe(12, 3, 48, 1.5, (4, 2), shared=40)),
+    layer(rglru(120, 5, 4), moe(15, 3, 48, 1.5, (5, 2), shared=40)),
     layer(rglru(48, 3, 2), None),
     layer(side(attention(3, 3, 32, 16, 0.31, base=500.0), lightning(40, 24, 0.97, 0.0), 1.4, 0.6), moe(6, 6, 24, 0.8)),
     layer(rglru(80, 1, 3), dense(56, 2.5)),
